@@ -18,7 +18,8 @@ prompt up front, cache/cache_manager.py:185-234): ``reserve(req, upto)``
 makes sure every group has pages for positions below ``upto``.
 ``commit(req, n)`` records that n tokens are computed and gives back, in
 windowed groups, each page j with (j+1)*page - 1 <= n - window: its newest key
-is out of sight of every query at position >= n.  In a chunked group (a query
+is out of sight of every query at position >= n; where a group keeps the first positions of a
+sequence beside the window, the pages that hold them stay.  In a chunked group (a query
 reads the keys of its own chunk of positions only) it gives back each page whose
 newest key lies before the chunk that position n belongs to.  ``release(req)`` gives
 everything back; a second call does nothing (double free is a no-op,
@@ -41,6 +42,7 @@ class GroupInfo:
     calls: List[int]               # entries of the execution order in this group
     num_pages: int = 0
     chunk: Optional[int] = None    # keys before the chunk of the next token are never read again
+    keep_first: int = 0            # beside a window: the first positions, which are never given back
 
     def first_needed(self, computed: int) -> int:
         """The first position that a query at position ``computed`` or later can still read."""
@@ -70,9 +72,10 @@ def group_needs(needs: Sequence[object]) -> List[GroupInfo]:
     for i, n in enumerate(needs):
         if isinstance(n, PagedKV):
             chunk = getattr(n, "chunk", None) if n.window is None else None
-            groups.setdefault((n.window, chunk), GroupInfo(n.window, [], chunk=chunk)).calls.append(i)
+            keep = int(getattr(n, "keep_first", 0) or 0) if n.window is not None else 0
+            groups.setdefault((n.window, chunk, keep), GroupInfo(n.window, [], chunk=chunk, keep_first=keep)).calls.append(i)
     # windowed groups first, by window; then chunked ones, by chunk; the all-keys group last
-    return sorted(groups.values(), key=lambda g: (g.window is None, g.window or 0, g.chunk is None, g.chunk or 0))
+    return sorted(groups.values(), key=lambda g: (g.window is None, g.window or 0, g.keep_first, g.chunk is None, g.chunk or 0))
 
 
 class CacheManager:
@@ -156,7 +159,8 @@ class CacheManager:
             out = []
             if info.releases:
                 t = r.tables[g]
-                j = r.first_live[g]
+                # pages that hold a kept first position stay
+                j = max(r.first_live[g], -(-info.keep_first // ps))
                 first = info.first_needed(computed)
                 while j < len(t) and (j + 1) * ps - 1 < first:
                     if t[j] >= 0:
@@ -239,6 +243,6 @@ class CacheManager:
 
     def stats(self) -> dict:
         return {"page_size": self.page_size,
-                "groups": [{"window": g.window, "chunk": g.chunk, "calls": len(g.calls), "pages": p.num_pages,
+                "groups": [{"window": g.window, "chunk": g.chunk, "keep_first": g.keep_first, "calls": len(g.calls), "pages": p.num_pages,
                             "free": p.free_pages} for g, p in zip(self.groups, self.pools)],
                 "live": len(self._reqs), "free_slots": self.slots.free_slots}

@@ -38,6 +38,7 @@ class LayerNormSpec:
     bias: Optional[str]
     streams: int = 1
     kind: str = "layernorm"
+    gain_scale: float = 1.0          # multiplies the gain (and the bias): a factor of whatever reads the norm linearly
 
 
 @dataclass(frozen=True)
@@ -52,6 +53,8 @@ class ShortConvSpec:
     activation: Optional[str] = None  # "silu": applied to the result
     channel_counts: Optional[Tuple[int, ...]] = None   # with several weight names: the channels of each
     bias: Optional[str] = None       # [size]: where the sum over the taps starts
+    in_bias: Any = None              # [size]: added to the rows before the taps see them (a projection's bias; rows
+    #                                  before a sequence's start stay zero): a name, or several stacked
 
 
 @dataclass(frozen=True)
@@ -111,6 +114,14 @@ class AttentionSpec:
     q_row_norm: Optional[str] = None         # gain [num_heads * head_dim] of an RMS norm over a token's whole query row
     #                                          (all heads at once, after the bias, before rotation; eps is norm_eps)
     k_row_norm: Optional[str] = None         # the same over the whole key row, gain [num_kv_heads * head_dim]
+    keep_first: int = 0                      # beside its window a query sees the sequence's first ``keep_first`` keys,
+    #                                          at their own positions (needs a window)
+    convs: Optional[Dict[str, str]] = None   # roles q, k, v -> [channels, conv_taps]: a causal convolution over time on
+    #                                          each channel right after the projections and their biases
+    conv_taps: int = 1
+    lend_values: bool = False                # the step's values (before any mixing) are lent to later layers
+    value_share: Optional[str] = None        # a number l: values are (1 - l) v + l v_lent, with the values that the
+    #                                          last lending layer lent for the same token; what is cached is the mix
     values_are_keys: bool = False            # no value projection: a value is its key as projected (with its bias,
     #                                          before norm and rotation); ``names`` and ``biases`` hold no role v
 
@@ -187,6 +198,22 @@ class DeltaRuleSpec:
 
 
 @dataclass(frozen=True)
+class GeneralDeltaSpec:
+    """The generalized delta rule: a matrix state per head [dim, dim] with a decay and a removal rate
+    per key channel, S <- diag(w) S - (a u)(u^T S) + k v^T with the unit key u = k / sqrt(sum k^2 +
+    1e-6), o = S^T r; w = exp(-exp(-1/2) sigmoid(W_w2 tanh(W_w1 x) + w0)), a = sigmoid(W_a x + b).
+    The read-out is divided by its root mean square per head, times a gain over all heads and
+    sigmoid(W_g x), then W_o.  The rank of W_w1 is read off the tensors where ``decay_rank`` is 0."""
+    hidden_size: int
+    num_heads: int
+    dim: int
+    decay_rank: int
+    eps: float                       # of the read-out's unit RMS
+    names: Dict[str, str]            # roles r, k, v, gate, a, a_bias, w1, w2, w0, norm, o
+    kind: str = "general_delta"
+
+
+@dataclass(frozen=True)
 class LinearAttentionSpec:
     """Gated linear attention: a matrix state per head that decays per key channel,
     S_t = diag(alpha_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, with q = W_q x key_dim^(-1/2) and
@@ -257,7 +284,8 @@ class GatedMLPSpec:
 
 @dataclass(frozen=True)
 class MLPSpec:
-    """act(x Wu^T), then Wd^T, without a gate.  ``activation``: "relu2" = max(z, 0)^2."""
+    """act(x Wu^T), then Wd^T, without a gate.  ``activation``: "relu2" = max(z, 0)^2, "gelu" =
+    z (1 + erf(z / sqrt(2))) / 2."""
     hidden_size: int
     intermediate_size: int
     activation: str
@@ -283,6 +311,12 @@ class RoutedMLPSpec:
     scale_input: bool = True
     kind: str = "routed_mlp"
     scoring: str = "sigmoid"         # or "softmax": scores exp(z) / sum over all experts
+    gated: bool = True               # False: an expert is act(x Wu^T) Wd^T with "relu2", and ``shared`` an MLPSpec
+    correction: Optional[str] = None    # [num_experts]: added to the scores for the choice, not for the weights
+    groups: Optional[Tuple[int, int]] = None    # (count, keep): equal runs of neighbouring experts, of which the ``keep``
+    #                                  with the largest sums of their two largest choice scores can be chosen from
+    normalise: bool = False          # the chosen scores are divided by their sum (+ 1e-20)
+    weight_scale: float = 1.0        # multiplies the weights
     shared_gate: Optional[str] = None   # [1, hidden]: the shared layer's result times sigmoid(W x), a number a token
 
 
@@ -323,6 +357,32 @@ class StreamsBlockSpec:
 
 
 @dataclass(frozen=True)
+class TokenSideSpec:
+    """A per-layer input that follows from the token itself: with e the columns [column, column + dim) of
+    the token's row of a table, h += rms(W_proj (gelu_tanh(W_gate h) * e)) * gain."""
+    dim: int
+    column: int
+    vocab_size: int
+    table_columns: int               # of the table, all layers' parts side by side
+    eps: float
+    names: Dict[str, str]            # roles table, gate, proj, norm
+
+
+@dataclass(frozen=True)
+class FilteredBlockSpec:
+    """A pre-norm layer, h += s1 * mixer(f1(norm1(h))); h += s2 * ffn(f2(norm2(h))), then the token's side
+    input.  f1, f2: short convolutions over time between norm and sublayer (None: nothing); s1, s2: a
+    gain per channel on each sublayer's result (None: 1)."""
+    mixer: Any
+    ffn: Any                         # None: the layer has no second sublayer
+    norms: Dict[str, Any]            # pre_mixer, pre_ffn: layer norms
+    filters: Dict[str, Any]          # pre_mixer, pre_ffn -> ShortConvSpec (missing: none)
+    scales: Dict[str, str]           # mixer, ffn -> names of [hidden] tensors (missing: none)
+    side: Optional[TokenSideSpec] = None
+    kind: str = "filtered"
+
+
+@dataclass(frozen=True)
 class PairTableSpec:
     """A table of token pairs whose row (previous token * mul_prev + token * mul_cur) mod buckets is
     added to the embedded row; a sequence's first token takes row ``buckets`` (the table's last).
@@ -342,6 +402,7 @@ class EmbeddingSpec:
     kind: str = "embedding"
     copies: int = 1                  # the row is written this many times (one per residual stream)
     pairs: Optional[PairTableSpec] = None
+    norm: Any = None                 # a layer norm of the embedded row; the stream begins with its result, in floats
 
 
 @dataclass(frozen=True)

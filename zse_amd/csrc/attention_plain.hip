@@ -7,7 +7,8 @@
 //
 // With ``chunk`` instead of a window, lo = floor(pos / chunk) * chunk: a query sees the keys of
 // its own chunk of positions, counted from position 0.  ``unit_sink``: a sink of score 0 that has
-// no value joins the denominator, exp(s_j) / (1 + sum exp(s)).
+// no value joins the denominator, exp(s_j) / (1 + sum exp(s)).  ``keep``: beside its window a query
+// sees the sequence's first ``keep`` keys, at their own positions.
 //
 // Keys are visited in tiles of 64 aligned to absolute positions, with a
 // running maximum and sum, so the order of every sum depends on the token's
@@ -30,7 +31,7 @@ __global__ __launch_bounds__(64) void attention_plain_kernel(
     const int* __restrict__ req_of_token, const int* __restrict__ positions,
     act_t* __restrict__ out, int nh, int nkv, int hd, int vd, int bs, float scale, float softcap,
     int window, int v_transposed, const float* __restrict__ v_freq, int v_interleaved,
-    const float* __restrict__ sinks, int v_in_k, int chunk, int unit_sink) {
+    const float* __restrict__ sinks, int v_in_k, int chunk, int unit_sink, int keep) {
   __shared__ float sq[MAXD];
   __shared__ float sp[64];
   __shared__ int spage[64];
@@ -51,9 +52,11 @@ __global__ __launch_bounds__(64) void attention_plain_kernel(
 
   float m = -INFINITY, l = 0.f;
   float acc[MAXD / 64] = {};
-  for (int j0 = (lo / 64) * 64; j0 <= pos; j0 += 64) {
+  // tiles of the kept first keys, then those from the window's first key on
+  const int lo_tile = lo / 64 * 64, kept_tiles = (keep + 63) / 64 * 64;
+  for (int j0 = keep > 0 ? 0 : lo_tile; j0 <= pos; j0 = (j0 + 64 >= kept_tiles && j0 + 64 < lo_tile) ? lo_tile : j0 + 64) {
     const int j = j0 + lane;
-    const bool valid = j >= lo && j <= pos;
+    const bool valid = (j >= lo || j < keep) && j <= pos;
     float s = -INFINITY;
     int page = -1;
     if (valid) {
@@ -139,12 +142,14 @@ __global__ __launch_bounds__(64) void attention_plain_kernel(
 // sinks (may be null): float [nh].  v_in_k: values are the first vd channels of the keys.
 // chunk > 0 (without a window): a query sees the keys of its own chunk of positions only.
 // unit_sink: a sink of score 0 joins every head's denominator (not together with sinks).
-extern "C" int zk_attention_plain_masked(const void* q, int q_stride, const void* kcache, const void* vcache,
+// keep > 0 (with a window): a query sees the sequence's first ``keep`` keys beside its window.
+extern "C" int zk_attention_plain_kept(const void* q, int q_stride, const void* kcache, const void* vcache,
                                          const int* block_table, int max_blocks, const int* req_of_token,
                                          const int* positions, void* out, int T, int nh, int nkv, int hd, int vd,
                                          int bs, float scale, float softcap, int window, int v_transposed,
                                          const float* v_freq, int v_interleaved, const float* sinks, int v_in_k,
-                                         int chunk, int unit_sink, void* stream) {
+                                         int chunk, int unit_sink, int keep, void* stream) {
+  ZK_REQUIRE(keep >= 0 && (keep == 0 || window > 0), "zk_attention_plain: first keys are kept beside a window");
   ZK_REQUIRE(chunk >= 0 && (chunk == 0 || window <= 0), "zk_attention_plain: a chunk or a window, not both");
   ZK_REQUIRE(!unit_sink || sinks == nullptr, "zk_attention_plain: a unit sink or learned sinks, not both");
   ZK_REQUIRE(T >= 0 && nh > 0 && nkv > 0 && hd > 0 && vd > 0 && bs > 0 && max_blocks > 0,
@@ -161,13 +166,24 @@ extern "C" int zk_attention_plain_masked(const void* q, int q_stride, const void
     attention_plain_kernel<AP_MAX_HD><<<grid, 64, 0, (hipStream_t)stream>>>(
         (const act_t*)q, q_stride, (const act_t*)kcache, (const act_t*)vcache, block_table, max_blocks,
         req_of_token, positions, (act_t*)out, nh, nkv, hd, vd, bs, scale, softcap, window, v_transposed, v_freq,
-        v_interleaved, sinks, v_in_k, chunk, unit_sink);
+        v_interleaved, sinks, v_in_k, chunk, unit_sink, keep);
   else
     attention_plain_kernel<1024><<<grid, 64, 0, (hipStream_t)stream>>>(
         (const act_t*)q, q_stride, (const act_t*)kcache, (const act_t*)vcache, block_table, max_blocks,
         req_of_token, positions, (act_t*)out, nh, nkv, hd, vd, bs, scale, softcap, window, v_transposed, v_freq,
-        v_interleaved, sinks, v_in_k, chunk, unit_sink);
+        v_interleaved, sinks, v_in_k, chunk, unit_sink, keep);
   return zk_launch_status("zk_attention_plain");
+}
+
+extern "C" int zk_attention_plain_masked(const void* q, int q_stride, const void* kcache, const void* vcache,
+                                         const int* block_table, int max_blocks, const int* req_of_token,
+                                         const int* positions, void* out, int T, int nh, int nkv, int hd, int vd,
+                                         int bs, float scale, float softcap, int window, int v_transposed,
+                                         const float* v_freq, int v_interleaved, const float* sinks, int v_in_k,
+                                         int chunk, int unit_sink, void* stream) {
+  return zk_attention_plain_kept(q, q_stride, kcache, vcache, block_table, max_blocks, req_of_token, positions, out, T,
+                                 nh, nkv, hd, vd, bs, scale, softcap, window, v_transposed, v_freq, v_interleaved,
+                                 sinks, v_in_k, chunk, unit_sink, 0, stream);
 }
 
 extern "C" int zk_attention_plain_sink(const void* q, int q_stride, const void* kcache, const void* vcache,
@@ -209,6 +225,9 @@ static const int attention_plain_sink_entered = zk_steplist_register(
 static const int attention_plain_masked_entered = zk_steplist_register(
     "zk_attention_plain_masked", zk_packed::Call<zk_attention_plain_masked>::nargs,
     (void*)zk_packed::Call<zk_attention_plain_masked>::call);
+static const int attention_plain_kept_entered = zk_steplist_register(
+    "zk_attention_plain_kept", zk_packed::Call<zk_attention_plain_kept>::nargs,
+    (void*)zk_packed::Call<zk_attention_plain_kept>::call);
 static const int attention_plain_ext_entered = zk_steplist_register(
     "zk_attention_plain_ext", zk_packed::Call<zk_attention_plain_ext>::nargs,
     (void*)zk_packed::Call<zk_attention_plain_ext>::call);

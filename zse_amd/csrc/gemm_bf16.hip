@@ -53,7 +53,8 @@ typedef float f32x16 __attribute__((ext_vector_type(16)));
 // <= 0: none) and that value's column in ``partials`` [M][strips] as (float, int), larger value
 // first, equal values to the lower column, NaN never, which a joining kernel reduces to one
 // column a row: the greedy choice without the logits ever reaching memory.
-enum { EPI_NONE = 0, EPI_SOFTCAP = 1, EPI_GELU_TANH = 2, EPI_SILU = 3, EPI_PICK = 4, EPI_RELU = 5, EPI_CLAMPED = 6, EPI_RELU2 = 7 };
+enum { EPI_NONE = 0, EPI_SOFTCAP = 1, EPI_GELU_TANH = 2, EPI_SILU = 3, EPI_PICK = 4, EPI_RELU = 5, EPI_CLAMPED = 6, EPI_RELU2 = 7,
+       EPI_GELU = 8 };
 
 struct Pick {
   float value;
@@ -88,13 +89,14 @@ __device__ __forceinline__ Pick pick_of_strip(const float (&x)[4], int n, int N,
 }
 
 // What a plain (not gated) product does to a sum before it is stored: the soft cap, the square of
-// relu, or nothing.
+// relu, the gelu with the error function, or nothing.
 __device__ __forceinline__ float epi_unary(float x, int epi, float cap) {
   if (epi == EPI_SOFTCAP) return cap * tanhf(x / cap);
   if (epi == EPI_RELU2) {
     const float r = fmaxf(x, 0.f);
     return r * r;
   }
+  if (epi == EPI_GELU) return 0.5f * x * (1.0f + erff(x * 0.7071067811865476f));
   return x;
 }
 
@@ -873,7 +875,7 @@ __global__ __launch_bounds__(256) void gemm_tile_join_kernel(
     // time, half a line's bytes from one wave and the other half from another).  The block's
     // 256 threads are (b, lr, j) here; the sums are the same, in the same order.
     const int m0 = tm * BM + (wave / NWN) * (32 * WMT) + i * 32, n0 = tn * BN + (wave % NWN) * 64;
-    if (!c_is_f32 && (epi == EPI_NONE || epi == EPI_RELU2) && ldc % 8 == 0 && (uintptr_t)C % 16 == 0 && m0 + 32 <= M && n0 + 64 <= N) {
+    if (!c_is_f32 && (epi == EPI_NONE || epi == EPI_RELU2 || epi == EPI_GELU) && ldc % 8 == 0 && (uintptr_t)C % 16 == 0 && m0 + 32 <= M && n0 + 64 <= N) {
       const int lr = lane & 31, j = lane >> 5;
       const f32x4* at = partials + ((size_t)tile * ksplit * NW + wave) * per_wave + ((size_t)(i * 2 + j) * 64 + lr) * 4 + b;
       f32x4 lo = at[0], hi = at[32 * 4];
@@ -1440,7 +1442,7 @@ static int gemm_bf16_run(const void* A, int lda, const void* W, void* C, int ldc
   ZK_REQUIRE(M >= 0 && N > 0 && K > 0, "zk_gemm_bf16: bad sizes");
   ZK_REQUIRE(K % 8 == 0 && lda % 8 == 0, "zk_gemm_bf16: K and lda must be multiples of 8");
   ZK_REQUIRE(lda >= K && ldc >= N, "zk_gemm_bf16: leading dimensions too small");
-  ZK_REQUIRE(epi >= 0 && epi <= EPI_RELU2, "zk_gemm_bf16: unknown epilogue");
+  ZK_REQUIRE(epi >= 0 && epi <= EPI_GELU, "zk_gemm_bf16: unknown epilogue");
   ZK_REQUIRE((epi != EPI_SOFTCAP && epi != EPI_CLAMPED) || cap > 0.f, "zk_gemm_bf16: soft cap or clamp limit must be positive");
   ZK_REQUIRE(((uintptr_t)A % 16 == 0) && ((uintptr_t)W % 16 == 0), "zk_gemm_bf16: operands must be 16-byte aligned");
   const bool gated = epi == EPI_GELU_TANH || epi == EPI_SILU || epi == EPI_RELU || epi == EPI_CLAMPED;

@@ -6,6 +6,10 @@
 //   q_h <- rot_p( q_h / sqrt(mean(q_h^2) + eps) * gq ) * c_h          (k likewise with gk, no c)
 //   v_g <- rot'_p( v_g )
 //
+// The values may be lent to a later layer (their rows after the bias are written to a buffer too)
+// or mixed with values that an earlier layer lent: v <- (1 - l) v + l v_lent with a number l of the
+// layer, before their rotation and store.
+//
 // rot_p turns pair (i, i + dims/2) of the first ``dims`` channels by p * inv_freq[i]; rot'_p turns
 // pair m of all value channels ((m, m + E/2), or (2m, 2m + 1) when interleaved) by p * v_freq[m].
 // A row of the input holds nh query heads of D, then nkv key heads of D, then nkv value heads of
@@ -23,7 +27,8 @@ __global__ __launch_bounds__(64) void head_prep_kernel(
     const float* __restrict__ q_gain, const float* __restrict__ k_gain, const float* __restrict__ head_scale, float eps,
     const float* __restrict__ inv_freq, int rot_dims, const float* __restrict__ v_freq, int v_interleaved,
     act_t* __restrict__ kcache, act_t* __restrict__ vcache, int nh, int nkv, int D, int E, int bs, int v_transposed,
-    const float* __restrict__ bias, float rot_scale, int qk_interleaved, int ld, int unit_norm) {
+    const float* __restrict__ bias, float rot_scale, int qk_interleaved, int ld, int unit_norm,
+    act_t* __restrict__ v_lend, const act_t* __restrict__ v_lent, const float* __restrict__ v_share) {
   __shared__ float buf[HP_MAX];
   const int t = blockIdx.x, head = blockIdx.y, lane = threadIdx.x;
   const int pos = positions[t];
@@ -39,6 +44,14 @@ __global__ __launch_bounds__(64) void head_prep_kernel(
   for (int d = lane; d < size; d += 64) {
     float x = to_f32(qkv[at + d]);
     if (bias) x += bias[at - (size_t)t * width + d];
+    if (kind == 2) {
+      const size_t vi = ((size_t)t * nkv + (head - nh - nkv)) * E + d;
+      if (v_lend) v_lend[vi] = from_f32<act_t>(x);
+      if (v_lent) {
+        const float l = *v_share;
+        x = fmaf(l, to_f32(v_lent[vi]), (1.0f - l) * x);
+      }
+    }
     buf[d] = x;
     sum = fmaf(x, x, sum);
   }
@@ -105,11 +118,15 @@ __global__ __launch_bounds__(64) void head_prep_kernel(
 // ld: the distance between rows of qkv in elements where a row holds more than the heads (0: the
 // heads alone).  unit_norm: queries and keys are divided by their root mean square over the head
 // (with eps), after the rotation and without a gain.
-extern "C" int zk_head_prep_unit(void* qkv, const int* positions, const int* slot_map, const float* q_gain,
+// v_lend (may be null): [T, nkv * E], receives the values after the bias.  v_lent (may be null): [T, nkv * E]
+// values of an earlier layer, of which each value takes the share *v_share (a float on the device).
+extern "C" int zk_head_prep_values(void* qkv, const int* positions, const int* slot_map, const float* q_gain,
                                  const float* k_gain, const float* head_scale, float eps, const float* inv_freq,
                                  int rot_dims, const float* v_freq, int v_interleaved, void* kcache, void* vcache, int T,
                                  int nh, int nkv, int D, int E, int bs, int v_transposed, const float* bias,
-                                 float rot_scale, int qk_interleaved, int ld, int unit_norm, void* stream) {
+                                 float rot_scale, int qk_interleaved, int ld, int unit_norm, void* v_lend,
+                                 const void* v_lent, const float* v_share, void* stream) {
+  ZK_REQUIRE(v_lent == nullptr || v_share != nullptr, "zk_head_prep: lent values are mixed in with a share");
   ZK_REQUIRE(ld == 0 || ld >= (nh + nkv) * D + nkv * E, "zk_head_prep: rows shorter than their heads");
   ZK_REQUIRE(T >= 0 && nh > 0 && nkv >= 0 && D > 0 && E > 0 && bs > 0, "zk_head_prep: bad sizes");
   ZK_REQUIRE(D <= HP_MAX && E <= HP_MAX, "zk_head_prep: heads of more than 256 channels are not supported");
@@ -123,8 +140,18 @@ extern "C" int zk_head_prep_unit(void* qkv, const int* positions, const int* slo
   head_prep_kernel<<<grid, 64, 0, (hipStream_t)stream>>>((act_t*)qkv, positions, slot_map, q_gain, k_gain, head_scale, eps,
                                                          inv_freq, rot_dims, v_freq, v_interleaved, (act_t*)kcache,
                                                          (act_t*)vcache, nh, nkv, D, E, bs, v_transposed, bias, rot_scale,
-                                                         qk_interleaved, ld, unit_norm);
+                                                         qk_interleaved, ld, unit_norm, (act_t*)v_lend, (const act_t*)v_lent, v_share);
   return zk_launch_status("zk_head_prep");
+}
+
+extern "C" int zk_head_prep_unit(void* qkv, const int* positions, const int* slot_map, const float* q_gain,
+                                 const float* k_gain, const float* head_scale, float eps, const float* inv_freq,
+                                 int rot_dims, const float* v_freq, int v_interleaved, void* kcache, void* vcache, int T,
+                                 int nh, int nkv, int D, int E, int bs, int v_transposed, const float* bias,
+                                 float rot_scale, int qk_interleaved, int ld, int unit_norm, void* stream) {
+  return zk_head_prep_values(qkv, positions, slot_map, q_gain, k_gain, head_scale, eps, inv_freq, rot_dims, v_freq,
+                             v_interleaved, kcache, vcache, T, nh, nkv, D, E, bs, v_transposed, bias, rot_scale,
+                             qk_interleaved, ld, unit_norm, nullptr, nullptr, nullptr, stream);
 }
 
 extern "C" int zk_head_prep_ext(void* qkv, const int* positions, const int* slot_map, const float* q_gain,
@@ -259,5 +286,7 @@ static const int head_prep_entered =
     zk_steplist_register("zk_head_prep", zk_packed::Call<zk_head_prep>::nargs, (void*)zk_packed::Call<zk_head_prep>::call);
 static const int head_prep_unit_entered = zk_steplist_register(
     "zk_head_prep_unit", zk_packed::Call<zk_head_prep_unit>::nargs, (void*)zk_packed::Call<zk_head_prep_unit>::call);
+static const int head_prep_values_entered = zk_steplist_register(
+    "zk_head_prep_values", zk_packed::Call<zk_head_prep_values>::nargs, (void*)zk_packed::Call<zk_head_prep_values>::call);
 static const int head_prep_ext_entered = zk_steplist_register(
     "zk_head_prep_ext", zk_packed::Call<zk_head_prep_ext>::nargs, (void*)zk_packed::Call<zk_head_prep_ext>::call);

@@ -7,8 +7,10 @@
 //
 // Variants, as parameters of the ``_ext`` entry points: scores softmax(router logits) over all experts
 // instead of sigmoids; the weight on the expert's output instead of its input (out_t = sum s_e Wd y);
-// y = silu(g) u instead of the clamped form.  ``zk_gate_rows`` multiplies float rows by the sigmoid
-// of a number a row (a shared layer's gate).
+// y = silu(g) u instead of the clamped form; experts without a gate, y = max(Wu x', 0)^2, whose
+// weights are [E][F][W].  ``zk_gate_rows`` multiplies float rows by the sigmoid
+// of a number a row (a shared layer's gate).  ``zk_moe_route_groups`` chooses by s + a correction per
+// expert, among the experts of the best groups only, and may bring the weights to a sum.
 //
 // Two ways through the experts.  Few tokens (decoding): one block per (token, choice) multiplies
 // the expert's rows by the token's row, and the weights stream once per choice.  Many tokens
@@ -35,6 +37,11 @@ __device__ __forceinline__ float clamped_swiglu(float g, float u, float limit) {
 
 __device__ __forceinline__ float expert_act(float g, float u, float limit, int act) {
   return act == 1 ? g / (1.0f + expf(-g)) * u : clamped_swiglu(g, u, limit);
+}
+#define MOE_NO_GATE 2             // act: experts without gate rows, the square of relu
+__device__ __forceinline__ float square_of_relu(float x) {
+  x = fmaxf(x, 0.f);
+  return x * x;
 }
 
 // ---- the router: one wave per token
@@ -98,6 +105,102 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
   }
 }
 
+// ---- the router with a correction per expert and groups of neighbouring experts: one wave per token.
+// Choice scores c = s + correction (s = sigmoid of the logits, or their softmax).  With groups, the E
+// experts form ``groups`` runs of E / groups; a group's value is the sum of its two largest c (of one, where it
+// has one), and only experts of the ``keep`` best groups can be chosen.  The ``top`` largest c are
+// chosen, the lower number among equals, of groups as of experts.  Weights: s, divided by the
+// chosen ones' sum (+ 1e-20) when ``normalise``, times ``scale``.
+__global__ __launch_bounds__(64) void moe_route_groups_kernel(const float* __restrict__ logits, int ld,
+                                                              const float* __restrict__ correction, int E, int top,
+                                                              int groups, int keep, int softmax, int normalise, float scale,
+                                                              int* __restrict__ ids, float* __restrict__ wts) {
+  __shared__ float sc[MOE_MAX_EXPERTS], ch[MOE_MAX_EXPERTS], gv[MOE_MAX_EXPERTS];
+  const int t = blockIdx.x, lane = threadIdx.x;
+  const float* z = logits + (size_t)t * ld;
+  float mx = 0.f, sum = 1.f;
+  if (softmax) {
+    mx = -INFINITY;
+    for (int e = lane; e < E; e += 64) mx = fmaxf(mx, z[e]);
+    mx = wave_max(mx);
+    sum = 0.f;
+    for (int e = lane; e < E; e += 64) sum += expf(z[e] - mx);
+    sum = wave_sum(sum);
+  }
+  for (int e = lane; e < E; e += 64) {
+    const float s = softmax ? expf(z[e] - mx) / sum : 1.0f / (1.0f + expf(-z[e]));
+    sc[e] = s;
+    ch[e] = correction ? s + correction[e] : s;
+  }
+  __syncthreads();
+  // the largest of v[0..n) still in the race, the lowest number among equals; one that was taken is
+  // left at -inf by its taker.  Always a number below n, whatever the values are.
+  auto best_of = [&](const float* v, int n) {
+    float best = -INFINITY;
+    int at = 0x7fffffff;
+    for (int e = lane; e < n; e += 64)
+      if (v[e] > best) {
+        best = v[e];
+        at = e;
+      }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ob = __shfl_xor(best, o, 64);
+      const int oa = __shfl_xor(at, o, 64);
+      if (ob > best || (ob == best && oa < at)) {
+        best = ob;
+        at = oa;
+      }
+    }
+    return at < n ? at : 0;
+  };
+  if (groups > 1 && keep < groups) {
+    const int size = E / groups;
+    for (int g = lane; g < groups; g += 64) {
+      float a = -INFINITY, b = -INFINITY;
+      for (int i = 0; i < size; i++) {
+        const float c = ch[g * size + i];
+        if (c > a) {
+          b = a;
+          a = c;
+        } else if (c > b) {
+          b = c;
+        }
+      }
+      gv[g] = size > 1 ? a + b : a;
+    }
+    __syncthreads();
+    for (int k = 0; k < keep; k++) {
+      const int g = best_of(gv, groups);
+      __syncthreads();
+      if (lane == 0) gv[g] = NAN;                  // kept: out of the race, told apart from the rest
+      __syncthreads();
+    }
+    for (int e = lane; e < E; e += 64)
+      if (!isnan(gv[e / size])) ch[e] = -INFINITY;
+    __syncthreads();
+  }
+  float total = 0.f;
+  for (int k = 0; k < top; k++) {
+    const int e = best_of(ch, E);
+    __syncthreads();
+    const float s = sc[e];
+    total += s;
+    if (lane == 0) {
+      ids[(size_t)t * top + k] = e;
+      wts[(size_t)t * top + k] = s * scale;
+      ch[e] = -INFINITY;
+    }
+    __syncthreads();
+  }
+  if (normalise && lane == 0) {
+    for (int k = 0; k < top; k++) {
+      const float s = sc[ids[(size_t)t * top + k]];
+      wts[(size_t)t * top + k] = s / (total + 1e-20f) * scale;
+    }
+  }
+}
+
 // Eight consecutive weights as floats (rows in whole groups of eight are read 16 bytes a lane).
 __device__ __forceinline__ void load8(const float* p, float v[8]) {
   const float4 a = *(const float4*)p, b = *(const float4*)(p + 4);
@@ -152,9 +255,14 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(const act_t* __restric
   const act_t* xr = x + (size_t)t * W;
   for (int i = tid; i < W; i += 256) xs[i] = on_out ? to_f32(xr[i]) : to_f32(from_f32<act_t>(s * to_f32(xr[i])));
   __syncthreads();
-  const act_t* wg = w_gu + (size_t)e * 2 * F * W;
+  const act_t* wg = w_gu + (size_t)e * (act == MOE_NO_GATE ? 1 : 2) * F * W;
   const int n0 = blockIdx.y * rows_per_block;
   for (int n = n0 + wave; n < min(F, n0 + rows_per_block); n += 4) {
+    if (act == MOE_NO_GATE) {
+      const float u = row_dot(wg + (size_t)n * W, xs, W, lane);
+      if (lane == 0) y[(size_t)pair * F + n] = from_f32<act_t>(square_of_relu(u));
+      continue;
+    }
     const act_t* gr = wg + (size_t)n * W;
     const act_t* ur = wg + (size_t)(F + n) * W;
     const float g = row_dot(gr, xs, W, lane), u = row_dot(ur, xs, W, lane);
@@ -238,7 +346,8 @@ typedef float floatx16 __attribute__((ext_vector_type(16)));
 #define GG_PAD 8
 
 // mode 0: C = act(gate, up) with B = [E][2F][K], stores y[i, n] (n < F); mode 1: plain product
-// with B = [E][N][K], stores float rows at out[order..] (see the launch).
+// with B = [E][N][K], stores float rows at out[order..] (see the launch); mode 2: the square of
+// relu of that product, stores y.
 template <int MODE>
 __global__ __launch_bounds__(256) void moe_grouped_kernel(const __bf16* __restrict__ A, const __bf16* __restrict__ B,
                                                           const int* __restrict__ first, int E, int N, int K,
@@ -304,6 +413,7 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(const __bf16* __restri
     const int r = wm + (i / 4) * 8 + (lane >> 5) * 4 + (i % 4);
     if (r < rows && col < N) {
       if (MODE == 0) y[(size_t)(row0 + r) * N + col] = (__bf16)expert_act(acc0[i], acc1[i], limit, act);
+      else if (MODE == 2) y[(size_t)(row0 + r) * N + col] = (__bf16)square_of_relu(acc0[i]);
       else out_rows[(size_t)(row0 + r) * N + col] = acc0[i];
     }
   }
@@ -355,6 +465,21 @@ int zk_moe_route(const float* logits, void* ids, float* wts, int T, int E, int t
   return zk_moe_route_ext(logits, E, ids, wts, T, E, top, 0, stream);
 }
 
+// As zk_moe_route_ext with a correction per expert (float [E], may be null: 0) that counts in the choice
+// alone, ``groups`` groups of neighbours of which ``keep`` stay (groups <= 1: none), and weights that are
+// divided by their sum (normalise) and times ``scale``.
+int zk_moe_route_groups(const float* logits, int ld, const float* correction, void* ids, float* wts, int T, int E, int top,
+                        int groups, int keep, int softmax, int normalise, float scale, void* stream) {
+  ZK_REQUIRE(T >= 0 && E > 0 && top > 0 && top <= E && ld >= E, "zk_moe_route_groups: bad sizes");
+  ZK_REQUIRE(E <= MOE_MAX_EXPERTS && top <= MOE_MAX_TOP, "zk_moe_route_groups: up to 1024 experts and 16 choices");
+  ZK_REQUIRE(groups <= 1 || (E % groups == 0 && keep >= 1 && keep <= groups && keep * (E / groups) >= top),
+             "zk_moe_route_groups: equal groups, of which enough stay for the choices");
+  if (T == 0) return 0;
+  moe_route_groups_kernel<<<T, 64, 0, (hipStream_t)stream>>>(logits, ld, correction, E, top, groups, keep, softmax, normalise,
+                                                            scale, (int*)ids, wts);
+  return zk_launch_status("zk_moe_route_groups");
+}
+
 // rows: float [T, W], each multiplied by sigmoid(z[t * ld]).
 int zk_gate_rows(float* rows, const float* z, int ld, int T, int W, void* stream) {
   ZK_REQUIRE(T >= 0 && W > 0 && ld > 0 && rows != nullptr && z != nullptr, "zk_gate_rows: bad arguments");
@@ -365,7 +490,8 @@ int zk_gate_rows(float* rows, const float* z, int ld, int T, int W, void* stream
 
 // x: [T, W]; w_gu: [E][2F][W], an expert's gate rows, then its up rows; w_down: [E][W][F].
 // y: scratch [T * top, F] activations; out: float [T, W].
-// act: 0 the clamped form, 1 silu(gate) up.  on_out: the weight multiplies the expert's output.
+// act: 0 the clamped form, 1 silu(gate) up, 2 the square of relu(up) without a gate (w_gu is then
+// [E][F][W]).  on_out: the weight multiplies the expert's output.
 int zk_moe_experts_ext(const void* x, const int* ids, const float* wts, const void* w_gu, const void* w_down, void* y,
                        float* out, int T, int top, int W, int F, float limit, int act, int on_out, void* stream) {
   ZK_REQUIRE(T >= 0 && top > 0 && top <= MOE_MAX_TOP && W > 0 && F > 0, "zk_moe_experts: bad sizes");
@@ -423,7 +549,10 @@ int zk_moe_experts_grouped_ext(const void* x, const int* ids, const float* wts, 
   moe_gather_kernel<<<pairs, 256, 0, st>>>((const act_t*)x, order, on_out ? nullptr : wts, (act_t*)xg, top, W);
   const int tiles = (pairs + GG_TM - 1) / GG_TM + E;        // each expert may end in a tile that is not full
   dim3 g0(tiles, (F + GG_TN - 1) / GG_TN);
-  moe_grouped_kernel<0><<<g0, 256, 0, st>>>((const __bf16*)xg, (const __bf16*)w_gu, first, E, F, W, (__bf16*)y, nullptr, limit, act);
+  if (act == MOE_NO_GATE)
+    moe_grouped_kernel<2><<<g0, 256, 0, st>>>((const __bf16*)xg, (const __bf16*)w_gu, first, E, F, W, (__bf16*)y, nullptr, limit, act);
+  else
+    moe_grouped_kernel<0><<<g0, 256, 0, st>>>((const __bf16*)xg, (const __bf16*)w_gu, first, E, F, W, (__bf16*)y, nullptr, limit, act);
   dim3 g1(tiles, (W + GG_TN - 1) / GG_TN);
   moe_grouped_kernel<1><<<g1, 256, 0, st>>>((const __bf16*)y, (const __bf16*)w_down, first, E, W, F, nullptr, rows, 0.f, 0);
   moe_combine_kernel<<<T, 256, 0, st>>>(rows, place, out, top, W, on_out ? wts : nullptr);
@@ -444,6 +573,7 @@ ZK_ENTER(zk_moe_experts_grouped)
 ZK_ENTER(zk_moe_experts_grouped_ext)
 #endif
 ZK_ENTER(zk_moe_route_ext)
+ZK_ENTER(zk_moe_route_groups)
 ZK_ENTER(zk_moe_experts_ext)
 ZK_ENTER(zk_gate_rows)
 ZK_ENTER(zk_moe_route)

@@ -1,6 +1,6 @@
 // Element by element: an activation without a gate, and a gate on the heads of a mixer.
 //
-//   zk_unary_act:   out = act(x)                        act 0: max(x, 0)^2
+//   zk_unary_act:   out = act(x)                        act 0: max(x, 0)^2;  1: 0.5 x (1 + erf(x / sqrt(2)))
 //   zk_gate_heads:  o <- o * sigmoid(g)                 g read from rows of another width; one g
 //                                                       for every ``per`` channels (a number a head)
 //
@@ -15,8 +15,8 @@ extern "C" int zk_steplist_register(const char* name, int nargs, void* fn);
 __global__ void unary_act_kernel(const act_t* __restrict__ x, act_t* __restrict__ out, size_t n, int act) {
   const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= n) return;
-  const float v = fmaxf(to_f32(x[i]), 0.f);
-  out[i] = from_f32<act_t>(v * v);
+  const float z = to_f32(x[i]), v = fmaxf(z, 0.f);
+  out[i] = from_f32<act_t>(act == 1 ? 0.5f * z * (1.0f + erff(z * 0.7071067811865476f)) : v * v);
 }
 
 __global__ void gate_heads_kernel(act_t* __restrict__ o, const act_t* __restrict__ g, int ldg, int W, int per) {
@@ -30,9 +30,9 @@ __global__ void gate_heads_kernel(act_t* __restrict__ o, const act_t* __restrict
 
 extern "C" {
 
-// x, out: n activations.  act: 0 = the square of relu.
+// x, out: n activations.  act: 0 = the square of relu, 1 = gelu with the error function.
 int zk_unary_act(const void* x, void* out, size_t n, int act, void* stream) {
-  ZK_REQUIRE(act == 0, "zk_unary_act: unknown activation");
+  ZK_REQUIRE(act == 0 || act == 1, "zk_unary_act: unknown activation");
   if (n == 0) return 0;
   ZK_REQUIRE((n + 255) / 256 < 2147483647ull, "zk_unary_act: too many elements");
   unary_act_kernel<<<(unsigned)((n + 255) / 256), 256, 0, (hipStream_t)stream>>>((const act_t*)x, (act_t*)out, n, act);

@@ -111,7 +111,7 @@ class Engine:
                                                               else (needs[c].value_dim or needs[c].head_dim)))
                        for c in g.calls) * item * block_size
         def windowed_pages(g):
-            per_request = -(-(g.window + step_tokens) // block_size) + 2
+            per_request = -(-(g.window + step_tokens) // block_size) + 2 + -(-g.keep_first // block_size)
             return max_seqs * min(per_request, -(-max_len // block_size))
         if num_blocks is None:
             budget = int(self.rt.info().free_memory * 0.6)

@@ -37,6 +37,13 @@ class Model:
             if call.cache_of is not None and not (0 <= call.cache_of < i):
                 raise ValueError(f"order entry {i} reads the cache of entry {call.cache_of}, "
                                  f"which does not run before it")
+        # rows that a layer lends to later layers of the same step: key -> channels
+        self.lent: Dict[str, int] = {}
+        for b in self.blocks:
+            for p in walk(b):
+                for key, channels in p.lends():
+                    if self.lent.setdefault(key, channels) != channels:
+                        raise ValueError(f"two layers lend {key!r} with {self.lent[key]} and {channels} channels")
         self.loaded_dtype: Optional[str] = None
         self.tuned = True            # set at load: whether weights may sit in the tuned kernels' layouts
 
@@ -74,7 +81,9 @@ class Model:
                 reader = self.blocks[call.layer].mixer.cache_need()
                 if isinstance(reader, PagedKV) and own.window is not None and \
                         (reader.window is None or reader.window > own.window):
-                    out[call.cache_of] = replace(own, window=reader.window)
+                    own = out[call.cache_of] = replace(own, window=reader.window)
+                if isinstance(reader, PagedKV) and reader.keep_first > own.keep_first:
+                    out[call.cache_of] = replace(own, keep_first=reader.keep_first)
         return out
 
     # ---- what a step costs, for measurements: read off the parts, whatever the architecture
@@ -94,6 +103,8 @@ class Model:
                     if need.window and last > need.window:
                         full = max(0, min(n, last - need.window))          # tokens that see a whole window
                         keys = full * need.window + sum(range(last - n + 1, last - full + 1))
+                        # and the kept first keys in front of it
+                        keys += sum(min(need.keep_first, p - need.window) for p in range(last - full + 1, last + 1))
                     else:
                         keys = sum(range(start + 1, last + 1))
                     total += mixer.flops_per_key() * keys
@@ -104,7 +115,7 @@ class Model:
         total = 0
         for need in self.cache_needs():
             if isinstance(need, PagedKV):
-                seen = min(context, need.window) if need.window else context
+                seen = min(context, need.window + need.keep_first) if need.window else context
                 vd = 0 if getattr(need, "values_in_keys", False) else (need.value_dim or need.head_dim)
                 nv = getattr(need, "value_heads", None) or need.num_kv_heads
                 total += (need.num_kv_heads * need.head_dim + nv * vd) * seen * itemsize
@@ -145,10 +156,13 @@ class Model:
         again = any(getattr(c, "add_embedding", False) for c in order)
         # (gathered a second time: a launch like any other, which a captured or written-down step repeats)
         first = self.embedding.forward(ctx) if again else None
+        ctx.lent = {key: ctx.alloc((T, channels)) for key, channels in self.lent.items()}
         x = None
         base = ctx.arena.mark()
+        cache_for = lambda i: caches[i] if caches[i].shared else caches[order[i].cache_of if order[i].cache_of is not None else i]
         for i, call in enumerate(order):
-            cache = caches[i] if caches[i].shared else caches[call.cache_of if call.cache_of is not None else i]
+            cache = cache_for(i)
+            ctx.next_cache = cache_for(i + 1) if i + 1 < len(order) else None      # of the entry whose input this one may make
             blk = self.blocks[call.layer]
             nxt = self.blocks[order[i + 1].layer] if i + 1 < len(order) else None
             if nxt is not None and getattr(order[i + 1], "add_embedding", False):

@@ -17,6 +17,7 @@ from typing import List
 
 import numpy as np
 
+from ..config.plan import ShortConvSpec
 from ..runtime.device import BF16, ITEMSIZE, Tensor
 from .base import ROLE_GAIN, PagedKV, Part, TensorReq, build_part, register_part
 from .ops import linear, tuned_gemm
@@ -57,7 +58,33 @@ class PagedAttention(Part):
             raise ValueError("an attention has a window or a chunk, not both")
         if self.chunk < 0:
             raise ValueError(f"chunk must be positive, got {self.chunk}")
-        self.general = bool(self.value_dim != s.head_dim or self.q_norm_name or self.k_norm_name or
+        # beside its window a query may see the sequence's first keys
+        self.keep = int(getattr(s, "keep_first", 0) or 0)
+        if self.keep < 0 or (self.keep and not s.window):
+            raise ValueError(f"first keys are kept beside a window, got keep_first {self.keep} and window {s.window}")
+        # a short convolution over time on the projected rows, which then takes the projections' biases
+        self.conv = None
+        conv_names = dict(getattr(s, "convs", None) or {})
+        if conv_names:
+            roles = ("q",) if self.shared_kv else ("q", "k", "v")
+            if set(conv_names) != set(roles) or self.values_are_keys:
+                raise ValueError(f"convolutions on {sorted(conv_names)}: all of {roles} or none (and no values that are keys)")
+            self.conv_counts = tuple(n for r, n in (("q", s.num_heads * s.head_dim), ("k", s.num_kv_heads * s.head_dim),
+                                                    ("v", s.num_kv_heads * self.value_dim)) if r in roles)
+            biased = [r for r in roles if r in self.bias_names]
+            if biased and len(biased) != len(roles):
+                raise ValueError("biases on the projections: all of q, k, v or none")
+            self.conv = build_part("filter", ShortConvSpec(
+                size=sum(self.conv_counts), taps=s.conv_taps, weight=tuple(conv_names[r] for r in roles), residual=False,
+                channel_counts=self.conv_counts, in_bias=tuple(self.bias_names[r] for r in roles) if biased else None))
+            for r in biased:
+                self.bias_names.pop(r)         # the convolution's own now
+        self.lend_values = bool(getattr(s, "lend_values", False))
+        self.share_name = getattr(s, "value_share", None)
+        self.value_share = None
+        if (self.lend_values or self.share_name) and (self.shared_kv or self.values_are_keys or self.by_rows):
+            raise ValueError("values are lent and mixed by mixers that project values of their own, with norms per head")
+        self.general = bool(self.conv or self.keep or self.lend_values or self.share_name or self.value_dim != s.head_dim or self.q_norm_name or self.k_norm_name or
                             self.head_scale_name or self.value_base or self.bias_names or
                             self.rot_scale != 1.0 or self.rot_interleaved or self.chunk or self.unit_sink or self.wide_weights or
                             self.unit_norm or self.gate_name or self.by_rows)
@@ -80,7 +107,12 @@ class PagedAttention(Part):
         self.decode_chunk = 64                     # keys a wave of the split decode attention takes
 
     def children(self):
-        return [self.position]
+        return [self.position] + ([self.conv] if self.conv is not None else [])
+
+    LENT = "values"
+
+    def lends(self):
+        return [(self.LENT, self.spec.num_kv_heads * self.value_dim)] if self.lend_values else []
 
     def tensor_reqs(self) -> List[TensorReq]:
         s = self.spec
@@ -88,6 +120,8 @@ class PagedAttention(Part):
                TensorReq(s.names["o"], (s.hidden_size, s.num_heads * self.value_dim))]
         if self.q_norm_name:
             out.append(TensorReq(self.q_norm_name, (s.head_dim,), ROLE_GAIN))
+        if self.share_name:
+            out.append(TensorReq(self.share_name, (), ROLE_GAIN))
         if self.head_scale_name:
             out.append(TensorReq(self.head_scale_name, (s.num_heads,), ROLE_GAIN))
         if self.gate_name:
@@ -126,6 +160,8 @@ class PagedAttention(Part):
             self.q_gain = weights.vector(self.q_norm_name)
         if self.k_norm_name and not self.shared_kv:
             self.k_gain = weights.vector(self.k_norm_name)
+        if self.share_name:
+            self.value_share = weights.vector(self.share_name)
         if self.head_scale_name:
             self.head_scale = weights.vector(self.head_scale_name)
         if self.q_row_norm_name:
@@ -146,7 +182,8 @@ class PagedAttention(Part):
     def cache_need(self):
         s = self.spec
         return PagedKV(s.num_kv_heads, s.head_dim, s.window,
-                       self.value_dim if self.value_dim != s.head_dim else None, chunk=self.chunk or None)
+                       self.value_dim if self.value_dim != s.head_dim else None, chunk=self.chunk or None,
+                       keep_first=self.keep, state_bytes=self.conv.state_bytes() if self.conv is not None else 0)
 
     def flops_per_key(self) -> float:
         return 2.0 * self.spec.num_heads * (self.spec.head_dim + self.value_dim)        # q.k and p.v
@@ -156,6 +193,8 @@ class PagedAttention(Part):
     def wants_v_transposed(self, kernels, dtype: str, page_size: int) -> bool:
         """The matrix-core kernel reads V as [page][kv head][hd][bs]."""
         s = self.spec
+        if self.keep:
+            return False
         if (self.chunk or self.unit_sink or self.wide_weights) and not kernels.has("zk_attention_bf16_masked"):
             return False
         return bool(dtype == BF16 and self.value_dim == s.head_dim and kernels.has("zk_attention_bf16") and
@@ -207,7 +246,10 @@ class PagedAttention(Part):
         width = heads_width + (nh * vd if self.gate_name else 0)
         g = ctx.group(cache.group)
         tables = self.position.rotary_tables()
-        qkv = linear(ctx, x, self.w_qkv, ctx.alloc((T, width)))
+        rows = qkv = linear(ctx, x, self.w_qkv, ctx.alloc((T, width)))
+        row_width = width            # of the projected rows, which may hold a gate behind the heads
+        if self.conv is not None:
+            qkv, width = self.conv.forward(ctx, rows, cache.state_offset, ld=row_width), heads_width
         if tables is None:
             self.position.apply(ctx, qkv, nh, n_store, hd)
         ptr = lambda t: t.ptr if t is not None else None
@@ -227,6 +269,15 @@ class PagedAttention(Part):
                 1 if self.rot_interleaved else 0)
         if prep is None:
             pass
+        elif self.lend_values or self.share_name:
+            lent = None
+            if self.share_name:
+                lent = ctx.lent[self.LENT]
+                if lent.shape != (T, n_store * vd):
+                    raise ValueError(f"values of {lent.shape[1]} channels were lent, this layer's have {n_store * vd}")
+            k.zk_head_prep_values(*prep, width, 1 if self.unit_norm else 0,
+                                  ctx.lent[self.LENT].ptr if self.lend_values else None, ptr(lent), ptr(self.value_share),
+                                  ctx.stream)
         elif self.unit_norm or width != heads_width:
             k.zk_head_prep_unit(*prep, width, 1 if self.unit_norm else 0, ctx.stream)
         else:
@@ -234,7 +285,7 @@ class PagedAttention(Part):
         o = ctx.alloc((T, nh * vd))
         cap = float(s.softcap) if s.softcap else 0.0
         win = int(s.window) if s.window else 0
-        masked = bool(self.chunk or self.unit_sink or self.wide_weights)
+        masked = bool(self.chunk or self.unit_sink or self.wide_weights or self.keep)
         if masked and cache.v_transposed and ctx.tuned and vd == hd:
             k.zk_attention_bf16_masked(qkv.ptr, width, cache.k.ptr, cache.v.ptr, g.block_table, g.max_blocks,
                                        ctx.q_start, ctx.ctx_len, o.ptr, ctx.R, ctx.n_multi, ctx.max_q_len,
@@ -242,10 +293,10 @@ class PagedAttention(Part):
                                        self.decode_chunk, ctx.workspace.ptr, ctx.workspace.nbytes, self.chunk,
                                        1 if self.unit_sink else 0, 1 if self.wide_weights else 0, ctx.stream)
         elif masked:
-            k.zk_attention_plain_masked(qkv.ptr, width, cache.k.ptr, cache.v.ptr, g.block_table, g.max_blocks,
+            k.zk_attention_plain_kept(qkv.ptr, width, cache.k.ptr, cache.v.ptr, g.block_table, g.max_blocks,
                                         ctx.req_of_token, ctx.positions, o.ptr, T, nh, nkv, hd, vd, g.page_size, s.scale,
                                         cap, win, 1 if cache.v_transposed else 0, vfreq, inter, None, 0, self.chunk,
-                                        1 if self.unit_sink else 0, ctx.stream)
+                                        1 if self.unit_sink else 0, self.keep, ctx.stream)
         elif cache.v_transposed and ctx.tuned and vd == hd:
             k.zk_attention_bf16(qkv.ptr, width, cache.k.ptr, cache.v.ptr, g.block_table, g.max_blocks,
                                 ctx.q_start, ctx.ctx_len, o.ptr, ctx.R, ctx.n_multi, ctx.max_q_len,
@@ -259,7 +310,7 @@ class PagedAttention(Part):
                                      cap, win, 1 if cache.v_transposed else 0, vfreq, inter, ctx.stream)
         if self.gate_name:
             # the heads times sigmoid(W_g x); the gate's columns lie behind the heads' in the product's rows
-            k.zk_gate_heads(o.ptr, qkv.ptr + heads_width * ITEMSIZE[ctx.dtype], width, T, nh * vd, ctx.stream)
+            k.zk_gate_heads(o.ptr, rows.ptr + heads_width * ITEMSIZE[ctx.dtype], row_width, T, nh * vd, ctx.stream)
         y = linear(ctx, o, self.w_o, ctx.alloc((T, s.hidden_size)), last_of=self if self.o_bias is None else None)
         if self.o_bias is not None:
             if getattr(ctx, "bias_welcome", None) is self:

@@ -54,6 +54,7 @@ class PagedKV:
     values_in_keys: bool = False        # a value is the first value_dim channels of its key: no value slab is kept
     chunk: Optional[int] = None
     state_bytes: int = 0
+    keep_first: int = 0                 # beside the window the first ``keep_first`` positions are read for ever
     value_heads: Optional[int] = None   # value heads where they are fewer than the key heads (several maps of keys
     #                                     over the same values); None: as many
 
@@ -88,6 +89,12 @@ class Part:
         none (a table that is gathered from), says so itself."""
         return float(sum(2 * r.shape[0] * r.shape[1] for r in self.tensor_reqs()
                          if r.role == ROLE_MATRIX and len(r.shape) == 2))
+
+    def lends(self) -> List[Tuple[str, int]]:
+        """(key, channels) of rows of activations, one per token of the step, that the part hands on
+        to layers that run later in the same step: ``ctx.lent[key]`` is a buffer that outlives
+        the layers."""
+        return []
 
     def flops_per_key(self) -> float:
         """A mixer over cached keys: multiply-adds x 2 per (token, key it attends to)."""

@@ -14,7 +14,7 @@ from typing import List
 import numpy as np
 
 from ..runtime.device import BF16, F32, Tensor
-from .base import Part, TensorReq, register_part
+from .base import Part, TensorReq, build_part, register_part
 from .ops import linear, tuned_gemm
 
 
@@ -25,6 +25,13 @@ class Embedding(Part):
         self.spec = spec
         self.table = None
         self.scale = float(spec.scale)
+        norm = getattr(spec, "norm", None)
+        self.norm = build_part("norm", norm) if norm is not None else None
+        if self.norm is not None and not hasattr(self.norm, "in_place"):
+            raise ValueError("an embedding's norm is one that works on the float stream in place (a layer norm)")
+
+    def children(self):
+        return [self.norm] if self.norm is not None else []
 
     def tensor_reqs(self) -> List[TensorReq]:
         out = [TensorReq(self.spec.weight, (self.spec.vocab_size, self.spec.hidden_size))]
@@ -78,6 +85,8 @@ class Embedding(Part):
             ctx.k.zk_add_pair_rows(row.ptr, self.pair_table.ptr, ctx.tokens, ctx.positions, ctx.req_of_token, ctx.q_start,
                                    before.ptr, pairs.buckets, pairs.mul_prev, pairs.mul_cur, ctx.T, s.hidden_size,
                                    ctx.stream)
+        if self.norm is not None:
+            self.norm.in_place(ctx, row)
         if copies > 1:          # every residual stream starts as the embedded row
             ctx.k.zk_replicate(row.ptr, h.ptr, ctx.T, copies, s.hidden_size, ctx.stream)
         return h

@@ -11,7 +11,7 @@ from __future__ import annotations
 from typing import List
 
 from ..runtime.device import BF16, F32, I32, Tensor
-from .base import Part, TensorReq, build_part, register_part
+from .base import ROLE_GAIN, Part, TensorReq, build_part, register_part
 from .ops import linear, tuned_gemm
 
 ACTIVATION_CODES = {"gelu_tanh": 0, "silu": 1, "relu": 2}
@@ -68,7 +68,7 @@ class GatedMLP(Part):
         return linear(ctx, a, self.w_down, out if out is not None else ctx.alloc((T, s.hidden_size)), last_of=last)
 
 
-UNARY_CODES = {"relu2": 0}     # max(z, 0)^2
+UNARY_CODES = {"relu2": 0, "gelu": 1}     # max(z, 0)^2;  z (1 + erf(z / sqrt(2))) / 2
 
 
 class MLP(Part):
@@ -93,7 +93,9 @@ class MLP(Part):
         self.w_up = weights.matrix([s.names["up"]], strip=bool(strip and strip(s.hidden_size)))
         self.w_down = weights.matrix([s.names["down"]], strip=bool(strip and strip(s.intermediate_size)))
 
-    def forward(self, ctx, x: Tensor) -> Tensor:
+    def forward(self, ctx, x: Tensor, out: Tensor = None) -> Tensor:
+        """``out``: where the result goes (activations or float32 [T, hidden]); the product that
+        ends the layer then never hands partial sums back."""
         s = self.spec
         T, I = x.shape[0], s.intermediate_size
         if tuned_gemm(ctx, s.hidden_size) and x.ptr % 16 == 0:
@@ -102,12 +104,14 @@ class MLP(Part):
             up = linear(ctx, x, self.w_up, ctx.alloc((T, I)))
             a = ctx.alloc((T, I))
             ctx.k.zk_unary_act(up.ptr, a.ptr, T * I, UNARY_CODES[s.activation], ctx.stream)
-        return linear(ctx, a, self.w_down, ctx.alloc((T, s.hidden_size)), last_of=self)
+        return linear(ctx, a, self.w_down, out if out is not None else ctx.alloc((T, s.hidden_size)),
+                      last_of=None if out is not None else self)
 
 
 class RoutedMLP(Part):
-    """A mixture of small gated layers: scores from a float router product (sigmoids, or a softmax
-    over all experts), the ``top_k`` largest chosen on the device (the lower index among equals),
+    """A mixture of small layers (gated, or without a gate): scores from a float router product (sigmoids, or a softmax
+    over all experts), the ``top_k`` largest chosen on the device (the lower index among equals;
+    optionally by score plus a correction, among the experts of the best groups only),
     the chosen scores as weights on the experts' inputs or on their outputs, the experts' results
     added in the order they were chosen, a shared layer on top (optionally times the sigmoid of a
     number a token, whose row rides below the router's in one product).  Steps of few tokens read each chosen expert's rows once per (token, choice); steps of
@@ -122,7 +126,20 @@ class RoutedMLP(Part):
 
     def __init__(self, spec):
         s = self.spec = spec
-        if s.activation not in (CLAMPED, "silu"):
+        self.gated = bool(getattr(s, "gated", True))
+        if not self.gated and (s.activation != "relu2" or s.scale_input):
+            raise ValueError(f"experts without a gate are relu2 layers with weights on their results, got {s.activation!r}")
+        self.correction_name = getattr(s, "correction", None)
+        self.groups = tuple(getattr(s, "groups", None) or (1, 1))
+        if s.num_experts % self.groups[0] or not (1 <= self.groups[1] <= self.groups[0]) or \
+                self.groups[1] * (s.num_experts // self.groups[0]) < s.top_k:
+            raise ValueError(f"equal groups of experts of which enough stay for {s.top_k} choices, got {s.num_experts} "
+                             f"experts in {self.groups[0]} groups, {self.groups[1]} kept")
+        # a choice by anything but the scores alone, or weights that are not the scores: the wider router kernel
+        self.wide_route = bool(self.correction_name or self.groups != (1, 1) or getattr(s, "normalise", False)
+                               or getattr(s, "weight_scale", 1.0) != 1.0)
+        self.correction = None
+        if self.gated and s.activation not in (CLAMPED, "silu"):
             raise ValueError(f"routed experts are {CLAMPED} or silu layers, got {s.activation!r}")
         if not (1 <= s.top_k <= min(s.num_experts, 16)) or s.num_experts > 1024:
             raise ValueError(f"1 to 16 of up to 1024 experts a token, got {s.top_k} of {s.num_experts}")
@@ -148,22 +165,28 @@ class RoutedMLP(Part):
         out = [TensorReq(s.router, (s.num_experts, s.hidden_size))]
         if self.shared_gate:
             out.append(TensorReq(self.shared_gate, (1, s.hidden_size)))
+        if self.correction_name:
+            out.append(TensorReq(self.correction_name, (s.num_experts,), ROLE_GAIN))
         for e in range(s.num_experts):
-            out += [TensorReq(self._name(e, "gate"), (s.intermediate_size, s.hidden_size)),
-                    TensorReq(self._name(e, "up"), (s.intermediate_size, s.hidden_size)),
+            if self.gated:
+                out.append(TensorReq(self._name(e, "gate"), (s.intermediate_size, s.hidden_size)))
+            out += [TensorReq(self._name(e, "up"), (s.intermediate_size, s.hidden_size)),
                     TensorReq(self._name(e, "down"), (s.hidden_size, s.intermediate_size))]
         return out
 
     def load(self, weights, rt, dtype):
         s = self.spec
         self.w_router = weights.matrix([s.router] + ([self.shared_gate] if self.shared_gate else []))
-        # expert e: rows [e 2F, e 2F + F) its gate, the next F its up; down: rows [e W, (e + 1) W)
-        self.w_gu = weights.matrix([self._name(e, r) for e in range(s.num_experts) for r in ("gate", "up")])
+        # expert e: rows [e 2F, e 2F + F) its gate, the next F its up (without a gate: F rows an expert); down: rows
+        # [e W, (e + 1) W)
+        roles = ("gate", "up") if self.gated else ("up",)
+        self.w_gu = weights.matrix([self._name(e, r) for e in range(s.num_experts) for r in roles])
+        self.correction = weights.vector(self.correction_name) if self.correction_name else None
         self.w_down = weights.matrix([self._name(e, "down") for e in range(s.num_experts)])
 
     def flops_per_token(self) -> float:
         s = self.spec
-        return 2.0 * s.num_experts * s.hidden_size + s.top_k * 6.0 * s.intermediate_size * s.hidden_size
+        return 2.0 * s.num_experts * s.hidden_size + s.top_k * (6.0 if self.gated else 4.0) * s.intermediate_size * s.hidden_size
 
     def forward(self, ctx, x: Tensor) -> Tensor:
         s, k = self.spec, ctx.k
@@ -171,8 +194,14 @@ class RoutedMLP(Part):
         ld = E + (1 if self.shared_gate else 0)
         logits = linear(ctx, x, self.w_router, ctx.alloc((T, ld), F32))
         ids, wts = ctx.alloc((T, top), I32), ctx.alloc((T, top), F32)
-        k.zk_moe_route_ext(logits.ptr, ld, ids.ptr, wts.ptr, T, E, top, 1 if self.scoring == "softmax" else 0, ctx.stream)
-        act, on_out, limit = (1 if s.activation == "silu" else 0), (0 if s.scale_input else 1), float(s.limit or 0.0)
+        softmax = 1 if self.scoring == "softmax" else 0
+        if self.wide_route:
+            k.zk_moe_route_groups(logits.ptr, ld, self.correction.ptr if self.correction is not None else None, ids.ptr, wts.ptr,
+                                  T, E, top, self.groups[0], self.groups[1], softmax, 1 if getattr(s, "normalise", False) else 0,
+                                  float(getattr(s, "weight_scale", 1.0)), ctx.stream)
+        else:
+            k.zk_moe_route_ext(logits.ptr, ld, ids.ptr, wts.ptr, T, E, top, softmax, ctx.stream)
+        act, on_out, limit = (2 if not self.gated else 1 if s.activation == "silu" else 0), (0 if s.scale_input else 1), float(s.limit or 0.0)
         P = 2 if self.shared is not None else 1
         planes = ctx.alloc((P, T, W), F32)
         y = ctx.alloc((T * top, F))

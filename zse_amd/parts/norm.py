@@ -8,6 +8,8 @@ from __future__ import annotations
 
 from typing import List, Optional
 
+import numpy as np
+
 from ..runtime.device import F32, Tensor
 from .base import ROLE_GAIN, Part, TensorReq, register_part
 
@@ -59,6 +61,19 @@ class LayerNorm(Part):
     def load(self, weights, rt, dtype):
         self.weight = weights.vector(self.spec.weight)
         self.bias = weights.vector(self.spec.bias) if self.spec.bias else None
+        scale = float(getattr(self.spec, "gain_scale", 1.0))
+        if scale != 1.0:
+            self.weight = rt.upload((rt.download(self.weight) * np.float32(scale)).astype(np.float32))
+            if self.bias is not None:
+                self.bias = rt.upload((rt.download(self.bias) * np.float32(scale)).astype(np.float32))
+
+    def in_place(self, ctx, x: Tensor) -> None:
+        """The float rows ``x`` replaced by their norm, not rounded."""
+        s = self.spec
+        if x.dtype != F32 or s.streams != 1 or x.shape[1] != s.size:
+            raise ValueError(f"a layer norm in place over float rows of {s.size}: got {x.dtype} {x.shape}")
+        ctx.k.zk_norm_stream(x.ptr, self.weight.ptr, self.bias.ptr if self.bias is not None else None, float(s.eps),
+                             x.shape[0], s.size, ctx.stream)
 
     def forward(self, ctx, x: Tensor, out_rows=None) -> Tensor:
         s = self.spec

@@ -6,7 +6,7 @@ import ctypes
 from ..runtime.device import BF16, F32, Tensor
 
 
-EPILOGUES = {None: 0, "softcap": 1, "gelu_tanh": 2, "silu": 3, "relu": 5, "clamped_swiglu": 6, "relu2": 7}
+EPILOGUES = {None: 0, "softcap": 1, "gelu_tanh": 2, "silu": 3, "relu": 5, "clamped_swiglu": 6, "relu2": 7, "gelu": 8}
 GATED = ("gelu_tanh", "silu", "relu", "clamped_swiglu")
 
 
@@ -27,7 +27,7 @@ def linear(ctx, x: Tensor, w: Tensor, out: Tensor, epilogue=None, cap: float = 0
     [2N, K], gate rows first, and store act(gate) * up; "clamped_swiglu" likewise, with ``cap`` as
     its limit: g = min(gate, cap), u = clamp(up, -cap, cap), g sigmoid(1.702 g) (u + 1).
 
-    "relu2" stores max(x, 0)^2.  ``lda``: the distance between the rows of ``x`` in elements
+    "relu2" stores max(x, 0)^2, "gelu" x (1 + erf(x / sqrt(2))) / 2.  ``lda``: the distance between the rows of ``x`` in elements
     where they are the first K columns of wider rows (0: K).
 
     ``last_of``: the part whose result this product is (it passes itself).  When the block

@@ -222,6 +222,17 @@ KERNEL_SIGNATURES = {
     "zk_diff_join": [_VP, _VP, _I, _I, _I, _F, _F, _F, _VP],
     "zk_selective_scan": [_VP, _I, _VP, _I, _VP, _VP, _I, _I, _I, _VP, _VP, _VP, _I, _VP, _I, _I, _VP, _VP, _VP, _I, _I, _I,
                           _I, _I, _I, _VP, _VP, _VP],
+    "zk_sublayer_step": [_VP, _VP, _I, _VP, _I, _F, _VP, _VP, _VP, _F, _VP, _VP, _I, _VP, _I, _I, _VP, _VP, _VP, _I, _I, _VP],
+    "zk_norm_stream": [_VP, _VP, _VP, _F, _I, _I, _VP],
+    "zk_token_gate": [_VP, _VP, _VP, _I, _I, _VP, _I, _I, _VP],
+    "zk_conv_rows": [_VP, _I, _VP, _VP, _VP, _VP, _I, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _VP],
+    "zk_head_prep_values": [_VP, _VP, _VP, _VP, _VP, _VP, _F, _VP, _I, _VP, _I, _VP, _VP, _I, _I, _I, _I, _I, _I, _I,
+                            _VP, _F, _I, _I, _I, _VP, _VP, _VP, _VP],
+    "zk_moe_route_groups": [_VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _F, _VP],
+    "zk_attention_plain_kept": [_VP, _I, _VP, _VP, _VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _F, _F,
+                                _I, _I, _VP, _I, _VP, _I, _I, _I, _I, _VP],
+    "zk_gdelta_gates": [_VP, _I, _I, _I, _VP, _VP, _VP, _VP, _VP, _I, _I, _VP],
+    "zk_gdelta": [_VP, _I, _I, _I, _VP, _I, _VP, _VP, _VP, _VP, _I, _I, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _F, _VP],
 }
 # present only in the bf16 library
 BF16_KERNEL_SIGNATURES = {
@@ -242,6 +253,7 @@ BF16_KERNEL_SIGNATURES = {
     "zk_latent_attention_bf16_window": [_VP, _VP, _VP, _I, _VP, _VP, _VP, _VP, _VP, _VP, _SZ, _I, _I, _I, _I, _I, _I, _I, _I, _F,
                                         _I, _I, _VP],
     "zk_moe_experts_grouped_ext": [_VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _F, _I, _I, _VP],
+    "zk_gdelta_token": [_VP, _I, _I, _I, _VP, _I, _VP, _VP, _VP, _VP, _I, _I, _VP, _VP, _VP, _VP, _I, _I, _I, _F, _VP],
 }
 
 
@@ -322,7 +334,11 @@ class KernelLibrary:
         self.zk_mlstm_state_bytes = self._dll.zk_mlstm_state_bytes
         self._dll.zk_mlstm_scan_floats.restype, self._dll.zk_mlstm_scan_floats.argtypes = C.c_size_t, [_I] * 6
         self.zk_mlstm_scan_floats = self._dll.zk_mlstm_scan_floats
+        self._dll.zk_conv_rows_most_taps.restype, self._dll.zk_conv_rows_most_taps.argtypes = C.c_int, []
+        self.zk_conv_rows_most_taps = self._dll.zk_conv_rows_most_taps
         if dtype == BF16:
+            self._dll.zk_gdelta_token_supports.restype, self._dll.zk_gdelta_token_supports.argtypes = C.c_int, [_I]
+            self.zk_gdelta_token_supports = self._dll.zk_gdelta_token_supports
             self._dll.zk_attention_bf16_supports.restype = C.c_int
             self._dll.zk_attention_bf16_supports.argtypes = [_I, _I, _I, _I]
             self.zk_attention_bf16_supports = self._dll.zk_attention_bf16_supports

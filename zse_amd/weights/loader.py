@@ -201,17 +201,18 @@ class CheckpointWeights(_Source):
         if same:
             self.rt.copy_h2d(dst.ptr, arr)
             return
-        chunk_rows = max(1, (64 << 20) // max(1, e.nbytes // max(1, e.shape[0])))
+        n_rows = e.shape[0] if e.shape else 1          # a tensor without axes is one number
+        chunk_rows = max(1, (64 << 20) // max(1, e.nbytes // max(1, n_rows)))
         # staging buffer: big enough for one chunk of rows of this tensor
-        row_bytes = e.nbytes // max(1, e.shape[0])
-        need = min(e.shape[0], chunk_rows) * row_bytes
+        row_bytes = e.nbytes // max(1, n_rows)
+        need = min(n_rows, chunk_rows) * row_bytes
         if self._staging is None or self._staging.nbytes < need:
             self._staging = self.rt.empty((need + 3) // 4, F32)
         inner = int(np.prod(e.shape[1:])) if len(e.shape) > 1 else 1
-        flat = arr.reshape(e.shape[0], inner) if e.shape else arr.reshape(1, 1)
+        flat = arr.reshape(n_rows, inner)
         item = 4 if dst.dtype == F32 else 2
-        for r0 in range(0, e.shape[0], chunk_rows):
-            r1 = min(e.shape[0], r0 + chunk_rows)
+        for r0 in range(0, n_rows, chunk_rows):
+            r1 = min(n_rows, r0 + chunk_rows)
             self.rt.copy_h2d(self._staging.ptr, flat[r0:r1])
             self.k.zk_convert(self._staging.ptr, SRC_TAGS[e.dtype], dst.ptr + r0 * inner * item,
                               dst_kind, (r1 - r0) * inner, self.rt.stream)
