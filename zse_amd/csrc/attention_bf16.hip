@@ -33,708 +33,17 @@
 // at most 16 heads a KV head the chunks run on 16x16x32 MFMAs (attn_decode_kernel):
 // a single query token fills only g of a tile's columns, and the narrower tile
 // halves both the accumulator registers and the wasted work, so two waves fit a SIMD.
-#include "common.h"
+//
+// A head's values may be half or twice as wide as its keys.  Where a window keeps the sequence's first
+// keys in sight, the tiles (or a decoded token's chunks) of those keys come first and are
+// followed by the window's.
+// The kernels are templates in attention_bf16_kernels.h.
+#include "attention_bf16_kernels.h"
 #include "packed_call.h"
 
 #include <algorithm>
 
 #if ZSE_ACT_BF16
-
-typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
-typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
-typedef float f32x4 __attribute__((ext_vector_type(4)));
-typedef float f32x16 __attribute__((ext_vector_type(16)));
-
-#define ATT_CHUNK 64
-#define ATT_MOST_RANGES 8      // ranges of keys a block of rows of a portion is cut into, at most
-
-struct AttnParams {
-  const __bf16* q;
-  int q_stride;
-  const __bf16* kcache;   // [page][nkv][bs][hd]
-  const __bf16* vcache;   // [page][nkv >> v_shift][hd][bs]
-  int v_shift;            // 2^v_shift neighbouring key heads share one value head (0: a value head per key head)
-  const int* block_table;
-  int max_blocks;
-  const int* q_start;     // [R + 1]
-  const int* ctx_len;     // [R]
-  __bf16* out;            // [T][nh][hd]
-  float* part_o;          // split: [slot][hd]
-  float* part_ml;         // split: [slot][2]
-  int nh, nkv, hd, bs;
-  int bs_shift;           // page size is 1 << bs_shift in the tuned kernels
-  float scale, softcap;
-  // scores in the log2 domain: with a cap c,  s2 = c2 * tanh(k2 * dot / 2)  computed as
-  // c2 * (1 - 2 / (exp2(k2 * dot) + 1)),  k2 = 2 * scale / c * log2(e),  c2 = c * log2(e);
-  // without a cap  s2 = k1 * dot,  k1 = scale * log2(e).  Probabilities are exp2(s2 - m2).
-  float k1, k2, c2;
-  int window;
-  int tpw;                // tokens a wave owns
-  int r_begin;            // first request of this launch
-  int nchunks;            // split: chunks the grid covers
-  int from_window;        // decode: block 0 of a request is the one its window begins in
-  int chunk;              // decoded tokens on 16-wide tiles: keys a wave takes, 32 or 64
-  int mask_chunk;         // > 0: a row sees the keys of its own chunk of this many positions only (no window then)
-  int sink;               // 1: a key of score 0 without a value joins every row's denominator
-  int wide_weights;       // 1: a weight meets the values as two bf16 numbers, its rounded value and what the
-                          // rounding left (16 bits of mantissa instead of 8; one more product a tile)
-};
-
-// The query head that is the hq-th of key head kvh.  Without shared values: kvh * g + hq.  With
-// 2^v_shift maps of keys over one value head, key head (v, m) serves map m of the g query heads
-// of value head v, and a query head's maps lie side by side: ((v * g + hq) << v_shift) + m.
-__device__ __forceinline__ int q_head_of(const AttnParams& p, int kvh, int hq) {
-  const int g = p.nh / p.nkv;
-  return (((kvh >> p.v_shift) * g + hq) << p.v_shift) | (kvh & ((1 << p.v_shift) - 1));
-}
-
-// The first key a row at position ``pos`` sees.  It never decreases as pos grows, which is all
-// the kernels' bounds over groups and blocks of rows rest on.
-__device__ __forceinline__ int first_key(const AttnParams& p, int pos) {
-  if (p.mask_chunk > 0) return pos - pos % p.mask_chunk;
-  return p.window > 0 ? max(0, pos - p.window + 1) : 0;
-}
-
-// What the sink adds to a row's sum of weights: 2^(0 - m), scores and maximum in the log2 domain.
-__device__ __forceinline__ float sink_weight(const AttnParams& p, float m) {
-  return p.sink ? __builtin_amdgcn_exp2f(-m) : 0.f;
-}
-
-__device__ __forceinline__ float score_log2(const AttnParams& p, float dot) {
-  if (p.softcap > 0.f) {
-    const float e = __builtin_amdgcn_exp2f(p.k2 * dot);
-    return p.c2 * (1.f - 2.f * __builtin_amdgcn_rcpf(e + 1.f));
-  }
-  return p.k1 * dot;
-}
-
-// Portions: which (group, KV head) a block takes.  Blocks go to the 8 XCDs in turn by their
-// number, and every XCD has an L2 of its own; blocks that read the same keys and values (those
-// of one KV head) are therefore given to as few XCDs as possible, so that what one of them has
-// fetched is in the L2 for the others instead of crossing from the memory side once per block.
-__device__ __forceinline__ void portion_block(int& bx, int& by) {
-  const int gx = gridDim.x, gy = gridDim.y;
-  bx = blockIdx.x;
-  by = blockIdx.y;
-  const int total = gx * gy;
-  if (total % 8) return;
-  const int lin = blockIdx.x + gx * blockIdx.y, xcd = lin & 7, slot = lin >> 3;
-  if (gy <= 8 && 8 % gy == 0) {            // 8 / gy XCDs a head
-    const int per = 8 / gy;
-    by = xcd % gy;
-    bx = slot * per + xcd / gy;
-  } else if (gy % 8 == 0) {                // gy / 8 heads an XCD
-    const int heads = gy / 8;
-    by = xcd + 8 * (slot % heads);
-    bx = slot / heads;
-  }
-}
-
-template <int HD16, bool SPLIT, bool PAIR>
-__global__ __launch_bounds__(256, (HD16 <= 8 && !PAIR) ? 2 : 1) void attn_mfma_kernel(AttnParams p) {
-  constexpr int DT = (HD16 + 1) / 2;
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int lr = lane & 31, lk = lane >> 5;
-  const int r = p.r_begin + blockIdx.z;
-  int block_x = blockIdx.x, kvh = blockIdx.y;
-  if (!SPLIT) portion_block(block_x, kvh);
-  const int qs = p.q_start[r], n = p.q_start[r + 1] - qs;
-  if (n <= 0) return;
-  const int start = p.ctx_len[r] - n;
-  // portions: a block owns one group of rows and its four waves take every fourth tile of
-  // keys (their results are joined at the end).  Or (PAIR, for portions whose groups would
-  // need a second, half-empty round of blocks) two groups: one from the end of the portion,
-  // which sees many keys, and its mirror from the start, which sees few, so that every block
-  // has about the same work; the four waves are shared out between the two by their numbers
-  // of key tiles (3 + 1, 2 + 2 or 1 + 3), a group's waves taking its tiles in turn.
-  // Decoded tokens: a wave owns one chunk of keys.
-  int gi = 0, phase = wave, nphase = 4, first_wave = 0;        // group, and the wave's place among its waves
-  int na_block = 4;                                            // waves of the block's first group
-  // single groups: the last group of a portion sees the most keys and goes first, so that the
-  // blocks still running at the end are the short ones
-  if (!SPLIT && !PAIR) gi = (n + p.tpw - 1) / p.tpw - 1 - block_x;
-  if (PAIR) {
-    const int groups = (n + p.tpw - 1) / p.tpw;
-    if (block_x >= (groups + 1) / 2) return;           // the whole block is past the portion
-    const int ga = groups - 1 - block_x, gb = block_x;
-    if (ga != gb) {
-      auto tiles_of = [&](int gr) {
-        const int lo = start + gr * p.tpw, hi = start + min(n, (gr + 1) * p.tpw) - 1;
-        const int klo = first_key(p, lo);
-        return hi / 32 - klo / 32 + 1;
-      };
-      const int ta = tiles_of(ga), tb = tiles_of(gb);
-      const int na = min(3, max(1, (4 * ta + (ta + tb) / 2) / (ta + tb)));
-      na_block = na;
-      if (wave < na) { gi = ga; phase = wave; nphase = na; }
-      else { gi = gb; phase = wave - na; nphase = 4 - na; first_wave = na; }
-    } else {
-      gi = ga;
-    }
-  }
-  const int chunk = SPLIT ? block_x * 4 + wave : 0;
-  const int t0 = gi * p.tpw;
-  if (!PAIR && (gi < 0 || t0 >= n)) return;
-  const int g = p.nh / p.nkv;
-  const int tok = lr / g, hq = lr - tok * g;
-  const int ntok = min(p.tpw, n - t0);
-  const bool row_ok = tok < ntok;
-  const int trow = qs + t0 + (row_ok ? tok : 0);
-  const int pos = start + t0 + (row_ok ? tok : 0);
-  const int head = q_head_of(p, kvh, row_ok ? hq : 0);
-  const int pos_lo = start + t0, pos_hi = start + t0 + ntok - 1;
-  int key_lo = first_key(p, pos_lo);
-  int key_hi = pos_hi;
-  if (SPLIT) {
-    key_lo = max(key_lo, chunk * ATT_CHUNK);
-    key_hi = min(key_hi, chunk * ATT_CHUNK + ATT_CHUNK - 1);
-  }
-  if (SPLIT && key_lo > key_hi) return;
-  const int row_lo = first_key(p, pos);
-  const int* table = p.block_table + (size_t)r * p.max_blocks;
-  const int hd = p.hd, bsh = p.bs_shift, bmask = p.bs - 1, nkv = p.nkv;
-
-  bf16x8 qf[HD16];
-  {
-    const __bf16* qr = p.q + (size_t)trow * p.q_stride + (size_t)head * hd + lk * 8;
-#pragma unroll
-    for (int ks = 0; ks < HD16; ks++) {
-      if (row_ok) qf[ks] = *(const bf16x8*)(qr + ks * 16);
-      else
-#pragma unroll
-        for (int e = 0; e < 8; e++) qf[ks][e] = (__bf16)0.f;
-    }
-  }
-  f32x16 o[DT];
-#pragma unroll
-  for (int dt = 0; dt < DT; dt++)
-#pragma unroll
-    for (int e = 0; e < 16; e++) o[dt][e] = 0.f;
-  float m_run = -INFINITY, l_run = 0.f;
-  // where the lane's channels dt * 32 + lr lie in a (page, kv head) block of the transposed V cache
-  int vrow[DT];
-#pragma unroll
-  for (int dt = 0; dt < DT; dt++) vrow[dt] = min(dt * 32 + lr, hd - 1) << bsh;
-  const bool capped = p.softcap > 0.f;
-  // keys every row of the group sees (none beyond the first row's position, none before the
-  // last row's window; no range at all unless every lane holds a row): tiles inside this range
-  // need no mask
-  const int all_hi = ntok * g == 32 ? pos_lo : -1;
-  const int all_lo = first_key(p, pos_hi);
-
-  // The pages of a tile are looked up a tile ahead as well, so that no load waits for a table
-  // entry: the lane's key row, and the four places its V pieces come from.
-  struct TilePages { int k, va[2], vb[2]; };
-  auto look_up = [&](int key0, TilePages& pg) {
-    pg.k = table[min(key0 + lr, key_hi) >> bsh];
-#pragma unroll
-    for (int h = 0; h < 2; h++) {
-      pg.va[h] = table[min(key0 + h * 16 + 4 * lk, key_hi & ~3) >> bsh];
-      pg.vb[h] = table[min(key0 + h * 16 + 8 + 4 * lk, key_hi & ~3) >> bsh];
-    }
-  };
-  auto load_k = [&](int key0, int page, bf16x8 (&kf)[HD16]) {
-    const int kk = min(key0 + lr, key_hi);
-    const __bf16* kr = p.kcache + ((((size_t)max(page, 0) * nkv + kvh) << bsh) + (kk & bmask)) * hd + lk * 8;
-#pragma unroll
-    for (int ks = 0; ks < HD16; ks++) kf[ks] = *(const bf16x8*)(kr + ks * 16);
-  };
-  auto tile = [&](int key0, const TilePages& pg, int knext, TilePages& pn) {
-    bf16x8 kf[HD16];
-    load_k(key0, pg.k, kf);
-    look_up(knext, pn);
-    // ---- S^T = K Q^T
-    f32x16 s;
-#pragma unroll
-    for (int e = 0; e < 16; e++) s[e] = 0.f;
-#pragma unroll
-    for (int ks = 0; ks < HD16; ks++) s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[ks], qf[ks], s, 0, 0, 0);
-    // ---- V^T pieces for this tile (issued early; used after the softmax)
-    bf16x8 vf[DT][2];
-#pragma unroll
-    for (int h = 0; h < 2; h++) {
-      const int ka = min(key0 + h * 16 + 4 * lk, key_hi & ~3), kb = min(key0 + h * 16 + 8 + 4 * lk, key_hi & ~3);
-      const int pa = max(pg.va[h], 0), pb = max(pg.vb[h], 0);
-      const __bf16* vpa = p.vcache + ((((size_t)pa * (nkv >> p.v_shift) + (kvh >> p.v_shift)) * hd) << bsh) + (ka & bmask);
-      const __bf16* vpb = p.vcache + ((((size_t)pb * (nkv >> p.v_shift) + (kvh >> p.v_shift)) * hd) << bsh) + (kb & bmask);
-#pragma unroll
-      for (int dt = 0; dt < DT; dt++) {
-        const bf16x4 va = *(const bf16x4*)(vpa + vrow[dt]);
-        const bf16x4 vb = *(const bf16x4*)(vpb + vrow[dt]);
-#pragma unroll
-        for (int e = 0; e < 4; e++) {
-          vf[dt][h][e] = va[e];
-          vf[dt][h][4 + e] = vb[e];
-        }
-      }
-    }
-    // ---- scale, cap, mask, running softmax (one query row per lane)
-    float mt = -INFINITY;
-    if (capped) {
-#pragma unroll
-      for (int e = 0; e < 16; e++) {
-        const float ex = __builtin_amdgcn_exp2f(p.k2 * s[e]);
-        s[e] = p.c2 * (1.f - 2.f * __builtin_amdgcn_rcpf(ex + 1.f));
-      }
-    } else {
-#pragma unroll
-      for (int e = 0; e < 16; e++) s[e] *= p.k1;
-    }
-    if (key0 < all_lo || key0 + 31 > all_hi || key0 < key_lo || key0 + 31 > key_hi) {
-#pragma unroll
-      for (int j = 0; j < 4; j++)
-#pragma unroll
-        for (int i = 0; i < 4; i++) {
-          const int key = key0 + 8 * j + 4 * lk + i;
-          const bool ok = row_ok && key >= row_lo && key <= pos && key >= key_lo && key <= key_hi;
-          s[4 * j + i] = ok ? s[4 * j + i] : -INFINITY;
-        }
-    }
-#pragma unroll
-    for (int e = 0; e < 16; e++) mt = fmaxf(mt, s[e]);
-    mt = fmaxf(mt, __shfl_xor(mt, 32, 64));
-    const float m_new = mt > m_run + 8.f ? mt : m_run;      // the reference follows the maximum lazily
-    const float m_use = m_new == -INFINITY ? 0.f : m_new;
-    const bool moved = m_new > m_run;
-    const float corr = moved ? __builtin_amdgcn_exp2f(m_run - m_use) : 1.f;
-    float rs = 0.f;
-#pragma unroll
-    for (int e = 0; e < 16; e++) {
-      const float pe = __builtin_amdgcn_exp2f(s[e] - m_use);
-      s[e] = pe;
-      rs += pe;
-    }
-    rs += __shfl_xor(rs, 32, 64);
-    l_run = l_run * corr + rs;
-    m_run = m_new;
-    bf16x8 pb[2];
-#pragma unroll
-    for (int h = 0; h < 2; h++)
-#pragma unroll
-      for (int e = 0; e < 8; e++) pb[h][e] = (__bf16)s[8 * h + e];
-    // ---- O^T = corr * O^T + V^T P^T  (the maximum rarely rises by the threshold after a
-    // row's first tiles; said so, the compiler keeps the accumulators where the products
-    // want them instead of moving all of them on every tile)
-    if (__builtin_expect(__any(moved), 0)) {
-      // in the accumulation registers, where the products keep them: written so, the compiler
-      // does not copy all of them to ordinary registers on every tile for this rare path
-#pragma unroll
-      for (int dt = 0; dt < DT; dt++)
-#pragma unroll
-        for (int e = 0; e < 16; e++) {
-          float t;
-          asm volatile("v_accvgpr_read_b32 %1, %0\n\tv_mul_f32 %1, %1, %2\n\ts_nop 0\n\tv_accvgpr_write_b32 %0, %1"
-                       : "+a"(o[dt][e]), "=&v"(t)
-                       : "v"(corr));
-        }
-    }
-#pragma unroll
-    for (int dt = 0; dt < DT; dt++) {
-      o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf[dt][0], pb[0], o[dt], 0, 0, 0);
-      o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf[dt][1], pb[1], o[dt], 0, 0, 0);
-    }
-    if (p.wide_weights) {
-#pragma unroll
-      for (int h = 0; h < 2; h++)
-#pragma unroll
-        for (int e = 0; e < 8; e++) pb[h][e] = (__bf16)(s[8 * h + e] - (float)pb[h][e]);
-#pragma unroll
-      for (int dt = 0; dt < DT; dt++) {
-        o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf[dt][0], pb[0], o[dt], 0, 0, 0);
-        o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf[dt][1], pb[1], o[dt], 0, 0, 0);
-      }
-    }
-  
-  };
-  {
-    const int kstep = SPLIT ? 32 : 32 * nphase;
-    int key0 = (key_lo / 32) * 32 + (SPLIT ? 0 : phase * 32);
-    TilePages p0, p1;
-    if (key0 <= key_hi) look_up(key0, p0);
-    for (; key0 <= key_hi; key0 += 2 * kstep) {
-      tile(key0, p0, key0 + kstep, p1);
-      if (key0 + kstep > key_hi) break;
-      tile(key0 + kstep, p1, key0 + 2 * kstep, p0);
-    }
-  }
-  if (SPLIT) {
-    if (!row_ok) return;
-    const size_t slot = ((size_t)(r - p.r_begin) * p.nh + head) * p.nchunks + chunk;
-    if (lk == 0) {
-      p.part_ml[slot * 2] = m_run;
-      p.part_ml[slot * 2 + 1] = l_run;
-    }
-    float* po = p.part_o + slot * hd;
-#pragma unroll
-    for (int dt = 0; dt < DT; dt++)
-#pragma unroll
-      for (int j = 0; j < 4; j++) {
-        const int d = dt * 32 + 8 * j + 4 * lk;
-        if (d < hd) *(f32x4*)(po + d) = f32x4{o[dt][4 * j], o[dt][4 * j + 1], o[dt][4 * j + 2], o[dt][4 * j + 3]};
-      }
-  } else {
-    // join a group's waves: common maximum and sum per row, then the accumulators of the
-    // group's other waves reach its first wave through LDS, one wave a round (a slot a group)
-    extern __shared__ float dyn[];
-    float* sm_ml = dyn;                          // [4][32][2]
-    float* sm_o = dyn + 4 * 32 * 2;              // [2][DT * 16][64]
-    if (lk == 0) {
-      sm_ml[(wave * 32 + lr) * 2] = m_run;
-      sm_ml[(wave * 32 + lr) * 2 + 1] = l_run;
-    }
-    __syncthreads();
-    float m_all = -INFINITY;
-    for (int w = first_wave; w < first_wave + nphase; w++) m_all = fmaxf(m_all, sm_ml[(w * 32 + lr) * 2]);
-    float l_all = 0.f;
-    for (int w = first_wave; w < first_wave + nphase; w++) {
-      const float mw = sm_ml[(w * 32 + lr) * 2];
-      l_all += mw == -INFINITY ? 0.f : sm_ml[(w * 32 + lr) * 2 + 1] * __builtin_amdgcn_exp2f(mw - m_all);
-    }
-    const float f = m_run == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m_run - m_all);
-#pragma unroll
-    for (int dt = 0; dt < DT; dt++)
-#pragma unroll
-      for (int e = 0; e < 16; e++) o[dt][e] *= f;
-    float* slot = sm_o + (size_t)(first_wave ? 1 : 0) * DT * 16 * 64;
-    const int rounds = max(na_block, 4 - na_block) - 1;
-    for (int step = 1; step <= rounds; step++) {
-      if (phase == step) {
-#pragma unroll
-        for (int dt = 0; dt < DT; dt++)
-#pragma unroll
-          for (int e = 0; e < 16; e++) slot[(dt * 16 + e) * 64 + lane] = o[dt][e];
-      }
-      __syncthreads();
-      if (phase == 0 && step < nphase) {
-#pragma unroll
-        for (int dt = 0; dt < DT; dt++)
-#pragma unroll
-          for (int e = 0; e < 16; e++) o[dt][e] += slot[(dt * 16 + e) * 64 + lane];
-      }
-      __syncthreads();
-    }
-    if (phase != 0 || !row_ok) return;
-    const float inv = 1.f / (l_all + sink_weight(p, m_all));
-    __bf16* orow = p.out + ((size_t)trow * p.nh + head) * hd;
-#pragma unroll
-    for (int dt = 0; dt < DT; dt++)
-#pragma unroll
-      for (int j = 0; j < 4; j++) {
-        const int d = dt * 32 + 8 * j + 4 * lk;
-        if (d < hd) {
-          bf16x4 w;
-#pragma unroll
-          for (int i = 0; i < 4; i++) w[i] = (__bf16)(o[dt][4 * j + i] * inv);
-          *(bf16x4*)(orow + d) = w;
-        }
-      }
-  }
-}
-
-// Long portions.  A block of NW waves owns NW groups of rows that follow each other in one
-// request (NW * tpw tokens times the g heads of a KV head), every wave one group, and all of
-// them walk the same keys: a tile of 32 keys and its values come from the cache once a block,
-// wait in LDS and serve every wave (attn_mfma_kernel fetches them once a group of 32 rows:
-// with many groups the way from L2 to the CUs then sets the time).  No join: a wave sees all
-// the keys of its rows.  Two buffers: the loads of the next tile are in flight while the
-// current one is multiplied, and one barrier a tile suffices.
-//   sK [2][32 keys][hd + 8]       a lane's piece for the first product is 16 bytes of a key's row
-//   sV [2][hd][32 + 8]            a channel's 32 keys in the order the second product wants:
-//                                 piece 2h + lk = keys 16h + 4lk + (0..3), 16h + 8 + 4lk + (0..3)
-// The padding of 16 bytes a row keeps the 16-byte reads of 16 lanes on different banks.
-// Pages of at least 8 keys (a 16-byte piece of the transposed V holds 8 keys of one page).
-//
-// SPLIT: a launch of few blocks with many keys each (a prompt of a few thousand tokens and few
-// heads) cuts the keys of a block of rows into ranges of p.chunk tiles, counted from the
-// block's first tile; blockIdx.x is (block of rows) * p.nchunks + range.  A block then leaves
-// (max, sum, O) of its range for every row, as the chunks of a decoded token do, and
-// attn_portion_join_kernel joins a row's ranges in their order.
-template <int HD16, int NW, bool SPLIT>
-__global__ __launch_bounds__(NW * 64, (HD16 <= 8 && NW <= 4) ? 2 : 1) void attn_shared_kernel(AttnParams p) {
-  constexpr int HD = HD16 * 16, DT = (HD16 + 1) / 2;
-  constexpr int KLD = HD + 8, VLD = 32 + 8;
-  constexpr int NT = NW * 64;
-  constexpr int PIECES = 4 * HD;                        // 16-byte pieces of a K tile, and of a V tile
-  constexpr int PPT = (PIECES + NT - 1) / NT;           // pieces of each a thread moves
-  constexpr int CPK = HD / 8;                           // pieces of a key's row
-  extern __shared__ __attribute__((aligned(16))) unsigned char shared_raw[];
-  __bf16* sK = (__bf16*)shared_raw;                     // [2][32][KLD]
-  __bf16* sV = sK + 2 * 32 * KLD;                       // [2][HD][VLD]
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int lr = lane & 31, lk = lane >> 5;
-  const int r = p.r_begin + blockIdx.z;
-  int block_x, kvh;
-  portion_block(block_x, kvh);
-  const int qs = p.q_start[r], n = p.q_start[r + 1] - qs;
-  if (n <= 0) return;
-  const int start = p.ctx_len[r] - n;
-  const int per_block = NW * p.tpw;
-  // the last rows of a portion see the most keys and go first
-  const int rows_x = SPLIT ? block_x / p.nchunks : block_x;
-  const int range = SPLIT ? block_x - rows_x * p.nchunks : 0;
-  const int bi = (n + per_block - 1) / per_block - 1 - rows_x;
-  if (bi < 0) return;
-  const int g = p.nh / p.nkv;
-  // the block's keys: from the window of its first row to its last row
-  const int blk_lo = start + bi * per_block, blk_hi = start + min(n, (bi + 1) * per_block) - 1;
-  int key_lo = first_key(p, blk_lo);
-  int key_hi = blk_hi;
-  if (SPLIT) {
-    const int first_tile = key_lo / 32 + range * p.chunk;
-    if (first_tile * 32 > key_hi) return;              // the block of rows has fewer ranges
-    key_lo = max(key_lo, first_tile * 32);
-    key_hi = min(key_hi, (first_tile + p.chunk) * 32 - 1);
-  }
-  // the wave's rows
-  const int t0 = bi * per_block + wave * p.tpw;
-  const int ntok = max(0, min(p.tpw, n - t0));
-  const int tok = lr / g, hq = lr - tok * g;
-  const bool row_ok = tok < ntok;
-  const int trow = qs + (row_ok ? t0 + tok : 0);
-  const int pos = start + (row_ok ? t0 + tok : 0);
-  const int head = q_head_of(p, kvh, row_ok ? hq : 0);
-  const int pos_lo = start + t0, pos_hi = start + t0 + ntok - 1;          // ntok == 0: no keys at all
-  const int row_lo = first_key(p, pos);
-  const int all_hi = ntok * g == 32 ? pos_lo : -1;
-  const int all_lo = first_key(p, pos_hi);
-  const int* table = p.block_table + (size_t)r * p.max_blocks;
-  const int bsh = p.bs_shift, bmask = p.bs - 1, nkv = p.nkv;
-
-  bf16x8 qf[HD16];
-  {
-    const __bf16* qr = p.q + (size_t)trow * p.q_stride + (size_t)head * HD + lk * 8;
-#pragma unroll
-    for (int ks = 0; ks < HD16; ks++) {
-      if (row_ok) qf[ks] = *(const bf16x8*)(qr + ks * 16);
-      else
-#pragma unroll
-        for (int e = 0; e < 8; e++) qf[ks][e] = (__bf16)0.f;
-    }
-  }
-  f32x16 o[DT];
-#pragma unroll
-  for (int dt = 0; dt < DT; dt++)
-#pragma unroll
-    for (int e = 0; e < 16; e++) o[dt][e] = 0.f;
-  float m_run = -INFINITY, l_run = 0.f;
-
-  // The thread's pieces of a tile.  K: piece q is 8 channels (q % CPK) of key q / CPK.  V: the
-  // pieces of a page's part of the tile lie one behind the other in the cache, channel by
-  // channel: with tk = min(page size, 32) keys of a page in the tile, piece q is the keys
-  // [8c, 8c + 8) of channel d in part q / (HD tk / 8), d = (q / (tk / 8)) % HD, c = q % (tk / 8).
-  const int tk_shift = min(bsh, 5);                     // log2 of a page's keys in a tile
-  const int cpp_shift = tk_shift - 3;                   // log2 of the pieces of a channel in a page's part
-  // What does not change from tile to tile is worked out here, per piece: its place in the page
-  // table relative to the tile's first entry, its offset inside a page's block of the cache (the
-  // KV head, the key's place in the page, the channels) and its place in LDS.  A tile then costs
-  // a piece one table entry and one multiply-add.  (Tiles start at multiples of 32 keys: with
-  // pages of up to 32 keys a key's place in its page does not depend on the tile, with larger
-  // pages the whole tile lies in one page and the tile's offset in it is the same for all.)
-  int k_idx[PPT], v_idx[PPT], k_lds[PPT], v_lds[PPT];
-  unsigned k_off[PPT], v_off[PPT];
-#pragma unroll
-  for (int j = 0; j < PPT; j++) {
-    const int q = min(tid + j * NT, PIECES - 1);
-    const int kk = q / CPK, col = (q % CPK) * 8;
-    const int part = q / (HD << cpp_shift), rem = q - part * (HD << cpp_shift);
-    const int d = rem >> cpp_shift;
-    const int vk = (part << tk_shift) + ((rem & ((1 << cpp_shift) - 1)) << 3);
-    k_idx[j] = kk >> bsh;
-    k_off[j] = (unsigned)(((kvh << bsh) + (kk & bmask)) * HD + col);
-    k_lds[j] = kk * KLD + col;
-    v_idx[j] = vk >> bsh;
-    v_off[j] = (unsigned)((((kvh >> p.v_shift) * HD + d) << bsh) + (vk & bmask));
-    // keys 8c + (0..3) go to piece 2h of the channel, keys 8c + 4 + (0..3) to piece 2h + 1,
-    // both at slot 4 (c % 2), with h = c / 2
-    const int c = vk >> 3;
-    v_lds[j] = d * VLD + (c >> 1) * 16 + (c & 1) * 4;
-  }
-  const size_t page_elems = ((size_t)nkv * HD) << bsh;        // of a page of K
-  const size_t v_page_elems = ((size_t)(nkv >> p.v_shift) * HD) << bsh;
-  const int last_entry = p.max_blocks - 1;
-  struct Pages { int k[PPT], v[PPT]; };
-  struct Stage { bf16x8 k[PPT], v[PPT]; };
-  // A key past the request's last (in its last tile, or in the tile fetched after the last) is
-  // read from wherever its table entry points, page 0 where there is none.  It is masked, but
-  // its value still meets a weight of 0 in the second product, and 0 x NaN is NaN: the caller
-  // keeps page 0 cleared and clears a page before a request first writes to part of it, so
-  // what is read here is the request's own or zero, never what another request left.
-  auto look_up = [&](int key0, Pages& pg) {
-    const int first = key0 >> bsh;
-#pragma unroll
-    for (int j = 0; j < PPT; j++) {
-      pg.k[j] = table[min(first + k_idx[j], last_entry)];
-      pg.v[j] = table[min(first + v_idx[j], last_entry)];
-    }
-  };
-  auto fetch = [&](int key0, const Pages& pg, Stage& st) {
-    const unsigned in_page = (unsigned)(key0 & bmask);
-#pragma unroll
-    for (int j = 0; j < PPT; j++) {
-      st.k[j] = *(const bf16x8*)(p.kcache + ((size_t)max(pg.k[j], 0) * page_elems + (k_off[j] + in_page * HD)));
-      st.v[j] = *(const bf16x8*)(p.vcache + ((size_t)max(pg.v[j], 0) * v_page_elems + (v_off[j] + in_page)));
-    }
-  };
-  auto stash = [&](int buf, const Stage& st) {
-    __bf16* kb = sK + buf * 32 * KLD;
-    __bf16* vb = sV + buf * HD * VLD;
-#pragma unroll
-    for (int j = 0; j < PPT; j++) {
-      if (PIECES % NT == 0 || tid + j * NT < PIECES) {
-        *(bf16x8*)(kb + k_lds[j]) = st.k[j];
-        __bf16* vrow = vb + v_lds[j];
-        bf16x4 lo4, hi4;
-#pragma unroll
-        for (int e = 0; e < 4; e++) {
-          lo4[e] = st.v[j][e];
-          hi4[e] = st.v[j][4 + e];
-        }
-        *(bf16x4*)vrow = lo4;
-        *(bf16x4*)(vrow + 8) = hi4;
-      }
-    }
-  };
-  const bool capped = p.softcap > 0.f;
-  auto tile = [&](int buf, int key0) {
-    const __bf16* kb = sK + buf * 32 * KLD + lr * KLD + lk * 8;
-    const __bf16* vb = sV + buf * HD * VLD + lk * 8;
-    // ---- S^T = K Q^T
-    f32x16 s;
-#pragma unroll
-    for (int e = 0; e < 16; e++) s[e] = 0.f;
-#pragma unroll
-    for (int ks = 0; ks < HD16; ks++)
-      s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8*)(kb + ks * 16), qf[ks], s, 0, 0, 0);
-    // ---- scale, cap, mask, running softmax (one query row per lane)
-    float mt = -INFINITY;
-    if (capped) {
-#pragma unroll
-      for (int e = 0; e < 16; e++) {
-        const float ex = __builtin_amdgcn_exp2f(p.k2 * s[e]);
-        s[e] = p.c2 * (1.f - 2.f * __builtin_amdgcn_rcpf(ex + 1.f));
-      }
-    } else {
-#pragma unroll
-      for (int e = 0; e < 16; e++) s[e] *= p.k1;
-    }
-    if (key0 < all_lo || key0 + 31 > all_hi) {
-#pragma unroll
-      for (int j = 0; j < 4; j++)
-#pragma unroll
-        for (int i = 0; i < 4; i++) {
-          const int key = key0 + 8 * j + 4 * lk + i;
-          const bool ok = row_ok && key >= row_lo && key <= pos;
-          s[4 * j + i] = ok ? s[4 * j + i] : -INFINITY;
-        }
-    }
-#pragma unroll
-    for (int e = 0; e < 16; e++) mt = fmaxf(mt, s[e]);
-    mt = fmaxf(mt, __shfl_xor(mt, 32, 64));
-    const float m_new = mt > m_run + 8.f ? mt : m_run;      // the maximum is followed lazily
-    const float m_use = m_new == -INFINITY ? 0.f : m_new;
-    const bool moved = m_new > m_run;
-    const float corr = moved ? __builtin_amdgcn_exp2f(m_run - m_use) : 1.f;
-    float rs = 0.f;
-#pragma unroll
-    for (int e = 0; e < 16; e++) {
-      const float pe = __builtin_amdgcn_exp2f(s[e] - m_use);
-      s[e] = pe;
-      rs += pe;
-    }
-    rs += __shfl_xor(rs, 32, 64);
-    l_run = l_run * corr + rs;
-    m_run = m_new;
-    bf16x8 pb[2];
-#pragma unroll
-    for (int h = 0; h < 2; h++)
-#pragma unroll
-      for (int e = 0; e < 8; e++) pb[h][e] = (__bf16)s[8 * h + e];
-    // ---- O^T = corr O^T + V^T P^T
-    if (__builtin_expect(__any(moved), 0)) {
-      // in the accumulation registers, where the products keep them
-#pragma unroll
-      for (int dt = 0; dt < DT; dt++)
-#pragma unroll
-        for (int e = 0; e < 16; e++) {
-          float t;
-          asm volatile("v_accvgpr_read_b32 %1, %0\n\tv_mul_f32 %1, %1, %2\n\ts_nop 0\n\tv_accvgpr_write_b32 %0, %1"
-                       : "+a"(o[dt][e]), "=&v"(t)
-                       : "v"(corr));
-        }
-    }
-#pragma unroll
-    for (int dt = 0; dt < DT; dt++) {
-      const __bf16* vr = vb + min(dt * 32 + lr, HD - 1) * VLD;
-      o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8*)vr, pb[0], o[dt], 0, 0, 0);
-      o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8*)(vr + 16), pb[1], o[dt], 0, 0, 0);
-    }
-    if (p.wide_weights) {
-#pragma unroll
-      for (int h = 0; h < 2; h++)
-#pragma unroll
-        for (int e = 0; e < 8; e++) pb[h][e] = (__bf16)(s[8 * h + e] - (float)pb[h][e]);
-#pragma unroll
-      for (int dt = 0; dt < DT; dt++) {
-        const __bf16* vr = vb + min(dt * 32 + lr, HD - 1) * VLD;
-        o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8*)vr, pb[0], o[dt], 0, 0, 0);
-        o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8*)(vr + 16), pb[1], o[dt], 0, 0, 0);
-      }
-    }
-  };
-
-  // Every wave takes every tile of the block, also the few near the diagonal (or before its
-  // window) that none of its rows sees: masked, such a tile adds nothing, and a loop without a
-  // branch around the products lets the compiler leave the accumulators where they are (with
-  // the branch it copied all of them to ordinary registers on every turn: 852 instead of 1,135 us
-  // at 16 heads of 256).  The turn after the last tile fetches that tile again and leaves it
-  // unused.
-  {
-    int key0 = (key_lo / 32) * 32;
-    Pages pg, pn;
-    Stage st;
-    look_up(key0, pg);
-    fetch(key0, pg, st);
-    look_up(key0 + 32, pn);
-    stash(0, st);
-    __syncthreads();
-    for (int buf = 0; key0 <= key_hi; key0 += 32, buf ^= 1) {
-      fetch(key0 + 32, pn, st);
-      look_up(key0 + 64, pn);
-      tile(buf, key0);
-      stash(buf ^ 1, st);
-      __syncthreads();
-    }
-  }
-  if (!SPLIT && !row_ok) return;
-  if (SPLIT) {
-    // A wave's results of its range, as they lie in its registers: 16 bytes a lane, a wave's 64
-    // lanes one contiguous KB per (dt, j), so every store is whole lines.  The joining kernel
-    // reads them back with the same lanes.  Every lane stores, rows or not.
-    const size_t slot = ((((size_t)blockIdx.z * p.nkv + kvh) * (gridDim.x / p.nchunks) + rows_x) * p.nchunks + range) * NW + wave;
-    p.part_ml[slot * 128 + lane] = lk == 0 ? m_run : l_run;
-    f32x4* po = (f32x4*)p.part_o + slot * (DT * 4 * 64) + lane;
-#pragma unroll
-    for (int dt = 0; dt < DT; dt++)
-#pragma unroll
-      for (int j = 0; j < 4; j++)
-        po[(dt * 4 + j) * 64] = f32x4{o[dt][4 * j], o[dt][4 * j + 1], o[dt][4 * j + 2], o[dt][4 * j + 3]};
-    return;
-  }
-  const float inv = 1.f / (l_run + sink_weight(p, m_run));
-  __bf16* orow = p.out + ((size_t)trow * p.nh + head) * HD;
-#pragma unroll
-  for (int dt = 0; dt < DT; dt++)
-#pragma unroll
-    for (int j = 0; j < 4; j++) {
-      const int d = dt * 32 + 8 * j + 4 * lk;
-      if (d < HD) {
-        bf16x4 w;
-#pragma unroll
-        for (int i = 0; i < 4; i++) w[i] = (__bf16)(o[dt][4 * j + i] * inv);
-        *(bf16x4*)(orow + d) = w;
-      }
-    }
-}
 
 // Joins the ranges of keys of a portion's rows (attn_shared_kernel, SPLIT), in their order: a
 // block of 64 threads per (32 channels of a wave of a block of rows, KV head, request), every
@@ -758,7 +67,7 @@ __global__ __launch_bounds__(64) void attn_portion_join_kernel(AttnParams p, int
   if (tok >= ntok) return;
   const int blk_lo = start + bi * per_block, blk_hi = start + min(n, (bi + 1) * per_block) - 1;
   const int key_lo = first_key(p, blk_lo);
-  const int ranges = (blk_hi / 32 - key_lo / 32) / p.chunk + 1;
+  const int ranges = (KeyTiles(p, key_lo, blk_hi).count - 1) / p.chunk + 1;
   const size_t slot0 = ((((size_t)blockIdx.z * p.nkv + kvh) * row_blocks + rows_x) * p.nchunks) * 4 + wave;
   float m = -INFINITY;
   for (int c = 0; c < ranges; c++) m = fmaxf(m, p.part_ml[(slot0 + (size_t)c * 4) * 128 + lr]);
@@ -776,204 +85,15 @@ __global__ __launch_bounds__(64) void attn_portion_join_kernel(AttnParams p, int
     for (int j = 0; j < 4; j++) acc[j] += w * po[j * 64];
   }
   const float inv = 1.f / (l + sink_weight(p, m));
-  __bf16* orow = p.out + ((size_t)(qs + t0 + tok) * p.nh + q_head_of(p, kvh, hq)) * p.hd;
+  __bf16* orow = p.out + ((size_t)(qs + t0 + tok) * p.nh + q_head_of(p, kvh, hq)) * p.vd;
 #pragma unroll
   for (int j = 0; j < 4; j++) {
     const int d = dt * 32 + 8 * j + 4 * lk;
-    if (d < p.hd) {
+    if (d < p.vd) {
       bf16x4 w4;
 #pragma unroll
       for (int i = 0; i < 4; i++) w4[i] = (__bf16)(acc[j][i] * inv);
       *(bf16x4*)(orow + d) = w4;
-    }
-  }
-}
-
-// One wave per (request, KV head, chunk of 64 keys) for requests that bring one token.
-// Columns of every tile are the g query heads of the KV head (col = lane % 16), rows are
-// keys (first product) or channels (second product).
-template <int HD32>
-__global__ __launch_bounds__(256, 2) void attn_decode_kernel(AttnParams p) {
-  constexpr int KS = HD32;       // 32-wide steps over head_dim
-  constexpr int DT = HD32 * 2;   // 16-channel output tiles
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int col = lane & 15, kq = lane >> 4;
-  const int r = p.r_begin + blockIdx.z;
-  const int kvh = blockIdx.y;
-  // Where the window is much shorter than the longest context, the grid covers a window's
-  // blocks only and counts them from the block the request's window begins in.
-  int block_x = blockIdx.x;
-  if (p.from_window) block_x += first_key(p, max(p.ctx_len[r] - 1, 0)) / (4 * p.chunk);
-  const int chunk = block_x * 4 + wave;
-  const int* table = p.block_table + (size_t)r * p.max_blocks;
-  const int hd = p.hd, bsh = p.bs_shift, bmask = p.bs - 1, nkv = p.nkv;
-  // The pages of the chunk's (up to two) tiles are asked for before the request's length is
-  // known, beside it: where a key lies follows from the chunk alone.  A key past the context is
-  // masked below; a hole in the table reads page 0, which the caller keeps cleared, and the
-  // places of a request's last page behind its last token are cleared too (a masked value
-  // still meets a weight of 0 in the second product, and 0 x NaN is NaN).
-  int kpage[2][2], vpage[2][2];
-#pragma unroll
-  for (int i = 0; i < 2; i++) {
-    const int k0 = chunk * p.chunk + 32 * i;
-#pragma unroll
-    for (int t = 0; t < 2; t++) {
-      kpage[i][t] = table[min((k0 + 16 * t + col) >> bsh, p.max_blocks - 1)];
-      vpage[i][t] = table[min((k0 + 16 * t + 4 * kq) >> bsh, p.max_blocks - 1)];
-    }
-  }
-  const int n = p.q_start[r + 1] - p.q_start[r];
-  if (n <= 0) return;
-  const int pos = p.ctx_len[r] - 1;
-  const int row_lo = first_key(p, pos);
-  // a block whose four chunks all lie past the context or before the window ends here, all
-  // its waves alike: the grid is sized for the longest context the caller allows
-  const int first_chunk = block_x * 4;
-  if (first_chunk * p.chunk > pos || first_chunk * p.chunk + 4 * p.chunk - 1 < row_lo) return;
-  const int key_lo = max(row_lo, chunk * p.chunk);
-  const int key_hi = min(pos, chunk * p.chunk + p.chunk - 1);
-  const bool active = key_lo <= key_hi;          // a wave without keys still meets the others at the barrier
-  const int g = p.nh / p.nkv;
-  const bool col_ok = col < g;
-  const int head = q_head_of(p, kvh, col_ok ? col : 0);
-  const int trow = p.q_start[r];
-
-  // the query operand waits in LDS (one 16-byte piece per lane and step), not in registers
-  __shared__ bf16x8 sq[4][KS][64];
-  {
-    const __bf16* qr = p.q + (size_t)trow * p.q_stride + (size_t)head * hd + kq * 8;
-#pragma unroll
-    for (int ks = 0; ks < KS; ks++) {
-      bf16x8 t;
-      if (col_ok) t = *(const bf16x8*)(qr + ks * 32);
-      else
-#pragma unroll
-        for (int e = 0; e < 8; e++) t[e] = (__bf16)0.f;
-      sq[wave][ks][lane] = t;
-    }
-  }
-  f32x4 o[DT];
-#pragma unroll
-  for (int dt = 0; dt < DT; dt++) o[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float m_run = -INFINITY, l_run = 0.f;
-
-#pragma unroll
-  for (int i = 0; i < 2; i++) {
-    const int key0 = chunk * p.chunk + 32 * i;
-    if (!active || 32 * i >= p.chunk || key0 > key_hi || key0 + 31 < key_lo) continue;
-    bf16x8 kf[2][KS];
-#pragma unroll
-    for (int t = 0; t < 2; t++) {
-      const int kk = key0 + 16 * t + col;
-      const int page = max(kpage[i][t], 0);
-      const __bf16* kr = p.kcache + ((((size_t)page * nkv + kvh) << bsh) + (kk & bmask)) * hd + kq * 8;
-#pragma unroll
-      for (int ks = 0; ks < KS; ks++) kf[t][ks] = *(const bf16x8*)(kr + ks * 32);
-    }
-    bf16x8 vf[DT];
-    {
-      const int ka = key0 + 4 * kq, kb = key0 + 16 + 4 * kq;
-      const int pa = max(vpage[i][0], 0), pb = max(vpage[i][1], 0);
-      const __bf16* va_base = p.vcache + ((((size_t)pa * (nkv >> p.v_shift) + (kvh >> p.v_shift)) * hd) << bsh) + (ka & bmask);
-      const __bf16* vb_base = p.vcache + ((((size_t)pb * (nkv >> p.v_shift) + (kvh >> p.v_shift)) * hd) << bsh) + (kb & bmask);
-#pragma unroll
-      for (int dt = 0; dt < DT; dt++) {
-        const int d = dt * 16 + col;
-        const bf16x4 va = *(const bf16x4*)(va_base + ((size_t)d << bsh));
-        const bf16x4 vb = *(const bf16x4*)(vb_base + ((size_t)d << bsh));
-#pragma unroll
-        for (int e = 0; e < 4; e++) {
-          vf[dt][e] = va[e];
-          vf[dt][4 + e] = vb[e];
-        }
-      }
-    }
-    f32x4 s[2];
-#pragma unroll
-    for (int t = 0; t < 2; t++) {
-      s[t] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int ks = 0; ks < KS; ks++) s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[t][ks], sq[wave][ks][lane], s[t], 0, 0, 0);
-    }
-    float mt = -INFINITY;
-#pragma unroll
-    for (int t = 0; t < 2; t++)
-#pragma unroll
-      for (int i = 0; i < 4; i++) {
-        const int key = key0 + 16 * t + 4 * kq + i;
-        float v = score_log2(p, s[t][i]);
-        v = (col_ok && key >= key_lo && key <= key_hi) ? v : -INFINITY;
-        s[t][i] = v;
-        mt = fmaxf(mt, v);
-      }
-    mt = fmaxf(mt, __shfl_xor(mt, 16, 64));
-    mt = fmaxf(mt, __shfl_xor(mt, 32, 64));
-    const float m_new = fmaxf(m_run, mt);
-    const float m_use = m_new == -INFINITY ? 0.f : m_new;
-    const float corr = __builtin_amdgcn_exp2f(m_run - m_use);
-    float rs = 0.f;
-    bf16x8 pb8;
-#pragma unroll
-    for (int t = 0; t < 2; t++)
-#pragma unroll
-      for (int i = 0; i < 4; i++) {
-        const float pe = __builtin_amdgcn_exp2f(s[t][i] - m_use);
-        rs += pe;
-        pb8[4 * t + i] = (__bf16)pe;
-        s[t][i] = pe;
-      }
-    rs += __shfl_xor(rs, 16, 64);
-    rs += __shfl_xor(rs, 32, 64);
-    l_run = l_run * corr + rs;
-    m_run = m_new;
-#pragma unroll
-    for (int dt = 0; dt < DT; dt++) {
-      o[dt] *= corr;
-      o[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[dt], pb8, o[dt], 0, 0, 0);
-    }
-    if (p.wide_weights) {
-#pragma unroll
-      for (int t = 0; t < 2; t++)
-#pragma unroll
-        for (int i = 0; i < 4; i++) pb8[4 * t + i] = (__bf16)(s[t][i] - (float)pb8[4 * t + i]);
-#pragma unroll
-      for (int dt = 0; dt < DT; dt++) o[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[dt], pb8, o[dt], 0, 0, 0);
-    }
-  }
-  // the block's four chunks are joined here, in chunk order: one partial result per 256 keys
-  extern __shared__ float dyn[];
-  float* sm_ml = dyn;                 // [4][16][2]
-  float* sm_o = dyn + 4 * 16 * 2;     // [4][g][hd]
-  if (col_ok) {
-    if (kq == 0) {
-      sm_ml[(wave * 16 + col) * 2] = m_run;
-      sm_ml[(wave * 16 + col) * 2 + 1] = l_run;
-    }
-    float* so = sm_o + ((size_t)wave * g + col) * hd;
-#pragma unroll
-    for (int dt = 0; dt < DT; dt++) *(f32x4*)(so + dt * 16 + 4 * kq) = o[dt];
-  }
-  __syncthreads();
-  for (int idx = threadIdx.x; idx < g * hd; idx += 256) {
-    const int c = idx / hd, d = idx - c * hd;
-    float mw[4], m = -INFINITY;
-#pragma unroll
-    for (int w = 0; w < 4; w++) {
-      mw[w] = sm_ml[(w * 16 + c) * 2];
-      m = fmaxf(m, mw[w]);
-    }
-    float acc = 0.f, l = 0.f;
-#pragma unroll
-    for (int w = 0; w < 4; w++) {
-      const float e = mw[w] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(mw[w] - m);
-      acc += e * sm_o[((size_t)w * g + c) * hd + d];
-      l += e * sm_ml[(w * 16 + c) * 2 + 1];
-    }
-    const size_t slot = ((size_t)(r - p.r_begin) * p.nh + q_head_of(p, kvh, c)) * p.nchunks + block_x;
-    p.part_o[slot * hd + d] = acc;
-    if (d == 0) {
-      p.part_ml[slot * 2] = m;
-      p.part_ml[slot * 2 + 1] = l;
     }
   }
 }
@@ -987,7 +107,7 @@ __global__ __launch_bounds__(256) void attn_combine_kernel(const float* __restri
                                                            const int* __restrict__ ctx_len,
                                                            __bf16* __restrict__ out, int nh, int hd,
                                                            int window, int r_begin, int nchunks, int span,
-                                                           int mask_chunk, int sink) {
+                                                           int mask_chunk, int sink, int keep) {
   __shared__ float wgt[ATT_MAX_CHUNKS];
   __shared__ float red[17];
   const int rr = blockIdx.x, head = blockIdx.y;
@@ -996,37 +116,40 @@ __global__ __launch_bounds__(256) void attn_combine_kernel(const float* __restri
   if (n <= 0) return;
   const int pos = ctx_len[r] - 1;
   const int lo = mask_chunk > 0 ? pos - pos % mask_chunk : window > 0 ? max(0, pos - window + 1) : 0;
-  const int c0 = lo / span, c1 = pos / span;
+  // the parts of the kept first keys, [0, kept), then those from the window's first on, [c0, c1]
+  const int c0 = lo / span, c1 = pos / span, kept = min((keep + span - 1) / span, c0);
+  auto part_of = [&](int i) { return i < kept ? i : c0 + i - kept; };
   const size_t base = ((size_t)rr * nh + head) * nchunks;
-  const int np = c1 - c0 + 1;
+  const int np = kept + c1 - c0 + 1;
   // the first partial results of the thread's channel are asked for now: they come in while
   // the weights are worked out (a part past the last is read from the last and not used)
   constexpr int PF = 16;
   const int d0 = min((int)threadIdx.x, hd - 1);
   float pf[PF];
   {
-    const float* po = part_o + (base + c0) * hd + d0;
+    const float* po = part_o + base * hd + d0;
 #pragma unroll
-    for (int c = 0; c < PF; c++) pf[c] = po[(size_t)min(c, np - 1) * hd];
+    for (int c = 0; c < PF; c++) pf[c] = po[(size_t)part_of(min(c, np - 1)) * hd];
   }
   float m = -INFINITY;
-  for (int c = c0 + threadIdx.x; c <= c1; c += 256) m = fmaxf(m, part_ml[(base + c) * 2]);
+  for (int c = threadIdx.x; c < np; c += 256) m = fmaxf(m, part_ml[(base + part_of(c)) * 2]);
   m = wave_max(m);
   if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = m;
   __syncthreads();
   m = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
   __syncthreads();
   float l = 0.f;
-  for (int c = c0 + threadIdx.x; c <= c1; c += 256) {
-    const float w = __builtin_amdgcn_exp2f(part_ml[(base + c) * 2] - m);
-    wgt[c - c0] = w;
-    l += part_ml[(base + c) * 2 + 1] * w;
+  for (int c = threadIdx.x; c < np; c += 256) {
+    const size_t at = (base + part_of(c)) * 2;
+    const float w = __builtin_amdgcn_exp2f(part_ml[at] - m);
+    wgt[c] = w;
+    l += part_ml[at + 1] * w;
   }
   l = block_sum(l, red);
   const float inv = 1.f / (l + (sink ? __builtin_amdgcn_exp2f(-m) : 0.f));
   __bf16* orow = out + ((size_t)q_start[r] * nh + head) * hd;
   for (int d = threadIdx.x; d < hd; d += 256) {
-    const float* po = part_o + (base + c0) * hd + d;
+    const float* po = part_o + base * hd + d;
     float acc = 0.f;
     int c = 0;
     if (d == d0) {                      // the channel whose first parts are here already
@@ -1036,58 +159,26 @@ __global__ __launch_bounds__(256) void attn_combine_kernel(const float* __restri
       c = min(np, PF);
     }
     for (; c + 4 <= np; c += 4) {       // four loads in flight, summed in part order
-      const float v0 = po[(size_t)c * hd], v1 = po[(size_t)(c + 1) * hd];
-      const float v2 = po[(size_t)(c + 2) * hd], v3 = po[(size_t)(c + 3) * hd];
+      const float v0 = po[(size_t)part_of(c) * hd], v1 = po[(size_t)part_of(c + 1) * hd];
+      const float v2 = po[(size_t)part_of(c + 2) * hd], v3 = po[(size_t)part_of(c + 3) * hd];
       acc += v0 * wgt[c];
       acc += v1 * wgt[c + 1];
       acc += v2 * wgt[c + 2];
       acc += v3 * wgt[c + 3];
     }
-    for (; c < np; c++) acc += po[(size_t)c * hd] * wgt[c];
+    for (; c < np; c++) acc += po[(size_t)part_of(c) * hd] * wgt[c];
     orow[d] = (__bf16)(acc * inv);
   }
 }
 
-template <bool SPLIT, bool PAIR>
-static int launch_attn(const AttnParams& p, dim3 grid, hipStream_t s) {
-  // the join of a portion's four waves needs [4][32][2] + [2][ceil(hd/32) * 16][64] floats of LDS
-  const size_t lds = SPLIT ? 0 : (4 * 32 * 2 + (size_t)2 * ((p.hd + 31) / 32) * 16 * 64) * sizeof(float);
+static int launch_attn(int what, const AttnParams& p, dim3 grid, hipStream_t s) {
+  if (p.vd != p.hd) return attn_launch_uneven(what, p, grid, s);
   switch (p.hd / 16) {
-    case 1: attn_mfma_kernel<1, SPLIT, PAIR><<<grid, 256, lds, s>>>(p); break;
-    case 2: attn_mfma_kernel<2, SPLIT, PAIR><<<grid, 256, lds, s>>>(p); break;
-    case 4: attn_mfma_kernel<4, SPLIT, PAIR><<<grid, 256, lds, s>>>(p); break;
-    case 8: attn_mfma_kernel<8, SPLIT, PAIR><<<grid, 256, lds, s>>>(p); break;
-    case 16: attn_mfma_kernel<16, SPLIT, PAIR><<<grid, 256, lds, s>>>(p); break;
-    default: return zk_fail("zk_attention_bf16: head_dim must be 16, 32, 64, 128 or 256");
-  }
-  return zk_launch_status("zk_attention_bf16");
-}
-
-template <int HD16, int NW, bool SPLIT>
-static int launch_shared_one(const AttnParams& p, dim3 grid, hipStream_t s) {
-  constexpr int HD = HD16 * 16;
-  constexpr size_t lds = ((size_t)2 * 32 * (HD + 8) + (size_t)2 * HD * (32 + 8)) * sizeof(__bf16);
-  static bool prepared = false;
-  if (!prepared) {
-    if (lds > 64 * 1024 && hipFuncSetAttribute((const void*)attn_shared_kernel<HD16, NW, SPLIT>,
-                                               hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
-      return zk_fail("zk_attention_bf16: the shared-tile kernel's LDS buffers were refused");
-    prepared = true;
-  }
-  attn_shared_kernel<HD16, NW, SPLIT><<<grid, NW * 64, lds, s>>>(p);
-  return zk_launch_status("zk_attention_bf16 (shared tiles)");
-}
-
-template <int NW, bool SPLIT>
-static int launch_shared(const AttnParams& p, dim3 grid, hipStream_t s) {
-  switch (p.hd / 16) {
-    case 1: return launch_shared_one<1, NW, SPLIT>(p, grid, s);
-    case 2: return launch_shared_one<2, NW, SPLIT>(p, grid, s);
-    case 4: return launch_shared_one<4, NW, SPLIT>(p, grid, s);
-    case 8: return launch_shared_one<8, NW, SPLIT>(p, grid, s);
-    case 16:
-      if constexpr (NW <= 4) return launch_shared_one<16, NW, SPLIT>(p, grid, s);
-      else return zk_fail("zk_attention_bf16: eight waves a block take head sizes up to 128");
+    case 1: return launch_sizes<1, 1>(what, p, grid, s);
+    case 2: return launch_sizes<2, 2>(what, p, grid, s);
+    case 4: return launch_sizes<4, 4>(what, p, grid, s);
+    case 8: return launch_sizes<8, 8>(what, p, grid, s);
+    case 16: return launch_sizes<16, 16>(what, p, grid, s);
     default: return zk_fail("zk_attention_bf16: head_dim must be 16, 32, 64, 128 or 256");
   }
 }
@@ -1107,13 +198,13 @@ static size_t portion_split_bytes(long row_blocks, int nkv, int hd, int ranges) 
 // results).  No split unless it at least halves the longest block's tiles; at most
 // ATT_MOST_RANGES ranges for the longest block of rows the caller's limits allow (bound_tiles),
 // which bounds the workspace.
-static int portion_ranges(int max_q_len, int max_ctx, int window, int mask_chunk, int per_block, int nkv, int r_prefill,
-                          int bound_tiles) {
+static int portion_ranges(int max_q_len, int max_ctx, int window, int mask_chunk, int keep, int per_block, int nkv,
+                          int r_prefill, int bound_tiles) {
   const int row_blocks = (max_q_len + per_block - 1) / per_block;
   auto tiles_of = [&](int bi) {
     const int lo = max_ctx - max_q_len + bi * per_block, hi = std::min(max_ctx, lo + per_block) - 1;
     const int klo = mask_chunk > 0 ? lo - lo % mask_chunk : window > 0 ? std::max(0, lo - window + 1) : 0;
-    return hi / 32 - klo / 32 + 1;
+    return std::min((keep + 31) / 32, klo / 32) + hi / 32 - klo / 32 + 1;
   };
   int longest = 0;
   for (int bi = 0; bi < row_blocks; bi++) longest = std::max(longest, tiles_of(bi));
@@ -1150,6 +241,12 @@ int zk_attention_bf16_supports(int nh, int nkv, int hd, int bs) {
   const int g = nh / nkv;
   const bool hd_ok = hd == 16 || hd == 32 || hd == 64 || hd == 128 || hd == 256;
   return hd_ok && g <= 32 && bs >= 4 && (bs & (bs - 1)) == 0;
+}
+
+// The same for heads whose values have vd channels: as wide as keys, half or twice as wide.
+int zk_attention_bf16_supports_values(int nh, int nkv, int hd, int vd, int bs) {
+  return zk_attention_bf16_supports(nh, nkv, hd, bs) && (vd == hd || (zk_attention_bf16_supports(nh, nkv, vd, bs) &&
+                                                                     (vd == 2 * hd || hd == 2 * vd)));
 }
 
 // Bytes of workspace the split variant needs for ``n_decode`` single-token requests.
@@ -1192,17 +289,22 @@ long long zk_attention_bf16_max_context(int nh, int nkv, int hd, int decode_chun
 // wide_weights: the weights keep 16 bits of mantissa in the product with the values.
 // v_shift: 2^v_shift neighbouring key heads read the values of one value head (the value cache
 // then holds nkv >> v_shift heads): several maps of keys over the same values.
-int zk_attention_bf16_maps(const void* q, int q_stride, const void* kcache, const void* vcache_t,
+// vd: channels of a value and of the output's heads (hd, hd / 2 or 2 hd); the workspace functions above
+// are asked with vd for their hd.  keep (with a window): a row sees the first ``keep`` keys of its sequence
+// beside its window; the caller keeps their pages.
+int zk_attention_bf16_sized(const void* q, int q_stride, const void* kcache, const void* vcache_t,
                            const int* block_table, int max_blocks, const int* q_start, const int* ctx_len,
                            void* out, int R, int r_prefill, int max_q_len, int max_ctx, int nh, int nkv,
                            int hd, int bs, float scale, float softcap, int window, int decode_chunk,
                            void* workspace, size_t workspace_bytes, int mask_chunk, int sink, int wide_weights,
-                           int v_shift, void* stream) {
+                           int v_shift, int vd, int keep, void* stream) {
+  ZK_REQUIRE(keep >= 0 && (keep == 0 || window > 0), "zk_attention_bf16: first keys are kept beside a window");
   ZK_REQUIRE(v_shift >= 0 && v_shift <= 4 && nkv % (1 << v_shift) == 0, "zk_attention_bf16: key heads in whole groups of a value head");
   ZK_REQUIRE(mask_chunk >= 0 && (mask_chunk == 0 || window == 0), "zk_attention_bf16: a window or a chunk, not both");
   ZK_REQUIRE(R >= 0 && r_prefill >= 0 && r_prefill <= R, "zk_attention_bf16: bad request counts");
-  ZK_REQUIRE(zk_attention_bf16_supports(nh, nkv, hd, bs), "zk_attention_bf16: sizes not supported "
-             "(head_dim 16/32/64/128/256, at most 32 heads a KV head, page size a power of two from 4)");
+  ZK_REQUIRE(zk_attention_bf16_supports_values(nh, nkv, hd, vd, bs), "zk_attention_bf16: sizes not supported "
+             "(head_dim 16/32/64/128/256, values as wide, half or twice as wide, at most 32 heads a KV head, page size a power of "
+             "two from 4)");
   ZK_REQUIRE(q_stride >= nh * hd && q_stride % 8 == 0 && ((uintptr_t)q % 16 == 0),
              "zk_attention_bf16: q rows must be 16-byte aligned");
   ZK_REQUIRE(max_blocks > 0 && nkv <= 65535 && R <= 65535, "zk_attention_bf16: grid too large");
@@ -1214,7 +316,7 @@ int zk_attention_bf16_maps(const void* q, int q_stride, const void* kcache, cons
     ZK_REQUIRE(max_ctx > 0, "zk_attention_bf16: max_ctx must be positive");
     ZK_REQUIRE(max_ctx <= zk_attention_bf16_max_context(nh, nkv, hd, decode_chunk),
                "zk_attention_bf16: context too long for the split variant");
-    ZK_REQUIRE(zk_attention_bf16_workspace(R - r_prefill, nh, hd, max_ctx) <= workspace_bytes,
+    ZK_REQUIRE(zk_attention_bf16_workspace(R - r_prefill, nh, vd, max_ctx) <= workspace_bytes,
                "zk_attention_bf16: workspace too small for the split partial results");
   }
   if (r_prefill > 0) ZK_REQUIRE(max_q_len > 0, "zk_attention_bf16: max_q_len must be positive");
@@ -1224,7 +326,7 @@ int zk_attention_bf16_maps(const void* q, int q_stride, const void* kcache, cons
   p.kcache = (const __bf16*)kcache; p.vcache = (const __bf16*)vcache_t; p.v_shift = v_shift;
   p.block_table = block_table; p.max_blocks = max_blocks;
   p.q_start = q_start; p.ctx_len = ctx_len; p.out = (__bf16*)out;
-  p.nh = nh; p.nkv = nkv; p.hd = hd; p.bs = bs;
+  p.nh = nh; p.nkv = nkv; p.hd = hd; p.vd = vd; p.bs = bs; p.keep = keep;
   p.scale = scale; p.softcap = softcap; p.window = window;
   p.from_window = 0;
   p.mask_chunk = mask_chunk; p.sink = sink ? 1 : 0; p.wide_weights = wide_weights ? 1 : 0;
@@ -1234,7 +336,7 @@ int zk_attention_bf16_maps(const void* q, int q_stride, const void* kcache, cons
   p.k1 = scale * log2e;
   p.k2 = softcap > 0.f ? 2.f * scale / softcap * log2e : 0.f;
   p.c2 = softcap * log2e;
-  const int g = nh / nkv;
+  const int g = nh / nkv, wide = std::max(hd, vd);
   if (r_prefill > 0) {
     p.tpw = 32 / g; p.r_begin = 0; p.nchunks = 1; p.part_o = nullptr; p.part_ml = nullptr;
     const int groups = (max_q_len + p.tpw - 1) / p.tpw;
@@ -1252,9 +354,9 @@ int zk_attention_bf16_maps(const void* q, int q_stride, const void* kcache, cons
     int shared_waves = 0;
     if (bs >= 8 && portion_kernel_mode != 1) {
       if (portion_kernel_mode > 1) shared_waves = portion_kernel_mode;
-      else if (single >= 4096 && hd <= 128) shared_waves = 8;
+      else if (single >= 4096 && wide <= 128) shared_waves = 8;
       else if (single >= 768) shared_waves = 4;
-      if (shared_waves == 8 && hd > 128) shared_waves = 4;       // no room for two waves a SIMD
+      if (shared_waves == 8 && wide > 128) shared_waves = 4;       // no room for two waves a SIMD
     }
     // Few blocks of rows with many keys each (a portion of a few hundred rows behind thousands of
     // tokens): four groups a block and the keys in ranges, where the workspace behind the decoded
@@ -1270,12 +372,12 @@ int zk_attention_bf16_maps(const void* q, int q_stride, const void* kcache, cons
       int bound = (max_ctx + 31) / 32;
       // (a chunk's rows see no more keys than a window of its size would show them)
       const int reach = mask_chunk > 0 ? mask_chunk : window;
-      if (reach > 0) bound = std::min(bound, (reach + per_block + 31) / 32 + 1);
-      range_tiles = portion_ranges(max_q_len, max_ctx, window, mask_chunk, per_block, nkv, r_prefill, bound);
+      if (reach > 0) bound = std::min(bound, (reach + per_block + 31) / 32 + 1 + (keep + 31) / 32);
+      range_tiles = portion_ranges(max_q_len, max_ctx, window, mask_chunk, keep, per_block, nkv, r_prefill, bound);
       if (range_tiles) {
         most_ranges = (bound + range_tiles - 1) / range_tiles;
-        if (R - r_prefill > 0) split_at = (zk_attention_bf16_workspace(R - r_prefill, nh, hd, max_ctx) + 255) / 256 * 256;
-        const size_t need = portion_split_bytes((long)r_prefill * ((max_q_len + per_block - 1) / per_block), nkv, hd,
+        if (R - r_prefill > 0) split_at = (zk_attention_bf16_workspace(R - r_prefill, nh, vd, max_ctx) + 255) / 256 * 256;
+        const size_t need = portion_split_bytes((long)r_prefill * ((max_q_len + per_block - 1) / per_block), nkv, vd,
                                                 most_ranges);
         if (workspace == nullptr || (uintptr_t)workspace % 16 != 0 || split_at + need > workspace_bytes)
           range_tiles = 0;
@@ -1288,20 +390,20 @@ int zk_attention_bf16_maps(const void* q, int q_stride, const void* kcache, cons
       ps.nchunks = most_ranges;
       const int row_blocks = (max_q_len + per_block - 1) / per_block;
       const size_t slots = (size_t)r_prefill * nkv * row_blocks * most_ranges * 4;
-      const int dts = (hd + 31) / 32;
+      const int dts = (vd + 31) / 32;
       ps.part_o = (float*)((char*)workspace + split_at);
       ps.part_ml = ps.part_o + slots * dts * 16 * 64;
       dim3 grid(row_blocks * most_ranges, nkv, r_prefill);
-      rc = launch_shared<4, true>(ps, grid, s);
+      rc = launch_attn(ATT_RANGES, ps, grid, s);
       if (rc) return rc;
       attn_portion_join_kernel<<<dim3(row_blocks * 4 * dts, nkv, r_prefill), 64, 0, s>>>(ps, per_block, row_blocks, dts);
       rc = zk_launch_status("zk_attention_bf16 (join of the portions' ranges)");
     } else if (shared_waves) {
       if (shared_waves == 5) shared_waves = 4;
       dim3 grid((groups + shared_waves - 1) / shared_waves, nkv, r_prefill);
-      rc = shared_waves == 4 ? launch_shared<4, false>(p, grid, s) : launch_shared<8, false>(p, grid, s);
-    } else if (single > 256 && paired <= 256) rc = launch_attn<false, true>(p, dim3((groups + 1) / 2, nkv, r_prefill), s);
-    else rc = launch_attn<false, false>(p, dim3(groups, nkv, r_prefill), s);
+      rc = launch_attn(shared_waves == 4 ? ATT_SHARED4 : ATT_SHARED8, p, grid, s);
+    } else if (single > 256 && paired <= 256) rc = launch_attn(ATT_PAIRS, p, dim3((groups + 1) / 2, nkv, r_prefill), s);
+    else rc = launch_attn(ATT_GROUPS, p, dim3(groups, nkv, r_prefill), s);
     if (rc) return rc;
   }
   const int n_dec = R - r_prefill;
@@ -1309,7 +411,7 @@ int zk_attention_bf16_maps(const void* q, int q_stride, const void* kcache, cons
     const int nchunks = (max_ctx + ATT_CHUNK - 1) / ATT_CHUNK;
     p.tpw = 1; p.r_begin = r_prefill; p.nchunks = nchunks;
     p.part_o = (float*)workspace;
-    p.part_ml = (float*)workspace + (size_t)n_dec * nh * nchunks * hd;
+    p.part_ml = (float*)workspace + (size_t)n_dec * nh * nchunks * vd;
     dim3 grid((nchunks + 3) / 4, nkv, n_dec);
     int rc = 0;
     int span = ATT_CHUNK;        // keys one partial result covers
@@ -1324,30 +426,34 @@ int zk_attention_bf16_maps(const void* q, int q_stride, const void* kcache, cons
       p.nchunks = grid.x;
       // a window covers at most ceil(window / span) + 1 blocks of span keys
       const int reach = mask_chunk > 0 ? mask_chunk : window;
-      const int window_blocks = reach > 0 ? (reach + span - 1) / span + 1 : 0;
+      const int window_blocks = reach > 0 ? (reach + span - 1) / span + 1 + (keep + span - 1) / span : 0;
       if (reach > 0 && window_blocks < (int)grid.x) {
         p.from_window = 1;
         grid.x = window_blocks;
       }
-      p.part_ml = (float*)workspace + (size_t)n_dec * nh * p.nchunks * hd;
-      const size_t lds = (4 * 16 * 2 + (size_t)4 * g * hd) * sizeof(float);
-      switch (hd / 32) {
-        case 1: attn_decode_kernel<1><<<grid, 256, lds, s>>>(p); break;
-        case 2: attn_decode_kernel<2><<<grid, 256, lds, s>>>(p); break;
-        case 4: attn_decode_kernel<4><<<grid, 256, lds, s>>>(p); break;
-        default: attn_decode_kernel<8><<<grid, 256, lds, s>>>(p); break;
-      }
-      rc = zk_launch_status("zk_attention_bf16 (decode)");
+      p.part_ml = (float*)workspace + (size_t)n_dec * nh * p.nchunks * vd;
+      rc = launch_attn(ATT_DECODE, p, grid, s);
     } else {
-      rc = launch_attn<true, false>(p, grid, s);
+      rc = launch_attn(ATT_DECODE_WIDE, p, grid, s);
     }
     if (rc) return rc;
     dim3 cgrid(n_dec, nh);
-    attn_combine_kernel<<<cgrid, 256, 0, s>>>(p.part_o, p.part_ml, q_start, ctx_len, (__bf16*)out, nh, hd,
-                                              window, r_prefill, p.nchunks, span, mask_chunk, sink);
+    attn_combine_kernel<<<cgrid, 256, 0, s>>>(p.part_o, p.part_ml, q_start, ctx_len, (__bf16*)out, nh, vd,
+                                              window, r_prefill, p.nchunks, span, mask_chunk, sink, keep);
     return zk_launch_status("zk_attention_bf16 (combine)");
   }
   return 0;
+}
+
+int zk_attention_bf16_maps(const void* q, int q_stride, const void* kcache, const void* vcache_t,
+                           const int* block_table, int max_blocks, const int* q_start, const int* ctx_len,
+                           void* out, int R, int r_prefill, int max_q_len, int max_ctx, int nh, int nkv,
+                           int hd, int bs, float scale, float softcap, int window, int decode_chunk,
+                           void* workspace, size_t workspace_bytes, int mask_chunk, int sink, int wide_weights,
+                           int v_shift, void* stream) {
+  return zk_attention_bf16_sized(q, q_stride, kcache, vcache_t, block_table, max_blocks, q_start, ctx_len, out, R,
+                                 r_prefill, max_q_len, max_ctx, nh, nkv, hd, bs, scale, softcap, window, decode_chunk,
+                                 workspace, workspace_bytes, mask_chunk, sink, wide_weights, v_shift, hd, 0, stream);
 }
 
 int zk_attention_bf16_masked(const void* q, int q_stride, const void* kcache, const void* vcache_t,
@@ -1377,6 +483,10 @@ extern "C" int zk_steplist_register(const char* name, int nargs, void* fn);
 static const int zk_attention_bf16_masked_entered = zk_steplist_register(
     "zk_attention_bf16_masked", zk_packed::Call<zk_attention_bf16_masked>::nargs,
     (void*)zk_packed::Call<zk_attention_bf16_masked>::call);
+
+static const int zk_attention_bf16_sized_entered = zk_steplist_register(
+    "zk_attention_bf16_sized", zk_packed::Call<zk_attention_bf16_sized>::nargs,
+    (void*)zk_packed::Call<zk_attention_bf16_sized>::call);
 
 static const int zk_attention_bf16_maps_entered = zk_steplist_register(
     "zk_attention_bf16_maps", zk_packed::Call<zk_attention_bf16_maps>::nargs,

@@ -191,14 +191,11 @@ class PagedAttention(Part):
     PORTION_RANGES_BYTES = 192 << 20
 
     def wants_v_transposed(self, kernels, dtype: str, page_size: int) -> bool:
-        """The matrix-core kernel reads V as [page][kv head][hd][bs]."""
+        """The matrix-core kernel reads V as [page][kv head][value channel][bs]; it takes values as wide as
+        keys, half or twice as wide."""
         s = self.spec
-        if self.keep:
-            return False
-        if (self.chunk or self.unit_sink or self.wide_weights) and not kernels.has("zk_attention_bf16_masked"):
-            return False
-        return bool(dtype == BF16 and self.value_dim == s.head_dim and kernels.has("zk_attention_bf16") and
-                    kernels.zk_attention_bf16_supports(s.num_heads, s.num_kv_heads, s.head_dim, page_size))
+        return bool(dtype == BF16 and kernels.has("zk_attention_bf16_sized") and
+                    kernels.zk_attention_bf16_supports_values(s.num_heads, s.num_kv_heads, s.head_dim, self.value_dim, page_size))
 
     def prepare(self, kernels, dtype, max_seqs, max_model_len, page_size, max_batch_tokens=0) -> int:
         """Workspace of the split attention of decoded tokens at the runner's limits, and the
@@ -216,13 +213,13 @@ class PagedAttention(Part):
             raise ValueError(f"attention with {s.num_heads} heads, {s.num_kv_heads} KV heads of "
                              f"{s.head_dim}: the longest context its decode kernel takes is {longest} "
                              f"tokens, the runner asks for {max_model_len}")
-        need = int(kernels.zk_attention_bf16_workspace(int(max_seqs), s.num_heads, s.head_dim, int(max_model_len)))
+        need = int(kernels.zk_attention_bf16_workspace(int(max_seqs), s.num_heads, self.value_dim, int(max_model_len)))
         # room for a launch of few, long portions to cut its keys into ranges: as much as a step's
         # tokens can ask for, but no more than PORTION_RANGES_BYTES (a launch that would need more
         # has blocks enough without the ranges, or runs on the kernels that need no workspace)
         if max_batch_tokens > 0 and kernels.has("zk_attention_bf16_portion_workspace"):
             extra = int(kernels.zk_attention_bf16_portion_workspace(int(max_batch_tokens), s.num_heads, s.num_kv_heads,
-                                                                    s.head_dim))
+                                                                    self.value_dim))
             need = (need + 255) // 256 * 256 + min(extra, self.PORTION_RANGES_BYTES)
         return need
 
@@ -285,29 +282,19 @@ class PagedAttention(Part):
         o = ctx.alloc((T, nh * vd))
         cap = float(s.softcap) if s.softcap else 0.0
         win = int(s.window) if s.window else 0
-        masked = bool(self.chunk or self.unit_sink or self.wide_weights or self.keep)
-        if masked and cache.v_transposed and ctx.tuned and vd == hd:
-            k.zk_attention_bf16_masked(qkv.ptr, width, cache.k.ptr, cache.v.ptr, g.block_table, g.max_blocks,
-                                       ctx.q_start, ctx.ctx_len, o.ptr, ctx.R, ctx.n_multi, ctx.max_q_len,
-                                       ctx.max_ctx, nh, nkv, hd, g.page_size, s.scale, cap, win,
-                                       self.decode_chunk, ctx.workspace.ptr, ctx.workspace.nbytes, self.chunk,
-                                       1 if self.unit_sink else 0, 1 if self.wide_weights else 0, ctx.stream)
-        elif masked:
-            k.zk_attention_plain_kept(qkv.ptr, width, cache.k.ptr, cache.v.ptr, g.block_table, g.max_blocks,
-                                        ctx.req_of_token, ctx.positions, o.ptr, T, nh, nkv, hd, vd, g.page_size, s.scale,
-                                        cap, win, 1 if cache.v_transposed else 0, vfreq, inter, None, 0, self.chunk,
-                                        1 if self.unit_sink else 0, self.keep, ctx.stream)
-        elif cache.v_transposed and ctx.tuned and vd == hd:
-            k.zk_attention_bf16(qkv.ptr, width, cache.k.ptr, cache.v.ptr, g.block_table, g.max_blocks,
-                                ctx.q_start, ctx.ctx_len, o.ptr, ctx.R, ctx.n_multi, ctx.max_q_len,
-                                ctx.max_ctx, nh, nkv, hd, g.page_size, s.scale, cap, win,
-                                self.decode_chunk, ctx.workspace.ptr, ctx.workspace.nbytes, ctx.stream)
+        if cache.v_transposed and ctx.tuned:
+            k.zk_attention_bf16_sized(qkv.ptr, width, cache.k.ptr, cache.v.ptr, g.block_table, g.max_blocks,
+                                      ctx.q_start, ctx.ctx_len, o.ptr, ctx.R, ctx.n_multi, ctx.max_q_len,
+                                      ctx.max_ctx, nh, nkv, hd, g.page_size, s.scale, cap, win,
+                                      self.decode_chunk, ctx.workspace.ptr, ctx.workspace.nbytes, self.chunk,
+                                      1 if self.unit_sink else 0, 1 if self.wide_weights else 0, 0, vd, self.keep, ctx.stream)
             if vfreq is not None:
                 k.zk_rotate_heads(o.ptr, ctx.positions, vfreq, T, nh, vd, inter, -1.0, ctx.stream)
         else:
-            k.zk_attention_plain_ext(qkv.ptr, width, cache.k.ptr, cache.v.ptr, g.block_table, g.max_blocks,
-                                     ctx.req_of_token, ctx.positions, o.ptr, T, nh, nkv, hd, vd, g.page_size, s.scale,
-                                     cap, win, 1 if cache.v_transposed else 0, vfreq, inter, ctx.stream)
+            k.zk_attention_plain_kept(qkv.ptr, width, cache.k.ptr, cache.v.ptr, g.block_table, g.max_blocks,
+                                      ctx.req_of_token, ctx.positions, o.ptr, T, nh, nkv, hd, vd, g.page_size, s.scale,
+                                      cap, win, 1 if cache.v_transposed else 0, vfreq, inter, None, 0, self.chunk,
+                                      1 if self.unit_sink else 0, self.keep, ctx.stream)
         if self.gate_name:
             # the heads times sigmoid(W_g x); the gate's columns lie behind the heads' in the product's rows
             k.zk_gate_heads(o.ptr, rows.ptr + heads_width * ITEMSIZE[ctx.dtype], row_width, T, nh * vd, ctx.stream)

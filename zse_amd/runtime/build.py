@@ -29,7 +29,7 @@ ARCH = "gfx950"
 COMMON_KERNELS = ["elementwise.hip", "gemm_plain.hip", "attention_plain.hip", "sampling.hip", "probe.hip", "steplist.hip",
                   "streams.hip", "headprep.hip", "mlstm.hip", "delta.hip", "moe.hip", "latent.hip", "residual.hip", "gla.hip", "scan.hip",
                   "pointwise.hip", "embed_pair.hip", "diffattn.hip", "sublayer.hip", "shortconv.hip", "gdelta.hip"]
-BF16_KERNELS = ["gemm_bf16.hip", "attention_bf16.hip"]
+BF16_KERNELS = ["gemm_bf16.hip", "attention_bf16.hip", "attention_bf16_uneven.hip"]
 
 LIBRARIES: Dict[str, dict] = {
     "runtime": {"sources": ["runtime.cpp"], "defines": [], "device": False},

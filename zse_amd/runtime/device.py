@@ -253,6 +253,8 @@ BF16_KERNEL_SIGNATURES = {
     "zk_latent_attention_bf16_window": [_VP, _VP, _VP, _I, _VP, _VP, _VP, _VP, _VP, _VP, _SZ, _I, _I, _I, _I, _I, _I, _I, _I, _F,
                                         _I, _I, _VP],
     "zk_moe_experts_grouped_ext": [_VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _F, _I, _I, _VP],
+    "zk_attention_bf16_sized": [_VP, _I, _VP, _VP, _VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I,
+                                _F, _F, _I, _I, _VP, _SZ, _I, _I, _I, _I, _I, _I, _VP],
     "zk_gdelta_token": [_VP, _I, _I, _I, _VP, _I, _VP, _VP, _VP, _VP, _I, _I, _VP, _VP, _VP, _VP, _I, _I, _I, _F, _VP],
 }
 
@@ -342,6 +344,9 @@ class KernelLibrary:
             self._dll.zk_attention_bf16_supports.restype = C.c_int
             self._dll.zk_attention_bf16_supports.argtypes = [_I, _I, _I, _I]
             self.zk_attention_bf16_supports = self._dll.zk_attention_bf16_supports
+            self._dll.zk_attention_bf16_supports_values.restype = C.c_int
+            self._dll.zk_attention_bf16_supports_values.argtypes = [_I, _I, _I, _I, _I]
+            self.zk_attention_bf16_supports_values = self._dll.zk_attention_bf16_supports_values
             self._dll.zk_attention_bf16_workspace.restype = C.c_size_t
             self._dll.zk_attention_bf16_workspace.argtypes = [_I, _I, _I, _I]
             self.zk_attention_bf16_workspace = self._dll.zk_attention_bf16_workspace
