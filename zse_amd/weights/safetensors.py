@@ -101,7 +101,7 @@ def f32_to_bf16_bits(x: np.ndarray) -> np.ndarray:
     nan = (u & 0x7FFFFFFF) > 0x7F800000
     rounded = (u + (0x7FFF + ((u >> 16) & 1))) >> 16
     rounded = np.where(nan, (u >> 16) | 0x40, rounded)
-    return rounded.astype(np.uint16)
+    return rounded.astype(np.uint16).reshape(np.shape(x))          # a number without axes keeps its shape
 
 
 def bf16_bits_to_f32(b: np.ndarray) -> np.ndarray:
