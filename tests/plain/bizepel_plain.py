@@ -233,13 +233,16 @@ def mixture(x, w, f, ml, dt, close=None):
     scores = sigmoid(x @ w[f + "router"].T.astype(dt))
     corr = w[f + "correction"].astype(dt)
     y = np.zeros_like(x)
+    share = np.zeros(scores.shape, dt)           # of every expert in every token; 0: not chosen
     for t in range(len(x)):
         ids = choose(scores[t], corr, ro["top"], ro.get("groups"))
-        weights = scores[t][ids] / (scores[t][ids].sum() + dt(1e-20)) * dt(ro.get("scale", 1.0))
-        for e, wt in zip(ids, weights):
-            y[t] += wt * expert(x[t:t + 1], w, f"{f}e{e}.", dt)[0]
+        share[t, ids] = scores[t][ids] / (scores[t][ids].sum() + dt(1e-20)) * dt(ro.get("scale", 1.0))
         if close is not None:
             close[t] = min(close[t], closeness(scores[t], corr, ro["top"], ro.get("groups")))
+    for e in range(ro["experts"]):
+        at = np.nonzero(share[:, e])[0]
+        if len(at):
+            y[at] += share[at, e][:, None] * expert(x[at], w, f"{f}e{e}.", dt)
     if ml.get("shared"):
         y += expert(x, w, f + "shared.", dt)
     return y
