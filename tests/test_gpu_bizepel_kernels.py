@@ -332,12 +332,14 @@ def test_decays_and_removal_rates(T, n, rank, dtype):
 DELTA_STEPS = ([150, 37], [70, 1], [1, 129], [1, 1], [1, 1], [6, 2])
 
 
-@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("H,D", [(3, 12), (2, 32), (2, 64), (1, 100), (2, 128), (1, 200), (1, 256)])
-def test_the_generalized_delta_rule_over_steps(H, D, dtype):
-    """Two requests over six steps, their states carried in slots; steps of single tokens on the kernel
-    of their own where there is one."""
+@pytest.mark.parametrize("dtype,how", [("float32", "walk"), ("bfloat16", "walk"), ("bfloat16", "chunks"), ("bfloat16", "chunks in passes")])
+@pytest.mark.parametrize("H,D", [(3, 12), (2, 32), (2, 64), (1, 100), (2, 128), (1, 200), (1, 256), (9, 32)])
+def test_the_generalized_delta_rule_over_steps(H, D, dtype, how):
+    """Two requests over six steps, their states carried in slots; in bfloat16 steps of single tokens on the kernel
+    of their own where there is one, and portions in chunks (with room for all of them, and for two at a time)."""
     rt, k = lib(dtype)
+    if "chunks" in how and not k.zk_gdelta_chunk_floats(D):
+        pytest.skip("head size not taken by the chunks")
     rng = np.random.default_rng(H * 1000 + D)
     total = [sum(s[r] for s in DELTA_STEPS) for r in range(2)]
     eps, offset = 1e-5, 16
@@ -346,7 +348,9 @@ def test_the_generalized_delta_rule_over_steps(H, D, dtype):
     data, want = [], []
     for n in total:
         r, kk, v, g = (bf16(rng.normal(size=(n, H, D))) for _ in range(4))
-        w, a = np.exp(-np.exp(-0.5) * P.sigmoid(rng.normal(-3, 2, (n, H, D)))), P.sigmoid(rng.normal(0, 2, (n, H, D)))
+        z = rng.normal(-3, 2, (n, H, D))
+        z[:, 0] = rng.normal(6, 3, (n, D))               # one head whose decays are about as strong as they can be
+        w, a = np.exp(-np.exp(-0.5) * P.sigmoid(z)), P.sigmoid(rng.normal(0, 2, (n, H, D)))
         data.append((r, kk, v, g, w, a))
         o = np.stack([P.general_delta_rule(*(x[:, h].astype(np.float64) for x in (r, kk, v, w, a)), np.float64)
                       for h in range(H)], axis=1)
@@ -363,6 +367,13 @@ def test_the_generalized_delta_rule_over_steps(H, D, dtype):
         if dtype == "bfloat16" and max(st) == 1 and k.zk_gdelta_token_supports(D):
             k.zk_gdelta_token(X.ptr, 4 * C, C, 2 * C, gate, 4 * C, W_.ptr, A_.ptr, up(rt, gain).ptr, state.ptr, slot_words, offset,
                               i32(rt, [5, 5]).ptr, i32(rt, [0, 1]).ptr, i32(rt, [1, 0]).ptr, out.ptr, T, H, D, eps, rt.stream)
+        elif "chunks" in how:
+            count = 2 if "passes" in how else -(-max(st) // 32)
+            floats = count * 2 * H * k.zk_gdelta_chunk_floats(D)
+            work = up(rt, np.full(floats, np.nan))
+            k.zk_gdelta_chunked(X.ptr, 4 * C, C, 2 * C, gate, 4 * C, W_.ptr, A_.ptr, up(rt, gain).ptr, state.ptr, slot_words, offset,
+                                i32(rt, [0, st[0], T]).ptr, i32(rt, [1, 0]).ptr, i32(rt, np.zeros(T)).ptr, out.ptr, raw.ptr, work.ptr,
+                                floats, T, 2, max(st), H, D, eps, rt.stream)
         else:
             k.zk_gdelta(X.ptr, 4 * C, C, 2 * C, gate, 4 * C, W_.ptr, A_.ptr, up(rt, gain).ptr, state.ptr, slot_words, offset,
                         i32(rt, [0, st[0], T]).ptr, i32(rt, [1, 0]).ptr, i32(rt, np.zeros(T)).ptr, out.ptr, raw.ptr, T, 2,

@@ -21,6 +21,19 @@
 //    only this one, a request's values are the same bits however its tokens are cut into steps.
 //  - single tokens (gdelta_token_kernel): a block a head, a thread a column's share of the rows, the
 //    state read and written in whole lines.
+//  - long portions (gdelta_chunk_kernel, gdelta_scan_kernel): chunks of 32 tokens as matrix products on the
+//    32-bit matrix cores.  With b_t the product of a chunk's decays up to token t (b_0 = 1; a decay is at least
+//    exp(-exp(-1/2)), so 1 / b stays below 3e8) and the rows
+//        B_t = u_t b_(t-1),   A_t = -(a_t u_t) / b_t,   K_t = k_t / b_t,   R_t = r_t b_t
+//    what the tokens of a chunk find along their keys is Y = B S_0 + L Y + M V with L = B A^T and
+//    M = B K^T below the diagonal, so with T = (I - L)^-1
+//        Y = (T B) S_0 + P V,                        P = T M
+//        O = (R + Q T B) S_0 + (N + Q P) V           Q = R A^T, N = R K^T up to the diagonal
+//        S = b_32 (S_0 + A^T (T B) S_0 + (K + P^T A)^T V)
+//    The first kernel makes, for all chunks side by side, everything that does not know S_0 or V and lays it
+//    out as the operands of the second, which goes through a request's chunks in order: a block a head and
+//    16 value channels, its waves sharing out the rows of S, which stays in the accumulators (the order
+//    in which they lie there is a valid order of contraction, so they are operands as they are).
 #include "common.h"
 #include "packed_call.h"
 
@@ -327,6 +340,412 @@ __global__ __launch_bounds__(1024) void gdelta_token_kernel(const act_t* __restr
 }
 #endif
 
+#if ZSE_ACT_BF16
+// ---- long portions, chunk by chunk
+typedef float gd_f4 __attribute__((ext_vector_type(4)));
+#define GD_CHUNK 32
+#define GD_SMALL 36                // the distance between rows of a 32 x 32 matrix in local memory
+
+__device__ __forceinline__ gd_f4 gd_mfma(float a, float b, gd_f4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+
+// What gdelta_chunk_kernel leaves for a (chunk, head), in floats: per 16 channels the operands T B, R + Q T B, A^T,
+// K + P^T A (two tiles of 64 lanes x 4 each), the three lower tiles of N + Q P, and b_32.
+template <int D>
+struct GdWork {
+  static constexpr int TILES = D / 16, PER_TILE = 4 * 2 * 64 * 4, N_AT = TILES * PER_TILE, B_AT = N_AT + 3 * 64 * 4;
+  static constexpr int FLOATS = B_AT + D;
+};
+
+// A block per (chunk, head, request), 8 waves.  Lane l of a wave has lr = l % 16 and g = l / 16: an operand's
+// row and its four places in a step of the contraction, or an accumulator's column and its rows 4 g + i.
+template <int D>
+__global__ __launch_bounds__(512) void gdelta_chunk_kernel(const act_t* __restrict__ rkv, int ld, int k_off,
+                                                           const float* __restrict__ decay, const float* __restrict__ rate,
+                                                           const int* __restrict__ q_start, int H, int first_chunk,
+                                                           float* __restrict__ work) {
+  constexpr int LD = D + 4, PARTS = 512 / D, PER = GD_CHUNK / PARTS, NT = D / 16;
+  using Wk = GdWork<D>;
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  float* Bm = lds;                               // [32][LD] each
+  float* Rm = Bm + GD_CHUNK * LD;
+  float* Am = Rm + GD_CHUNK * LD;
+  float* Km = Am + GD_CHUNK * LD;
+  float* Lm = Km + GD_CHUNK * LD;                // [32][GD_SMALL] each: L, then T
+  float* Mm = Lm + GD_CHUNK * GD_SMALL;
+  float* Qm = Mm + GD_CHUNK * GD_SMALL;
+  float* Nm = Qm + GD_CHUNK * GD_SMALL;
+  float* Pm = Nm + GD_CHUNK * GD_SMALL;
+  float* kn = Pm + GD_CHUNK * GD_SMALL;          // [32]
+  float* pp = kn + GD_CHUNK;                     // [PARTS][D]
+  const int h = blockIdx.y, r = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int lr = lane & 15, g = lane >> 4;
+  const int base = (first_chunk + blockIdx.x) * GD_CHUNK;
+  const int n = q_start[r + 1] - q_start[r];
+  if (base >= n) return;
+  const int m = min(GD_CHUNK, n - base), t0 = q_start[r] + base;
+  float* out = work + (((size_t)r * gridDim.x + blockIdx.x) * H + h) * Wk::FLOATS;
+
+  // key lengths, a wave four tokens
+  for (int t = wave; t < GD_CHUNK; t += 8) {
+    float ss = 0.f;
+    if (t < m)
+      for (int d = lane; d < D; d += 64) {
+        const float x = to_f32(rkv[(size_t)(t0 + t) * ld + k_off + (size_t)h * D + d]);
+        ss = fmaf(x, x, ss);
+      }
+    ss = wave_sum(ss);
+    if (lane == 0) kn[t] = sqrtf(ss + 1e-6f);
+  }
+  // the four scaled rows: a thread PER tokens of a channel; tokens past the portion's end change nothing (decay 1, rows 0)
+  {
+    const int d = tid % D, part = tid / D;
+    float w[PER], prod = 1.f;
+#pragma unroll
+    for (int i = 0; i < PER; i++) {
+      const int t = part * PER + i;
+      w[i] = t < m ? decay[((size_t)(t0 + t) * H + h) * D + d] : 1.f;
+      prod *= w[i];
+    }
+    pp[part * D + d] = prod;
+    __syncthreads();
+    float b = 1.f;
+    for (int q = 0; q < part; q++) b *= pp[q * D + d];
+#pragma unroll
+    for (int i = 0; i < PER; i++) {
+      const int t = part * PER + i;
+      float kk = 0.f, rr = 0.f, aa = 0.f;
+      if (t < m) {
+        const act_t* row = rkv + (size_t)(t0 + t) * ld + (size_t)h * D + d;
+        rr = to_f32(row[0]);
+        kk = to_f32(row[k_off]);
+        aa = rate[((size_t)(t0 + t) * H + h) * D + d];
+      }
+      const float u = kk / kn[t];
+      Bm[t * LD + d] = u * b;
+      b *= w[i];
+      const float ib = 1.0f / b;
+      Rm[t * LD + d] = rr * b;
+      Am[t * LD + d] = -(aa * u) * ib;
+      Km[t * LD + d] = kk * ib;
+    }
+    if (part == PARTS - 1) out[Wk::B_AT + d] = b;
+  }
+  __syncthreads();
+  // L, M, Q, N: a wave one of them and 16 of its rows
+  {
+    const int mt = wave >> 2;
+    const float* X = (wave & 1) ? Rm : Bm;
+    const float* Z = (wave & 2) ? Km : Am;
+    float* dst = (wave & 1) ? ((wave & 2) ? Nm : Qm) : ((wave & 2) ? Mm : Lm);
+    const int strict = (wave & 1) ? 0 : 1;
+    gd_f4 acc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+    for (int j = 0; j < NT; j++) {
+      const gd_f4 x = *(const gd_f4*)(X + (mt * 16 + lr) * LD + 16 * j + 4 * g);
+      const gd_f4 z0 = *(const gd_f4*)(Z + lr * LD + 16 * j + 4 * g);
+#pragma unroll
+      for (int i = 0; i < 4; i++) acc[0] = gd_mfma(x[i], z0[i], acc[0]);
+      if (mt == 1) {
+        const gd_f4 z1 = *(const gd_f4*)(Z + (16 + lr) * LD + 16 * j + 4 * g);
+#pragma unroll
+        for (int i = 0; i < 4; i++) acc[1] = gd_mfma(x[i], z1[i], acc[1]);
+      }
+    }
+#pragma unroll
+    for (int nt = 0; nt < 2; nt++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const int t = mt * 16 + 4 * g + i, c = nt * 16 + lr;
+        dst[t * GD_SMALL + c] = c + strict <= t ? acc[nt][i] : 0.f;
+      }
+  }
+  __syncthreads();
+  // T = (I - L)^-1: the two diagonal blocks by substitution, a lane a column, then T21 = T22 (L21 T11)
+  if (wave == 0) {
+    float x[16];
+    const int o = (lane >> 4 & 1) * 16, c = lane & 15;
+#pragma unroll
+    for (int t = 0; t < 16; t++) x[t] = t == c ? 1.f : 0.f;
+#pragma unroll
+    for (int s = 0; s < 15; s++)
+#pragma unroll
+      for (int t = s + 1; t < 16; t++) x[t] = fmaf(Lm[(o + t) * GD_SMALL + o + s], x[s], x[t]);
+    __builtin_amdgcn_wave_barrier();
+    if (lane < 32) {
+#pragma unroll
+      for (int t = 0; t < 16; t++) Lm[(o + t) * GD_SMALL + o + c] = x[t];
+    }
+    __threadfence_block();
+    __builtin_amdgcn_wave_barrier();
+    gd_f4 z = {0.f, 0.f, 0.f, 0.f}, t21 = {0.f, 0.f, 0.f, 0.f};
+    const gd_f4 l21 = *(const gd_f4*)(Lm + (16 + lr) * GD_SMALL + 4 * g);
+#pragma unroll
+    for (int i = 0; i < 4; i++) z = gd_mfma(l21[i], Lm[(4 * g + i) * GD_SMALL + lr], z);
+    const gd_f4 t22 = *(const gd_f4*)(Lm + (16 + lr) * GD_SMALL + 16 + 4 * g);
+#pragma unroll
+    for (int i = 0; i < 4; i++) t21 = gd_mfma(t22[i], z[i], t21);
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int i = 0; i < 4; i++) Lm[(16 + 4 * g + i) * GD_SMALL + lr] = t21[i];
+  }
+  __syncthreads();
+  // a tile of a lower triangular 32 x 32 product X Z, (mt, nt) with nt <= mt
+  auto lower = [&](const float* X, const float* Z, int mt, int nt, gd_f4 acc) {
+    for (int kt = nt; kt <= mt; kt++) {
+      const gd_f4 x = *(const gd_f4*)(X + (mt * 16 + lr) * GD_SMALL + 16 * kt + 4 * g);
+#pragma unroll
+      for (int i = 0; i < 4; i++) acc = gd_mfma(x[i], Z[(16 * kt + 4 * g + i) * GD_SMALL + 16 * nt + lr], acc);
+    }
+    return acc;
+  };
+  const int lower_m = wave % 3 > 0, lower_n = wave % 3 > 1;            // waves 0, 1, 2 (and 3, 4, 5): tiles (0, 0), (1, 0), (1, 1)
+  if (wave < 3) {
+    const gd_f4 acc = lower(Lm, Mm, lower_m, lower_n, gd_f4{0.f, 0.f, 0.f, 0.f});
+#pragma unroll
+    for (int i = 0; i < 4; i++) Pm[(16 * lower_m + 4 * g + i) * GD_SMALL + 16 * lower_n + lr] = acc[i];
+  }
+  if (wave == 3) {                                                      // above the diagonal: nothing
+#pragma unroll
+    for (int i = 0; i < 4; i++) Pm[(4 * g + i) * GD_SMALL + 16 + lr] = 0.f;
+  }
+  // T B, 16 channels at a time
+  constexpr int MINE = (NT + 7) / 8;
+  gd_f4 tb[MINE][2];
+#pragma unroll
+  for (int q = 0; q < MINE; q++) {
+    const int nt = wave + 8 * q;
+    tb[q][0] = tb[q][1] = gd_f4{0.f, 0.f, 0.f, 0.f};
+    if (nt < NT) {
+      const gd_f4 t00 = *(const gd_f4*)(Lm + lr * GD_SMALL + 4 * g), t10 = *(const gd_f4*)(Lm + (16 + lr) * GD_SMALL + 4 * g),
+                  t11 = *(const gd_f4*)(Lm + (16 + lr) * GD_SMALL + 16 + 4 * g);
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const float b0 = Bm[(4 * g + i) * LD + 16 * nt + lr], b1 = Bm[(16 + 4 * g + i) * LD + 16 * nt + lr];
+        tb[q][0] = gd_mfma(t00[i], b0, tb[q][0]);
+        tb[q][1] = gd_mfma(t10[i], b0, tb[q][1]);
+        tb[q][1] = gd_mfma(t11[i], b1, tb[q][1]);
+      }
+    }
+  }
+  __syncthreads();
+  if (wave >= 3 && wave < 6) {                                          // N + Q P
+    gd_f4 acc;
+#pragma unroll
+    for (int i = 0; i < 4; i++) acc[i] = Nm[(16 * lower_m + 4 * g + i) * GD_SMALL + 16 * lower_n + lr];
+    acc = lower(Qm, Pm, lower_m, lower_n, acc);
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int i = 0; i < 4; i++) Nm[(16 * lower_m + 4 * g + i) * GD_SMALL + 16 * lower_n + lr] = acc[i];
+    __threadfence_block();
+    __builtin_amdgcn_wave_barrier();
+    *(gd_f4*)(out + Wk::N_AT + ((wave - 3) * 64 + lane) * 4) =
+        *(const gd_f4*)(Nm + (16 * lower_m + lr) * GD_SMALL + 16 * lower_n + 4 * g);
+  }
+#pragma unroll
+  for (int q = 0; q < MINE; q++) {
+    const int nt = wave + 8 * q;
+    if (nt >= NT) continue;
+    const int col = 16 * nt + lr;
+    gd_f4 rq[2], kp[2], at[2];
+#pragma unroll
+    for (int tt = 0; tt < 2; tt++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const int row = (16 * tt + 4 * g + i) * LD + col;
+        rq[tt][i] = Rm[row];
+        kp[tt][i] = Km[row];
+        at[tt][i] = Am[row];
+      }
+    const gd_f4 q00 = *(const gd_f4*)(Qm + lr * GD_SMALL + 4 * g), q10 = *(const gd_f4*)(Qm + (16 + lr) * GD_SMALL + 4 * g),
+                q11 = *(const gd_f4*)(Qm + (16 + lr) * GD_SMALL + 16 + 4 * g);
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+      rq[0] = gd_mfma(q00[i], tb[q][0][i], rq[0]);
+      rq[1] = gd_mfma(q10[i], tb[q][0][i], rq[1]);
+      rq[1] = gd_mfma(q11[i], tb[q][1][i], rq[1]);
+      const float* p0 = Pm + (4 * g + i) * GD_SMALL;                    // row 4 g + i of P, as a column of P^T
+      const float* p1 = p0 + 16 * GD_SMALL;
+      kp[0] = gd_mfma(p0[lr], at[0][i], kp[0]);
+      kp[0] = gd_mfma(p1[lr], at[1][i], kp[0]);
+      kp[1] = gd_mfma(p1[16 + lr], at[1][i], kp[1]);
+    }
+    // back into local memory (these columns are this wave's own), to be read along the rows
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int tt = 0; tt < 2; tt++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const int row = (16 * tt + 4 * g + i) * LD + col;
+        Bm[row] = tb[q][tt][i];
+        Rm[row] = rq[tt][i];
+      }
+    __threadfence_block();
+    __builtin_amdgcn_wave_barrier();
+    gd_f4* o4 = (gd_f4*)(out + nt * Wk::PER_TILE) + lane;
+#pragma unroll
+    for (int tt = 0; tt < 2; tt++) {
+      o4[(0 + tt) * 64] = *(const gd_f4*)(Bm + (16 * tt + lr) * LD + 16 * nt + 4 * g);
+      o4[(2 + tt) * 64] = *(const gd_f4*)(Rm + (16 * tt + lr) * LD + 16 * nt + 4 * g);
+      o4[(4 + tt) * 64] = at[tt];
+      o4[(6 + tt) * 64] = kp[tt];
+    }
+  }
+}
+
+// A block per (head, 16 value channels, request): through the chunks [first_chunk, first_chunk + per_pass) in
+// order.  NW waves, each ST tiles of 16 rows of S in its accumulators.
+template <int D, int NW>
+__global__ __launch_bounds__(NW * 64) void gdelta_scan_kernel(const act_t* __restrict__ rkv, int ld, int v_off,
+                                                              const float* __restrict__ work, float* __restrict__ state,
+                                                              int slot_words, int offset_words,
+                                                              const int* __restrict__ q_start,
+                                                              const int* __restrict__ slot_of_req, float* __restrict__ raw,
+                                                              int H, int first_chunk, int per_pass) {
+  constexpr int ST = D / 16 / NW, NN = (3 + NW - 1) / NW;
+  using Wk = GdWork<D>;
+  __shared__ gd_f4 part[2][NW][4][64];               // partial Y (two tiles), partial O (two tiles)
+  // the value channels of one head read the same operands: neighbours in the launch differ by the head, so
+  // that (with heads in whole eights) a head's blocks meet in one L2
+  const int h = blockIdx.x % H, e0 = blockIdx.x / H * 16, r = blockIdx.y;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lr = lane & 15, g = lane >> 4;
+  const int q0 = q_start[r], n = q_start[r + 1] - q0;
+  if (first_chunk * GD_CHUNK >= n) return;
+  const int chunks = min(per_pass, (n - first_chunk * GD_CHUNK + GD_CHUNK - 1) / GD_CHUNK);
+  float* S0 = state + (size_t)slot_of_req[r] * slot_words + offset_words + (size_t)h * D * D + e0 + lr;
+  gd_f4 S[ST];
+#pragma unroll
+  for (int j = 0; j < ST; j++)
+#pragma unroll
+    for (int i = 0; i < 4; i++) S[j][i] = S0[(size_t)(16 * (wave * ST + j) + 4 * g + i) * D];
+  struct Operands {
+    gd_f4 tb[ST][2], rq[ST][2], at[ST][2], kp[ST][2], bc[ST], nq[NN];
+    float v[2][4];
+  };
+  auto fetch = [&](int c, Operands& x) {
+    const float* w = work + (((size_t)r * per_pass + c) * H + h) * Wk::FLOATS;
+#pragma unroll
+    for (int j = 0; j < ST; j++) {
+      const gd_f4* f = (const gd_f4*)(w + (wave * ST + j) * Wk::PER_TILE) + lane;
+#pragma unroll
+      for (int tt = 0; tt < 2; tt++) {
+        x.tb[j][tt] = f[tt * 64];
+        x.rq[j][tt] = f[(2 + tt) * 64];
+        x.at[j][tt] = f[(4 + tt) * 64];
+        x.kp[j][tt] = f[(6 + tt) * 64];
+      }
+      x.bc[j] = *(const gd_f4*)(w + Wk::B_AT + 16 * (wave * ST + j) + 4 * g);
+    }
+#pragma unroll
+    for (int q = 0; q < NN; q++)
+      if (wave + q * NW < 3) x.nq[q] = *((const gd_f4*)(w + Wk::N_AT) + (wave + q * NW) * 64 + lane);
+    const int t = (first_chunk + c) * GD_CHUNK;
+#pragma unroll
+    for (int tt = 0; tt < 2; tt++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const int at = t + 16 * tt + 4 * g + i;
+        x.v[tt][i] = at < n ? to_f32(rkv[(size_t)(q0 + at) * ld + v_off + (size_t)h * D + e0 + lr]) : 0.f;
+      }
+  };
+  auto chunk = [&](int c, const Operands& x, Operands& next) {
+    if (c + 1 < chunks) fetch(c + 1, next);
+    const int buf = c & 1;
+    gd_f4 y[2], o[2];
+#pragma unroll
+    for (int tt = 0; tt < 2; tt++) y[tt] = o[tt] = gd_f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < ST; j++)
+#pragma unroll
+      for (int i = 0; i < 4; i++)
+#pragma unroll
+        for (int tt = 0; tt < 2; tt++) y[tt] = gd_mfma(x.tb[j][tt][i], S[j][i], y[tt]);
+    part[buf][wave][0][lane] = y[0];
+    part[buf][wave][1][lane] = y[1];
+#pragma unroll
+    for (int j = 0; j < ST; j++)
+#pragma unroll
+      for (int i = 0; i < 4; i++)
+#pragma unroll
+        for (int tt = 0; tt < 2; tt++) o[tt] = gd_mfma(x.rq[j][tt][i], S[j][i], o[tt]);
+#pragma unroll
+    for (int q = 0; q < NN; q++) {
+      const int idx = wave + q * NW;
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        if (idx == 0) o[0] = gd_mfma(x.nq[q][i], x.v[0][i], o[0]);
+        if (idx == 1) o[1] = gd_mfma(x.nq[q][i], x.v[0][i], o[1]);
+        if (idx == 2) o[1] = gd_mfma(x.nq[q][i], x.v[1][i], o[1]);
+      }
+    }
+    part[buf][wave][2][lane] = o[0];
+    part[buf][wave][3][lane] = o[1];
+#pragma unroll
+    for (int tt = 0; tt < 2; tt++)
+#pragma unroll
+      for (int i = 0; i < 4; i++)
+#pragma unroll
+        for (int j = 0; j < ST; j++) S[j] = gd_mfma(x.kp[j][tt][i], x.v[tt][i], S[j]);
+    __syncthreads();          // two buffers: one barrier a chunk suffices
+#pragma unroll
+    for (int tt = 0; tt < 2; tt++) {
+      gd_f4 sum = part[buf][0][tt][lane];
+#pragma unroll
+      for (int w = 1; w < NW; w++) sum += part[buf][w][tt][lane];
+      y[tt] = sum;
+    }
+#pragma unroll
+    for (int tt = 0; tt < 2; tt++)
+#pragma unroll
+      for (int i = 0; i < 4; i++)
+#pragma unroll
+        for (int j = 0; j < ST; j++) S[j] = gd_mfma(x.at[j][tt][i], y[tt][i], S[j]);
+#pragma unroll
+    for (int j = 0; j < ST; j++) S[j] *= x.bc[j];
+    if (wave < 2) {
+      gd_f4 sum = part[buf][0][2 + wave][lane];
+#pragma unroll
+      for (int w = 1; w < NW; w++) sum += part[buf][w][2 + wave][lane];
+      const int t = (first_chunk + c) * GD_CHUNK + 16 * wave + 4 * g;
+#pragma unroll
+      for (int i = 0; i < 4; i++)
+        if (t + i < n) raw[((size_t)(q0 + t + i) * H + h) * D + e0 + lr] = sum[i];
+    }
+  };
+  Operands x0, x1;
+  fetch(0, x0);
+  for (int c = 0; c < chunks; c += 2) {
+    chunk(c, x0, x1);
+    if (c + 1 < chunks) chunk(c + 1, x1, x0);
+  }
+#pragma unroll
+  for (int j = 0; j < ST; j++)
+#pragma unroll
+    for (int i = 0; i < 4; i++) S0[(size_t)(16 * (wave * ST + j) + 4 * g + i) * D] = S[j][i];
+}
+
+template <int D, int NW>
+static int gdelta_chunked_sizes(const act_t* rkv, int ld, int k_off, int v_off, const float* decay, const float* rate, float* state,
+                                int slot_words, int offset_words, const int* q_start, const int* slot_of_req, float* raw,
+                                float* work, size_t work_floats, int R, int max_q_len, int H, hipStream_t s) {
+  constexpr size_t lds = ((size_t)4 * GD_CHUNK * (D + 4) + 5 * GD_CHUNK * GD_SMALL + GD_CHUNK + 512) * sizeof(float);
+  static bool raised = false;
+  if (!raised) {
+    if (hipFuncSetAttribute((const void*)gdelta_chunk_kernel<D>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
+      return zk_fail("zk_gdelta_chunked: the chunk kernel's local memory was refused");
+    raised = true;
+  }
+  const int total = (max_q_len + GD_CHUNK - 1) / GD_CHUNK;
+  const long long room = (long long)(work_floats / ((size_t)GdWork<D>::FLOATS * H * R));
+  ZK_REQUIRE(room >= 1, "zk_gdelta_chunked: the workspace does not hold a chunk of every request");
+  const int per_pass = (int)(room < total ? room : total);
+  for (int first = 0; first < total; first += per_pass) {
+    gdelta_chunk_kernel<D><<<dim3(per_pass, H, R), 512, lds, s>>>(rkv, ld, k_off, decay, rate, q_start, H, first, work);
+    gdelta_scan_kernel<D, NW><<<dim3(H * (D / 16), R), NW * 64, 0, s>>>(rkv, ld, v_off, work, state, slot_words, offset_words, q_start,
+                                                                      slot_of_req, raw, H, first, per_pass);
+  }
+  return 0;
+}
+#endif
+
 extern "C" {
 
 // rows: float [T, ld]: n removal-rate numbers (before bias and sigmoid), and at column low_off ``rank`` numbers
@@ -428,6 +847,49 @@ int zk_gdelta_token(const void* rkv, int ld, int k_off, int v_off, const void* g
 #undef LAUNCH
   return zk_launch_status("zk_gdelta_token");
 }
+// Floats that zk_gdelta_chunked's workspace takes for one chunk of 32 tokens of one head (0: heads of this size
+// are not taken).
+int zk_gdelta_chunk_floats(int D) {
+  switch (D) {
+    case 32: return GdWork<32>::FLOATS;
+    case 64: return GdWork<64>::FLOATS;
+    case 128: return GdWork<128>::FLOATS;
+    case 256: return GdWork<256>::FLOATS;
+    default: return 0;
+  }
+}
+
+// As zk_gdelta (raw is always used), in chunks of 32 tokens.  work: scratch of work_floats floats, at least
+// R * H * zk_gdelta_chunk_floats(D); with room for fewer chunks than the longest portion has, the portions
+// are taken in several passes.
+int zk_gdelta_chunked(const void* rkv, int ld, int k_off, int v_off, const void* g, int ldg, const float* decay,
+                      const float* rate, const float* gain, float* state, int slot_words, int offset_words,
+                      const int* q_start, const int* slot_of_req, const int* positions, void* out, float* raw, float* work,
+                      size_t work_floats, int T, int R, int max_q_len, int H, int D, float eps, void* stream) {
+  ZK_REQUIRE(T >= 0 && R >= 0 && H > 0 && zk_gdelta_chunk_floats(D) > 0, "zk_gdelta_chunked: bad sizes");
+  ZK_REQUIRE(H <= 65535 && R <= 65535 && max_q_len > 0, "zk_gdelta_chunked: too many heads or requests, or no tokens");
+  ZK_REQUIRE(state != nullptr && (long long)slot_words >= (long long)offset_words + (long long)H * D * D,
+             "zk_gdelta_chunked: the state does not fit its slot");
+  ZK_REQUIRE(ld >= k_off + H * D && ld >= v_off + H * D && ldg >= H * D && k_off >= 0 && v_off >= 0,
+             "zk_gdelta_chunked: rows too short");
+  ZK_REQUIRE(raw != nullptr && positions != nullptr && work != nullptr && (uintptr_t)work % 16 == 0,
+             "zk_gdelta_chunked: needs scratch");
+  if (R == 0 || T == 0) return 0;
+  hipStream_t s = (hipStream_t)stream;
+  const act_t* x = (const act_t*)rkv;
+  int rc;
+#define RUN(N, NW)                                                                                                            \
+  rc = gdelta_chunked_sizes<N, NW>(x, ld, k_off, v_off, decay, rate, state, slot_words, offset_words, q_start, slot_of_req, raw, \
+                                   work, work_floats, R, max_q_len, H, s)
+  if (D == 32) RUN(32, 2);
+  else if (D == 64) RUN(64, 4);
+  else if (D == 128) RUN(128, 4);
+  else RUN(256, 8);
+#undef RUN
+  if (rc) return rc;
+  gdelta_finish_kernel<<<dim3(T, H), 64, 0, s>>>(raw, (const act_t*)g, ldg, gain, positions, (act_t*)out, H, D, eps);
+  return zk_launch_status("zk_gdelta_chunked");
+}
 #endif
 
 }  // extern "C"
@@ -436,4 +898,5 @@ ZK_ENTER(zk_gdelta_gates)
 ZK_ENTER(zk_gdelta)
 #if ZSE_ACT_BF16
 ZK_ENTER(zk_gdelta_token)
+ZK_ENTER(zk_gdelta_chunked)
 #endif

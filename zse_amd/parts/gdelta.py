@@ -10,8 +10,9 @@ floats in the request's state slot:
 
 r, k, v and the gate are one product; a and the narrow W_w1 a second one whose results stay floats.
 One small kernel makes w and a of the step's tokens (tanh, W_w2, sigmoids and the exponential in
-floats).  Portions of prompts are walked token by token, single tokens have a kernel of their own
-(one arithmetic; the 32-bit library has the walk alone).
+floats).  Portions of prompts run in chunks of 32 tokens on the 32-bit matrix cores, short ones token by
+token, single tokens in a kernel of their own; the 32-bit library has the walk token by token alone,
+so a request's values there are the same bits however its tokens are cut.
 """
 from __future__ import annotations
 
@@ -24,6 +25,8 @@ from .ops import linear
 
 class GeneralDelta(Part):
     graph_safe = True      # rows, requests and slots are read by the kernels from device memory
+    CHUNKED_FROM = 16      # tokens of a step's longest portion from which the chunks are used (bfloat16)
+    WORK_BYTES = 96 << 20  # of operands at a time: what the last-level cache keeps until they are read
 
     def __init__(self, spec):
         s = self.spec = spec
@@ -83,6 +86,15 @@ class GeneralDelta(Part):
         if ctx.dtype == BF16 and ctx.tuned and ctx.max_q_len == 1 and T == ctx.R and k.zk_gdelta_token_supports(D):
             k.zk_gdelta_token(rows.ptr, ld, C, 2 * C, gate, ld, decay.ptr, rate.ptr, self.gain.ptr, *place, ctx.positions,
                               ctx.req_of_token, ctx.slot_of_req, out.ptr, T, H, D, float(s.eps), ctx.stream)
+        elif ctx.dtype == BF16 and ctx.tuned and ctx.max_q_len >= self.CHUNKED_FROM and k.zk_gdelta_chunk_floats(D):
+            raw = ctx.alloc((T, C), F32)
+            # the operands of as many chunks of every request as WORK_BYTES hold (one at least)
+            chunk = ctx.R * H * k.zk_gdelta_chunk_floats(D)
+            count = max(1, min(-(-int(ctx.max_q_len) // 32), self.WORK_BYTES // (4 * chunk)))
+            work = ctx.alloc((count * chunk,), F32)
+            k.zk_gdelta_chunked(rows.ptr, ld, C, 2 * C, gate, ld, decay.ptr, rate.ptr, self.gain.ptr, *place, ctx.q_start,
+                                ctx.slot_of_req, ctx.positions, out.ptr, raw.ptr, work.ptr, count * chunk, T, ctx.R,
+                                int(ctx.max_q_len), H, D, float(s.eps), ctx.stream)
         else:
             raw = ctx.alloc((T, C), F32)
             k.zk_gdelta(rows.ptr, ld, C, 2 * C, gate, ld, decay.ptr, rate.ptr, self.gain.ptr, *place, ctx.q_start,

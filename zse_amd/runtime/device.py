@@ -255,6 +255,8 @@ BF16_KERNEL_SIGNATURES = {
     "zk_moe_experts_grouped_ext": [_VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _F, _I, _I, _VP],
     "zk_attention_bf16_sized": [_VP, _I, _VP, _VP, _VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I,
                                 _F, _F, _I, _I, _VP, _SZ, _I, _I, _I, _I, _I, _I, _VP],
+    "zk_gdelta_chunked": [_VP, _I, _I, _I, _VP, _I, _VP, _VP, _VP, _VP, _I, _I, _VP, _VP, _VP, _VP, _VP, _VP, _SZ, _I, _I, _I, _I,
+                          _I, _F, _VP],
     "zk_gdelta_token": [_VP, _I, _I, _I, _VP, _I, _VP, _VP, _VP, _VP, _I, _I, _VP, _VP, _VP, _VP, _I, _I, _I, _F, _VP],
 }
 
@@ -341,6 +343,8 @@ class KernelLibrary:
         if dtype == BF16:
             self._dll.zk_gdelta_token_supports.restype, self._dll.zk_gdelta_token_supports.argtypes = C.c_int, [_I]
             self.zk_gdelta_token_supports = self._dll.zk_gdelta_token_supports
+            self._dll.zk_gdelta_chunk_floats.restype, self._dll.zk_gdelta_chunk_floats.argtypes = C.c_int, [_I]
+            self.zk_gdelta_chunk_floats = self._dll.zk_gdelta_chunk_floats
             self._dll.zk_attention_bf16_supports.restype = C.c_int
             self._dll.zk_attention_bf16_supports.argtypes = [_I, _I, _I, _I]
             self.zk_attention_bf16_supports = self._dll.zk_attention_bf16_supports
