@@ -95,7 +95,8 @@ def test_short_convolution_over_steps(C, taps, pad, kind, dtype):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("W,parts,unit,taps", [(64, 0, 0, 0), (64, 3, 0, 4), (50, 1, 1, 3), (2048, 2, 1, 4), (36, 0, 1, 1), (4100, 0, 0, 2)])
+@pytest.mark.parametrize("W,parts,unit,taps", [(64, 0, 0, 0), (64, 3, 0, 4), (50, 1, 1, 3), (2048, 2, 1, 4), (36, 0, 1, 1), (4100, 0, 0, 2), (4100, 2, 1, 4), (300, 0, 1, 2),
+                                                (300, 2, 0, 6), (4096, 4, 1, 3)])
 def test_the_kernel_between_two_sublayers(W, parts, unit, taps, dtype):
     """h += g y (or g times the unit root mean square of y), the stream as activations, the next layer norm, and in
     a step of single tokens the convolution over the rows that the state holds."""

@@ -606,7 +606,8 @@ __global__ __launch_bounds__(NW * 64) void gdelta_scan_kernel(const act_t* __res
   // the value channels of one head read the same operands: neighbours in the launch differ by the head, so
   // that (with heads in whole eights) a head's blocks meet in one L2
   const int h = blockIdx.x % H, e0 = blockIdx.x / H * 16, r = blockIdx.y;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lr = lane & 15, g = lane >> 4;
+  const int tid = threadIdx.x, lane = tid & 63, lr = lane & 15, g = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int q0 = q_start[r], n = q_start[r + 1] - q0;
   if (first_chunk * GD_CHUNK >= n) return;
   const int chunks = min(per_pass, (n - first_chunk * GD_CHUNK + GD_CHUNK - 1) / GD_CHUNK);
@@ -618,7 +619,7 @@ __global__ __launch_bounds__(NW * 64) void gdelta_scan_kernel(const act_t* __res
     for (int i = 0; i < 4; i++) S[j][i] = S0[(size_t)(16 * (wave * ST + j) + 4 * g + i) * D];
   struct Operands {
     gd_f4 tb[ST][2], rq[ST][2], at[ST][2], kp[ST][2], bc[ST], nq[NN];
-    float v[2][4];
+    act_t v[2][4];          // as they lie in memory: turned into floats where they are used, so that nothing waits for them here
   };
   auto fetch = [&](int c, Operands& x) {
     const float* w = work + (((size_t)r * per_pass + c) * H + h) * Wk::FLOATS;
@@ -636,22 +637,44 @@ __global__ __launch_bounds__(NW * 64) void gdelta_scan_kernel(const act_t* __res
     }
 #pragma unroll
     for (int q = 0; q < NN; q++)
-      if (wave + q * NW < 3) x.nq[q] = *((const gd_f4*)(w + Wk::N_AT) + (wave + q * NW) * 64 + lane);
+      x.nq[q] = *((const gd_f4*)(w + Wk::N_AT) + min(wave + q * NW, 2) * 64 + lane);
     const int t = (first_chunk + c) * GD_CHUNK;
 #pragma unroll
     for (int tt = 0; tt < 2; tt++)
 #pragma unroll
       for (int i = 0; i < 4; i++) {
-        const int at = t + 16 * tt + 4 * g + i;
-        x.v[tt][i] = at < n ? to_f32(rkv[(size_t)(q0 + at) * ld + v_off + (size_t)h * D + e0 + lr]) : 0.f;
+        const int at = min(t + 16 * tt + 4 * g + i, n - 1);      // (rows past the portion's end meet zeros in K, A and N)
+        x.v[tt][i] = rkv[(size_t)(q0 + at) * ld + v_off + (size_t)h * D + e0 + lr];
       }
   };
-  auto chunk = [&](int c, const Operands& x, Operands& next) {
-    if (c + 1 < chunks) fetch(c + 1, next);
+  // the read-outs of a chunk: two waves add up the partial sums of 16 tokens each
+  auto read_out = [&](int c) {
+    if (wave >= 2) return;
+    gd_f4 sum = part[c & 1][0][2 + wave][lane];
+#pragma unroll
+    for (int w = 1; w < NW; w++) sum += part[c & 1][w][2 + wave][lane];
+    const int t = (first_chunk + c) * GD_CHUNK + 16 * wave + 4 * g;
+#pragma unroll
+    for (int i = 0; i < 4; i++)
+      if (t + i < n) raw[((size_t)(q0 + t + i) * H + h) * D + e0 + lr] = sum[i];
+  };
+  Operands x, next;
+  fetch(0, x);
+  for (int c = 0; c < chunks; c++) {
+    // The stores of the chunk before, then the next chunk's loads, then this one's arithmetic: whoever waits for
+    // the loads at the end of the turn waits for nothing younger.  (Always a fetch, the last chunk's twice: a
+    // branch around it would make the waits behind it wait for everything.)
+    if (c > 0) read_out(c - 1);
+    fetch(min(c + 1, chunks - 1), next);
     const int buf = c & 1;
+    float v[2][4];
     gd_f4 y[2], o[2];
 #pragma unroll
-    for (int tt = 0; tt < 2; tt++) y[tt] = o[tt] = gd_f4{0.f, 0.f, 0.f, 0.f};
+    for (int tt = 0; tt < 2; tt++) {
+      y[tt] = o[tt] = gd_f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int i = 0; i < 4; i++) v[tt][i] = to_f32(x.v[tt][i]);
+    }
 #pragma unroll
     for (int j = 0; j < ST; j++)
 #pragma unroll
@@ -668,12 +691,14 @@ __global__ __launch_bounds__(NW * 64) void gdelta_scan_kernel(const act_t* __res
         for (int tt = 0; tt < 2; tt++) o[tt] = gd_mfma(x.rq[j][tt][i], S[j][i], o[tt]);
 #pragma unroll
     for (int q = 0; q < NN; q++) {
+      // the three lower tiles of N + Q P, a wave one (or two) of them; a wave without one adds zeros
       const int idx = wave + q * NW;
+      const float on0 = idx == 0 ? 1.f : 0.f, on1 = idx == 1 || idx == 2 ? 1.f : 0.f;
 #pragma unroll
       for (int i = 0; i < 4; i++) {
-        if (idx == 0) o[0] = gd_mfma(x.nq[q][i], x.v[0][i], o[0]);
-        if (idx == 1) o[1] = gd_mfma(x.nq[q][i], x.v[0][i], o[1]);
-        if (idx == 2) o[1] = gd_mfma(x.nq[q][i], x.v[1][i], o[1]);
+        const float nv = x.nq[q][i];
+        o[0] = gd_mfma(nv * on0, v[0][i], o[0]);
+        o[1] = gd_mfma(nv * on1, idx == 2 ? v[1][i] : v[0][i], o[1]);
       }
     }
     part[buf][wave][2][lane] = o[0];
@@ -683,7 +708,7 @@ __global__ __launch_bounds__(NW * 64) void gdelta_scan_kernel(const act_t* __res
 #pragma unroll
       for (int i = 0; i < 4; i++)
 #pragma unroll
-        for (int j = 0; j < ST; j++) S[j] = gd_mfma(x.kp[j][tt][i], x.v[tt][i], S[j]);
+        for (int j = 0; j < ST; j++) S[j] = gd_mfma(x.kp[j][tt][i], v[tt][i], S[j]);
     __syncthreads();          // two buffers: one barrier a chunk suffices
 #pragma unroll
     for (int tt = 0; tt < 2; tt++) {
@@ -700,22 +725,9 @@ __global__ __launch_bounds__(NW * 64) void gdelta_scan_kernel(const act_t* __res
         for (int j = 0; j < ST; j++) S[j] = gd_mfma(x.at[j][tt][i], y[tt][i], S[j]);
 #pragma unroll
     for (int j = 0; j < ST; j++) S[j] *= x.bc[j];
-    if (wave < 2) {
-      gd_f4 sum = part[buf][0][2 + wave][lane];
-#pragma unroll
-      for (int w = 1; w < NW; w++) sum += part[buf][w][2 + wave][lane];
-      const int t = (first_chunk + c) * GD_CHUNK + 16 * wave + 4 * g;
-#pragma unroll
-      for (int i = 0; i < 4; i++)
-        if (t + i < n) raw[((size_t)(q0 + t + i) * H + h) * D + e0 + lr] = sum[i];
-    }
-  };
-  Operands x0, x1;
-  fetch(0, x0);
-  for (int c = 0; c < chunks; c += 2) {
-    chunk(c, x0, x1);
-    if (c + 1 < chunks) chunk(c + 1, x1, x0);
+    x = next;
   }
+  read_out(chunks - 1);
 #pragma unroll
   for (int j = 0; j < ST; j++)
 #pragma unroll

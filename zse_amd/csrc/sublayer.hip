@@ -199,6 +199,137 @@ __global__ __launch_bounds__(1024) void sublayer_step_kernel(float* __restrict__
   }
 }
 
+// A sum over the block with one barrier: every wave leaves its own, every thread adds them up in order.  Each
+// use in a kernel has its own ``red`` (16 floats), so nothing is read after it was overwritten.
+__device__ __forceinline__ float rows_sum(float x, float* red) {
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x140, 0xf, 0xf, false));   // row_mirror
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x141, 0xf, 0xf, false));   // row_half_mirror
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0xB1, 0xf, 0xf, false));    // quad_perm [1,0,3,2]
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x4E, 0xf, 0xf, false));    // quad_perm [2,3,0,1]
+  x += __shfl_xor(x, 16, 64);
+  x += __shfl_xor(x, 32, 64);
+  const int nw = blockDim.x >> 6;
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = x;
+  __syncthreads();
+  float t = red[0];
+  for (int w = 1; w < nw; w++) t += red[w];
+  return t;
+}
+
+// The same for rows of whole groups of four channels, a thread a group: everything the row needs is asked for
+// at once, before the first sum.  TAPS: 0 without the convolution, 2 to 4 taps known to the
+// compiler (their weights and state rows are asked for at once too), -1 any other number.
+template <int TAPS>
+__global__ __launch_bounds__(1024) void sublayer_row_kernel(float* __restrict__ h, const void* __restrict__ y, int y_parts,
+                                                            size_t y_plane, const float* __restrict__ y_gain, int y_unit,
+                                                            float y_eps, act_t* __restrict__ raw,
+                                                            const float* __restrict__ norm_w, const float* __restrict__ norm_b,
+                                                            float eps, act_t* __restrict__ out, SublayerConv cv, int W) {
+  __shared__ float red[3][16];
+  constexpr int N = TAPS > 0 ? TAPS : 1;
+  const int t = blockIdx.x, c = threadIdx.x * 4;
+  const bool in = c < W;
+  const size_t at = (size_t)t * W + (in ? c : 0);
+  const int taps = TAPS > 0 ? TAPS : cv.taps;
+  float x[4] = {}, v[4] = {}, g[4] = {1.f, 1.f, 1.f, 1.f}, nw[4], nb[4] = {}, cw[4 * N], older[N][4];
+  const bool padding = TAPS != 0 && cv.positions[t] < 0;          // a padding row of a captured step
+  float* st = (TAPS != 0 && !padding && taps > 1)
+                  ? cv.state + (size_t)cv.slot_of_req[cv.req_of_token[t]] * cv.slot_words + cv.offset_words + c : nullptr;
+  if (in) {
+    get_floats<4>(h + at, x);
+    if (y != nullptr) {
+      if (y_parts > 0) {
+        const float* p = (const float*)y + at;
+        get_floats<4>(p, v);
+        for (int k = 1; k < y_parts; k++) {
+          float u[4];
+          get_floats<4>(p + (size_t)k * y_plane, u);
+#pragma unroll
+          for (int e = 0; e < 4; e++) v[e] += u[e];
+        }
+      } else {
+        get_acts<4>((const act_t*)y + at, v);
+      }
+      if (y_gain) get_floats<4>(y_gain + c, g);
+    }
+    if (out != nullptr) {
+      get_floats<4>(norm_w + c, nw);
+      if (norm_b) get_floats<4>(norm_b + c, nb);
+    }
+    if (TAPS > 0) {
+#pragma unroll
+      for (int q = 0; q < N; q++) {
+        float u[4];
+        get_floats<4>(cv.w + (size_t)c * N + 4 * q, u);
+#pragma unroll
+        for (int e = 0; e < 4; e++) cw[4 * q + e] = u[e];
+      }
+      if (!padding) {
+#pragma unroll
+        for (int a = 0; a < N - 1; a++) get_floats<4>(st + (size_t)a * W, older[a]);
+      }
+    }
+  }
+  if (y != nullptr) {
+    float inv_y = 1.f;
+    if (y_unit) {
+      float ss = 0.f;
+#pragma unroll
+      for (int e = 0; e < 4; e++) ss = fmaf(v[e], v[e], ss);
+      inv_y = 1.0f / sqrtf(rows_sum(ss, red[0]) / (float)W + y_eps);
+    }
+#pragma unroll
+    for (int e = 0; e < 4; e++) x[e] = fmaf(v[e] * inv_y, g[e], x[e]);
+    if (in) put_floats<4>(h + at, x);
+  }
+  if (in && raw != nullptr) put_acts<4>(raw + at, x);
+  if (out == nullptr) return;
+  const float mean = rows_sum(in ? (x[0] + x[1]) + (x[2] + x[3]) : 0.f, red[1]) / (float)W;
+  float dev = 0.f;
+  if (in) {
+#pragma unroll
+    for (int e = 0; e < 4; e++) {
+      const float d = x[e] - mean;
+      dev = fmaf(d, d, dev);
+    }
+  }
+  const float inv = 1.0f / sqrtf(rows_sum(dev, red[2]) / (float)W + eps);
+  if (!in) return;
+#pragma unroll
+  for (int e = 0; e < 4; e++) x[e] = fmaf((x[e] - mean) * inv, nw[e], nb[e]);
+  if (TAPS != 0) {
+    float acc[4] = {};
+#pragma unroll
+    for (int e = 0; e < 4; e++) x[e] = padding ? 0.f : to_f32(from_f32<act_t>(x[e]));
+    if (!padding) {
+      if (TAPS > 0) {
+#pragma unroll
+        for (int a = N - 2; a >= 0; a--)
+#pragma unroll
+          for (int e = 0; e < 4; e++) acc[e] = fmaf(cw[e * N + N - 2 - a], older[a][e], acc[e]);
+#pragma unroll
+        for (int a = 1; a < N - 1; a++) put_floats<4>(st + (size_t)a * W, older[a - 1]);
+#pragma unroll
+        for (int e = 0; e < 4; e++) acc[e] = fmaf(cw[e * N + N - 1], x[e], acc[e]);
+      } else {
+        for (int a = taps - 2; a >= 0; a--) {
+          float u[4];
+          get_floats<4>(st + (size_t)a * W, u);
+          if (a < taps - 2) put_floats<4>(st + (size_t)(a + 1) * W, u);
+#pragma unroll
+          for (int e = 0; e < 4; e++) acc[e] = fmaf(cv.w[(size_t)(c + e) * taps + taps - 2 - a], u[e], acc[e]);
+        }
+#pragma unroll
+        for (int e = 0; e < 4; e++) acc[e] = fmaf(cv.w[(size_t)(c + e) * taps + taps - 1], x[e], acc[e]);
+      }
+      if (taps > 1) put_floats<4>(st, x);
+    }
+#pragma unroll
+    for (int e = 0; e < 4; e++) x[e] += acc[e];
+  }
+  put_acts<4>(out + at, x);
+}
+
 // h <- (h - mean) / sqrt(var + eps) * w + b, in place and in float
 __global__ __launch_bounds__(1024) void norm_stream_kernel(float* __restrict__ h, const float* __restrict__ w,
                                                            const float* __restrict__ b, float eps, int W) {
@@ -254,8 +385,23 @@ int zk_sublayer_step(float* h, const void* y, int y_parts, const float* y_gain, 
   auto aligned = [](const void* p, size_t n) { return (uintptr_t)p % n == 0; };
   const size_t act4 = 4 * sizeof(act_t);
   const bool vec = W % 4 == 0 && aligned(h, 16) && aligned(y_gain, 16) && aligned(norm_w, 16) && aligned(norm_b, 16) &&
-                   aligned(raw, act4) && aligned(out, act4) && aligned(y, y_parts > 0 ? 16 : act4) &&
+                   aligned(conv_w, 16) && aligned(raw, act4) && aligned(out, act4) && aligned(y, y_parts > 0 ? 16 : act4) &&
                    (conv_w == nullptr || (aligned(state, 16) && slot_words % 4 == 0 && offset_words % 4 == 0));
+  if (vec && W <= 4096) {
+    // (which kernel follows from the width and the operands' places alone, and the block from the width: the order
+    // of a row's sums does not follow from how many rows a step brings)
+    const int width = (W / 4 + 63) / 64 * 64;
+#define ROW(N)                                                                                                            \
+  sublayer_row_kernel<N><<<T, width, 0, (hipStream_t)stream>>>(h, y, y_parts, (size_t)T * W, y_gain, y_unit, y_eps, (act_t*)raw, \
+                                                               norm_w, norm_b, eps, (act_t*)out, cv, W)
+    if (conv_w == nullptr) ROW(0);
+    else if (taps == 2) ROW(2);
+    else if (taps == 3) ROW(3);
+    else if (taps == 4) ROW(4);
+    else ROW(-1);
+#undef ROW
+    return zk_launch_status("zk_sublayer_step");
+  }
   const size_t lds = (size_t)W * 4;
   if (lds > 48 * 1024) {
     static bool raised = false;
