@@ -164,9 +164,11 @@ def scan_mixer(x, w, m, mx, dt):
 
 
 # ---------------------------------------------------------------- generalized delta rule
-def general_delta_rule(r, k, v, w, a, dt):
+def general_delta_rule(r, k, v, w, a, dt, cancel=None):
     """One head: r, k, w, a [T, D], v [T, D] -> o [T, D].  S <- diag(w) S - (a u)(u^T S) + k v^T with
-    the unit key u, both terms from the old S; o = S^T r."""
+    the unit key u, both terms from the old S; o = S^T r.
+    ``cancel``: an array [T] that receives the least size of o beside that of an o whose terms do not
+    cancel: what is normalised next carries the rounding of r and S over this number."""
     D = r.shape[1]
     S = np.zeros((D, v.shape[1]), dt)
     o = np.zeros(v.shape, dt)
@@ -174,17 +176,20 @@ def general_delta_rule(r, k, v, w, a, dt):
         u = k[t] / np.sqrt((k[t] * k[t]).sum() + dt(1e-6))
         S = w[t][:, None] * S - np.outer(a[t] * u, u @ S) + np.outer(k[t], v[t])
         o[t] = S.T @ r[t]
+        if cancel is not None:
+            whole = np.linalg.norm(r[t]) * np.linalg.norm(S) / math.sqrt(D)
+            cancel[t] = min(cancel[t], np.linalg.norm(o[t]) / max(whole, 1e-30))
     return o
 
 
-def general_delta_mixer(x, w, m, mx, eps, dt):
+def general_delta_mixer(x, w, m, mx, eps, dt, cancel=None):
     T, H, D = len(x), mx["heads"], mx["dim"]
     f = lambda name: w[m + name].astype(dt)
     heads = lambda y: y.reshape(T, H, D)
     r, k, v = (heads(x @ f(n).T) for n in ("r", "k", "v"))
     decay = heads(np.exp(-math.exp(-0.5) * sigmoid(np.tanh(x @ f("w1").T) @ f("w2").T + f("w0"))))
     rate = heads(sigmoid(x @ f("a").T + f("a.b")))
-    o = np.stack([general_delta_rule(r[:, h], k[:, h], v[:, h], decay[:, h], rate[:, h], dt) for h in range(H)], axis=1)
+    o = np.stack([general_delta_rule(r[:, h], k[:, h], v[:, h], decay[:, h], rate[:, h], dt, cancel) for h in range(H)], axis=1)
     o = unit_rms(o, eps, dt).reshape(T, H * D) * f("norm")
     return (o * sigmoid(x @ f("g").T)) @ f("o").T
 
@@ -257,9 +262,10 @@ def side_input(h, tokens, i, w, cfg, dt):
     return unit_rms(g @ w[p + "proj"].T.astype(dt), cfg["norm"]["eps"], dt) * w[p + "norm"].astype(dt)
 
 
-def forward(cfg, w, tokens, dt=np.float64, layers_out=None, close=None):
+def forward(cfg, w, tokens, dt=np.float64, layers_out=None, close=None, cancel=None):
     """Logits [T, vocab].  ``layers_out``: a list that receives the stream after every layer.
-    ``close``: an array [T] that receives how close each token's nearest choice of experts was."""
+    ``close``: an array [T] that receives how close each token's nearest choice of experts was.
+    ``cancel``: an array [T] that receives how far the worst read of a recurrence cancels."""
     eps = cfg["norm"]["eps"]
     tokens = np.asarray(tokens)
     pos = np.arange(len(tokens))
@@ -267,6 +273,8 @@ def forward(cfg, w, tokens, dt=np.float64, layers_out=None, close=None):
     v_first = None
     if close is not None:
         close[:] = np.inf
+    if cancel is not None:
+        cancel[:] = np.inf
 
     def read(p, q):
         x = layer_norm(h, w[f"{p}norm{q}"], eps, dt)
@@ -278,7 +286,7 @@ def forward(cfg, w, tokens, dt=np.float64, layers_out=None, close=None):
         if l["type"] == "mamba1":
             y = scan_mixer(x, w, p + "mix.", mx, dt)
         elif l["type"] == "general_delta":
-            y = general_delta_mixer(x, w, p + "mix.", mx, eps, dt)
+            y = general_delta_mixer(x, w, p + "mix.", mx, eps, dt, cancel)
         else:
             mixes = bool(mx.get("v_mix"))
             y, own = attention_mixer(x, pos, w, p + "mix.", mx, eps, v_first if mixes else None, dt)
