@@ -25,6 +25,14 @@ class NormSpec:
     unit_offset: bool
     weight: str                      # checkpoint tensor name
     kind: str = "rmsnorm"
+    gain_scale: float = 1.0          # multiplies the gain: a factor of whatever reads the norm linearly
+
+
+@dataclass(frozen=True)
+class NoNormSpec:
+    """Where a norm could stand and none does: the rows themselves, in the activation type."""
+    size: int
+    kind: str = "none"
 
 
 @dataclass(frozen=True)
@@ -122,6 +130,9 @@ class AttentionSpec:
     lend_values: bool = False                # the step's values (before any mixing) are lent to later layers
     value_share: Optional[str] = None        # a number l: values are (1 - l) v + l v_lent, with the values that the
     #                                          last lending layer lent for the same token; what is cached is the mix
+    sinks: Optional[str] = None              # [num_heads]: exp(sink) joins a head's denominator, with no key and no value
+    head_gate: Optional[str] = None          # [num_heads, hidden]: a head's output times sigmoid(W x)_h before W_o, one
+    #                                          number a head
     values_are_keys: bool = False            # no value projection: a value is its key as projected (with its bias,
     #                                          before norm and rotation); ``names`` and ``biases`` hold no role v
 
@@ -314,7 +325,10 @@ class RoutedMLPSpec:
     gated: bool = True               # False: an expert is act(x Wu^T) Wd^T with "relu2", and ``shared`` an MLPSpec
     correction: Optional[str] = None    # [num_experts]: added to the scores for the choice, not for the weights
     groups: Optional[Tuple[int, int]] = None    # (count, keep): equal runs of neighbouring experts, of which the ``keep``
-    #                                  with the largest sums of their two largest choice scores can be chosen from
+    #                                  with the largest sums of their ``group_best`` largest choice scores can be chosen from
+    group_best: int = 2              # 1: a group is judged by its largest choice score alone
+    identity: int = 0                # so many more router outputs behind the experts': experts without weights that give
+    #                                  their input back (they count in the softmax, the choice and the groups)
     normalise: bool = False          # the chosen scores are divided by their sum (+ 1e-20)
     weight_scale: float = 1.0        # multiplies the weights
     shared_gate: Optional[str] = None   # [1, hidden]: the shared layer's result times sigmoid(W x), a number a token
@@ -327,10 +341,11 @@ class BlockSpec:
     ``arrangement``:
       "sandwich": h += post_m(mixer(pre_m(h))); h += post_f(ffn(pre_f(h)))
       "prenorm" : h += mixer(pre_m(h));         h += ffn(pre_f(h))
+      "postnorm": h += post_m(mixer(h));        h += post_f(ffn(h))            (the sublayers read the stream itself)
       "parallel": x = pre_m(h);  h += mixer(x) + ffn(x)      (``ffn`` may be None); with a norm
                   ``pre_ffn`` among the norms the feed-forward reads pre_f(h) of the same h instead
     ``norms`` holds the roles pre_mixer, post_mixer, pre_ffn, post_ffn that the
-    arrangement uses.  ``residual_scale`` (parallel): h += residual_scale * (mixer + ffn).
+    arrangement uses (a layer whose ``ffn`` is None needs none of the feed-forward's).  ``residual_scale`` (parallel): h += residual_scale * (mixer + ffn).
     """
     arrangement: str
     mixer: Any
@@ -402,6 +417,7 @@ class EmbeddingSpec:
     kind: str = "embedding"
     copies: int = 1                  # the row is written this many times (one per residual stream)
     pairs: Optional[PairTableSpec] = None
+    exact_scale: bool = False        # the scale is not rounded to the type the table is stored in
     norm: Any = None                 # a layer norm of the embedded row; the stream begins with its result, in floats
 
 

@@ -84,8 +84,9 @@ __global__ __launch_bounds__(64) void attn_portion_join_kernel(AttnParams p, int
 #pragma unroll
     for (int j = 0; j < 4; j++) acc[j] += w * po[j * 64];
   }
-  const float inv = 1.f / (l + sink_weight(p, m));
-  __bf16* orow = p.out + ((size_t)(qs + t0 + tok) * p.nh + q_head_of(p, kvh, hq)) * p.vd;
+  const int row = qs + t0 + tok, head = q_head_of(p, kvh, hq);
+  const float inv = row_factor(p, row, head, l, m);
+  __bf16* orow = p.out + ((size_t)row * p.nh + head) * p.vd;
 #pragma unroll
   for (int j = 0; j < 4; j++) {
     const int d = dt * 32 + 8 * j + 4 * lk;
@@ -107,7 +108,9 @@ __global__ __launch_bounds__(256) void attn_combine_kernel(const float* __restri
                                                            const int* __restrict__ ctx_len,
                                                            __bf16* __restrict__ out, int nh, int hd,
                                                            int window, int r_begin, int nchunks, int span,
-                                                           int mask_chunk, int sink, int keep) {
+                                                           int mask_chunk, int sink, int keep,
+                                                           const float* __restrict__ sinks,
+                                                           const __bf16* __restrict__ gate, int gate_ld) {
   __shared__ float wgt[ATT_MAX_CHUNKS];
   __shared__ float red[17];
   const int rr = blockIdx.x, head = blockIdx.y;
@@ -146,8 +149,9 @@ __global__ __launch_bounds__(256) void attn_combine_kernel(const float* __restri
     l += part_ml[at + 1] * w;
   }
   l = block_sum(l, red);
-  const float inv = 1.f / (l + (sink ? __builtin_amdgcn_exp2f(-m) : 0.f));
-  __bf16* orow = out + ((size_t)q_start[r] * nh + head) * hd;
+  const int row = q_start[r];
+  const float inv = gate_factor(gate, gate_ld, row, head) / (l + sink_weight(sinks, sink, head, m));
+  __bf16* orow = out + ((size_t)row * nh + head) * hd;
   for (int d = threadIdx.x; d < hd; d += 256) {
     const float* po = part_o + base * hd + d;
     float acc = 0.f;
@@ -292,12 +296,17 @@ long long zk_attention_bf16_max_context(int nh, int nkv, int hd, int decode_chun
 // vd: channels of a value and of the output's heads (hd, hd / 2 or 2 hd); the workspace functions above
 // are asked with vd for their hd.  keep (with a window): a row sees the first ``keep`` keys of its sequence
 // beside its window; the caller keeps their pages.
-int zk_attention_bf16_sized(const void* q, int q_stride, const void* kcache, const void* vcache_t,
+// sinks (may be null; not together with ``sink``): float [nh], exp(sinks[h]) joins head h's denominators.
+// gate (may be null): bf16, row t's nh numbers at gate + t * gate_ld; head h's output times sigmoid of the h-th.
+int zk_attention_bf16_gated(const void* q, int q_stride, const void* kcache, const void* vcache_t,
                            const int* block_table, int max_blocks, const int* q_start, const int* ctx_len,
                            void* out, int R, int r_prefill, int max_q_len, int max_ctx, int nh, int nkv,
                            int hd, int bs, float scale, float softcap, int window, int decode_chunk,
                            void* workspace, size_t workspace_bytes, int mask_chunk, int sink, int wide_weights,
-                           int v_shift, int vd, int keep, void* stream) {
+                           int v_shift, int vd, int keep, const float* sinks, const void* gate, int gate_ld,
+                           void* stream) {
+  ZK_REQUIRE(!sink || sinks == nullptr, "zk_attention_bf16: a unit sink or learned sinks, not both");
+  ZK_REQUIRE(gate == nullptr || gate_ld >= nh, "zk_attention_bf16: gate rows hold a number per head");
   ZK_REQUIRE(keep >= 0 && (keep == 0 || window > 0), "zk_attention_bf16: first keys are kept beside a window");
   ZK_REQUIRE(v_shift >= 0 && v_shift <= 4 && nkv % (1 << v_shift) == 0, "zk_attention_bf16: key heads in whole groups of a value head");
   ZK_REQUIRE(mask_chunk >= 0 && (mask_chunk == 0 || window == 0), "zk_attention_bf16: a window or a chunk, not both");
@@ -330,6 +339,7 @@ int zk_attention_bf16_sized(const void* q, int q_stride, const void* kcache, con
   p.scale = scale; p.softcap = softcap; p.window = window;
   p.from_window = 0;
   p.mask_chunk = mask_chunk; p.sink = sink ? 1 : 0; p.wide_weights = wide_weights ? 1 : 0;
+  p.sinks = sinks; p.gate = (const __bf16*)gate; p.gate_ld = gate_ld;
   p.bs_shift = 0;
   while ((1 << p.bs_shift) < bs) p.bs_shift++;
   const float log2e = 1.4426950408889634f;
@@ -439,10 +449,23 @@ int zk_attention_bf16_sized(const void* q, int q_stride, const void* kcache, con
     if (rc) return rc;
     dim3 cgrid(n_dec, nh);
     attn_combine_kernel<<<cgrid, 256, 0, s>>>(p.part_o, p.part_ml, q_start, ctx_len, (__bf16*)out, nh, vd,
-                                              window, r_prefill, p.nchunks, span, mask_chunk, sink, keep);
+                                              window, r_prefill, p.nchunks, span, mask_chunk, sink, keep, sinks,
+                                              (const __bf16*)gate, gate_ld);
     return zk_launch_status("zk_attention_bf16 (combine)");
   }
   return 0;
+}
+
+int zk_attention_bf16_sized(const void* q, int q_stride, const void* kcache, const void* vcache_t,
+                           const int* block_table, int max_blocks, const int* q_start, const int* ctx_len,
+                           void* out, int R, int r_prefill, int max_q_len, int max_ctx, int nh, int nkv,
+                           int hd, int bs, float scale, float softcap, int window, int decode_chunk,
+                           void* workspace, size_t workspace_bytes, int mask_chunk, int sink, int wide_weights,
+                           int v_shift, int vd, int keep, void* stream) {
+  return zk_attention_bf16_gated(q, q_stride, kcache, vcache_t, block_table, max_blocks, q_start, ctx_len, out, R,
+                                 r_prefill, max_q_len, max_ctx, nh, nkv, hd, bs, scale, softcap, window, decode_chunk,
+                                 workspace, workspace_bytes, mask_chunk, sink, wide_weights, v_shift, vd, keep, nullptr,
+                                 nullptr, 0, stream);
 }
 
 int zk_attention_bf16_maps(const void* q, int q_stride, const void* kcache, const void* vcache_t,
@@ -483,6 +506,10 @@ extern "C" int zk_steplist_register(const char* name, int nargs, void* fn);
 static const int zk_attention_bf16_masked_entered = zk_steplist_register(
     "zk_attention_bf16_masked", zk_packed::Call<zk_attention_bf16_masked>::nargs,
     (void*)zk_packed::Call<zk_attention_bf16_masked>::call);
+
+static const int zk_attention_bf16_gated_entered = zk_steplist_register(
+    "zk_attention_bf16_gated", zk_packed::Call<zk_attention_bf16_gated>::nargs,
+    (void*)zk_packed::Call<zk_attention_bf16_gated>::call);
 
 static const int zk_attention_bf16_sized_entered = zk_steplist_register(
     "zk_attention_bf16_sized", zk_packed::Call<zk_attention_bf16_sized>::nargs,

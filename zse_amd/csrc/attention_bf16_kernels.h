@@ -47,6 +47,9 @@ struct AttnParams {
   int mask_chunk;         // > 0: a row sees the keys of its own chunk of this many positions only (no window then)
   int keep;               // beside its window a row sees the first ``keep`` keys of its sequence
   int sink;               // 1: a key of score 0 without a value joins every row's denominator
+  const float* sinks;     // [nh] (may be null): exp(sinks[h]) joins head h's denominator, with no key and no value
+  const __bf16* gate;     // (may be null) row t's numbers per head at gate + t * gate_ld; head h's output is
+  int gate_ld;            // multiplied by the sigmoid of the h-th
   int wide_weights;       // 1: a weight meets the values as two bf16 numbers, its rounded value and what the
                           // rounding left (16 bits of mantissa instead of 8; one more product a tile)
 };
@@ -78,9 +81,21 @@ struct KeyTiles {
   __device__ __forceinline__ int key_of(int i) const { return 32 * (i < kept ? i : lo + i - kept); }
 };
 
-// What the sink adds to a row's sum of weights: 2^(0 - m), scores and maximum in the log2 domain.
-__device__ __forceinline__ float sink_weight(const AttnParams& p, float m) {
-  return p.sink ? __builtin_amdgcn_exp2f(-m) : 0.f;
+// What a head's sink adds to a row's sum of weights: 2^(sink - m), scores and maximum in the log2 domain.
+__device__ __forceinline__ float sink_weight(const float* sinks, int unit_sink, int head, float m) {
+  if (sinks) return __builtin_amdgcn_exp2f(sinks[head] * 1.4426950408889634f - m);
+  return unit_sink ? __builtin_amdgcn_exp2f(-m) : 0.f;
+}
+
+// The sigmoid of a row's gate for a head.
+__device__ __forceinline__ float gate_factor(const __bf16* gate, int gate_ld, int row, int head) {
+  if (!gate) return 1.f;
+  return 1.f / (1.f + __expf(-(float)gate[(size_t)row * gate_ld + head]));
+}
+
+// What a row's sum of weighted values is multiplied by: 1 over the sum of its weights, and its gate.
+__device__ __forceinline__ float row_factor(const AttnParams& p, int row, int head, float l, float m) {
+  return gate_factor(p.gate, p.gate_ld, row, head) / (l + sink_weight(p.sinks, p.sink, head, m));
 }
 
 __device__ __forceinline__ float score_log2(const AttnParams& p, float dot) {
@@ -402,7 +417,7 @@ __global__ __launch_bounds__(256, (HD16 <= 8 && VD16 <= 8 && !PAIR) ? 2 : 1) voi
       __syncthreads();
     }
     if (phase != 0 || !row_ok) return;
-    const float inv = 1.f / (l_all + sink_weight(p, m_all));
+    const float inv = row_factor(p, trow, head, l_all, m_all);
     __bf16* orow = p.out + ((size_t)trow * p.nh + head) * vd;
 #pragma unroll
     for (int dt = 0; dt < DT; dt++)
@@ -713,7 +728,7 @@ __global__ __launch_bounds__(NW * 64, (HD16 <= 8 && VD16 <= 8 && NW <= 4) ? 2 : 
         po[(dt * 4 + j) * 64] = f32x4{o[dt][4 * j], o[dt][4 * j + 1], o[dt][4 * j + 2], o[dt][4 * j + 3]};
     return;
   }
-  const float inv = 1.f / (l_run + sink_weight(p, m_run));
+  const float inv = row_factor(p, trow, head, l_run, m_run);
   __bf16* orow = p.out + ((size_t)trow * p.nh + head) * VD;
 #pragma unroll
   for (int dt = 0; dt < DT; dt++)

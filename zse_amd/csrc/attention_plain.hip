@@ -8,7 +8,8 @@
 // With ``chunk`` instead of a window, lo = floor(pos / chunk) * chunk: a query sees the keys of
 // its own chunk of positions, counted from position 0.  ``unit_sink``: a sink of score 0 that has
 // no value joins the denominator, exp(s_j) / (1 + sum exp(s)).  ``keep``: beside its window a query
-// sees the sequence's first ``keep`` keys, at their own positions.
+// sees the sequence's first ``keep`` keys, at their own positions.  ``gate``: a number z per token and
+// query head; the head's output is multiplied by sigmoid(z).
 //
 // Keys are visited in tiles of 64 aligned to absolute positions, with a
 // running maximum and sum, so the order of every sum depends on the token's
@@ -31,7 +32,8 @@ __global__ __launch_bounds__(64) void attention_plain_kernel(
     const int* __restrict__ req_of_token, const int* __restrict__ positions,
     act_t* __restrict__ out, int nh, int nkv, int hd, int vd, int bs, float scale, float softcap,
     int window, int v_transposed, const float* __restrict__ v_freq, int v_interleaved,
-    const float* __restrict__ sinks, int v_in_k, int chunk, int unit_sink, int keep) {
+    const float* __restrict__ sinks, int v_in_k, int chunk, int unit_sink, int keep, const act_t* __restrict__ gate,
+    int gate_ld) {
   __shared__ float sq[MAXD];
   __shared__ float sp[64];
   __shared__ int spage[64];
@@ -106,7 +108,8 @@ __global__ __launch_bounds__(64) void attention_plain_kernel(
 #pragma unroll
     for (int c = 0; c < MAXD / 64; c++) acc[c] *= corr;
   }
-  const float inv = 1.f / l;
+  float inv = 1.f / l;
+  if (gate != nullptr) inv *= 1.f / (1.f + expf(-to_f32(gate[(size_t)t * gate_ld + h])));
   if (v_freq == nullptr) {
 #pragma unroll
     for (int c = 0; c < MAXD / 64; c++) {
@@ -143,12 +146,14 @@ __global__ __launch_bounds__(64) void attention_plain_kernel(
 // chunk > 0 (without a window): a query sees the keys of its own chunk of positions only.
 // unit_sink: a sink of score 0 joins every head's denominator (not together with sinks).
 // keep > 0 (with a window): a query sees the sequence's first ``keep`` keys beside its window.
-extern "C" int zk_attention_plain_kept(const void* q, int q_stride, const void* kcache, const void* vcache,
+// gate (may be null): row t's nh numbers lie at gate + t * gate_ld; head h's output times sigmoid of the h-th.
+extern "C" int zk_attention_plain_gated(const void* q, int q_stride, const void* kcache, const void* vcache,
                                          const int* block_table, int max_blocks, const int* req_of_token,
                                          const int* positions, void* out, int T, int nh, int nkv, int hd, int vd,
                                          int bs, float scale, float softcap, int window, int v_transposed,
                                          const float* v_freq, int v_interleaved, const float* sinks, int v_in_k,
-                                         int chunk, int unit_sink, int keep, void* stream) {
+                                         int chunk, int unit_sink, int keep, const void* gate, int gate_ld, void* stream) {
+  ZK_REQUIRE(gate == nullptr || gate_ld >= nh, "zk_attention_plain: gate rows hold a number per head");
   ZK_REQUIRE(keep >= 0 && (keep == 0 || window > 0), "zk_attention_plain: first keys are kept beside a window");
   ZK_REQUIRE(chunk >= 0 && (chunk == 0 || window <= 0), "zk_attention_plain: a chunk or a window, not both");
   ZK_REQUIRE(!unit_sink || sinks == nullptr, "zk_attention_plain: a unit sink or learned sinks, not both");
@@ -166,13 +171,24 @@ extern "C" int zk_attention_plain_kept(const void* q, int q_stride, const void* 
     attention_plain_kernel<AP_MAX_HD><<<grid, 64, 0, (hipStream_t)stream>>>(
         (const act_t*)q, q_stride, (const act_t*)kcache, (const act_t*)vcache, block_table, max_blocks,
         req_of_token, positions, (act_t*)out, nh, nkv, hd, vd, bs, scale, softcap, window, v_transposed, v_freq,
-        v_interleaved, sinks, v_in_k, chunk, unit_sink, keep);
+        v_interleaved, sinks, v_in_k, chunk, unit_sink, keep, (const act_t*)gate, gate_ld);
   else
     attention_plain_kernel<1024><<<grid, 64, 0, (hipStream_t)stream>>>(
         (const act_t*)q, q_stride, (const act_t*)kcache, (const act_t*)vcache, block_table, max_blocks,
         req_of_token, positions, (act_t*)out, nh, nkv, hd, vd, bs, scale, softcap, window, v_transposed, v_freq,
-        v_interleaved, sinks, v_in_k, chunk, unit_sink, keep);
+        v_interleaved, sinks, v_in_k, chunk, unit_sink, keep, (const act_t*)gate, gate_ld);
   return zk_launch_status("zk_attention_plain");
+}
+
+extern "C" int zk_attention_plain_kept(const void* q, int q_stride, const void* kcache, const void* vcache,
+                                         const int* block_table, int max_blocks, const int* req_of_token,
+                                         const int* positions, void* out, int T, int nh, int nkv, int hd, int vd,
+                                         int bs, float scale, float softcap, int window, int v_transposed,
+                                         const float* v_freq, int v_interleaved, const float* sinks, int v_in_k,
+                                         int chunk, int unit_sink, int keep, void* stream) {
+  return zk_attention_plain_gated(q, q_stride, kcache, vcache, block_table, max_blocks, req_of_token, positions, out, T,
+                                  nh, nkv, hd, vd, bs, scale, softcap, window, v_transposed, v_freq, v_interleaved,
+                                  sinks, v_in_k, chunk, unit_sink, keep, nullptr, 0, stream);
 }
 
 extern "C" int zk_attention_plain_masked(const void* q, int q_stride, const void* kcache, const void* vcache,
@@ -228,6 +244,9 @@ static const int attention_plain_masked_entered = zk_steplist_register(
 static const int attention_plain_kept_entered = zk_steplist_register(
     "zk_attention_plain_kept", zk_packed::Call<zk_attention_plain_kept>::nargs,
     (void*)zk_packed::Call<zk_attention_plain_kept>::call);
+static const int attention_plain_gated_entered = zk_steplist_register(
+    "zk_attention_plain_gated", zk_packed::Call<zk_attention_plain_gated>::nargs,
+    (void*)zk_packed::Call<zk_attention_plain_gated>::call);
 static const int attention_plain_ext_entered = zk_steplist_register(
     "zk_attention_plain_ext", zk_packed::Call<zk_attention_plain_ext>::nargs,
     (void*)zk_packed::Call<zk_attention_plain_ext>::call);

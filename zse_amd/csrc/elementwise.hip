@@ -72,7 +72,8 @@ __device__ __forceinline__ float sub_value(const void* __restrict__ sub, int par
   return to_f32(from_f32<act_t>(x));
 }
 
-// h += N_post(sub)  (w_post null: h += sub);  then, if w_next: out = N_next(h)
+// h += N_post(sub)  (w_post null: h += sub);  then, if w_next: out = N_next(h), or with an output and
+// no next norm: out = h in the activation type (a next sublayer that reads the stream itself)
 __global__ void norm_add_norm_kernel(const void* __restrict__ sub, int parts, const float* __restrict__ w_post,
                                      float eps_post, int uo_post, float* __restrict__ h,
                                      const float* __restrict__ w_next, float eps_next, int uo_next,
@@ -97,6 +98,7 @@ __global__ void norm_add_norm_kernel(const void* __restrict__ sub, int parts, co
     if (w_post) v = v * rs * gain(w_post, i, uo_post);
     v = hr[i] + v;
     hr[i] = v;
+    if (!w_next && out) out[row + i] = from_f32<act_t>(v);
     ss2 += v * v;
   }
   if (!w_next) return;
@@ -295,6 +297,7 @@ __global__ __launch_bounds__(256) void norm_add_norm_fast_kernel(
         ss2 += t * t;
       }
       store4(hr + i, v[j]);
+      if (!w_next && out) store4(out + (size_t)r * H + i, v[j]);
     }
   }
   if (!w_next) return;
@@ -403,6 +406,7 @@ __global__ __launch_bounds__(1024) void norm_add_norm_wide_kernel(
         ss2 += t * t;
       }
       store4(hr + i, v[j]);
+      if (!w_next && out) store4(out + (size_t)r * H + i, v[j]);
     }
   }
   if (!w_next) return;
@@ -725,6 +729,11 @@ __global__ void fill_normal_kernel(D* __restrict__ dst, size_t n, uint64_t seed,
   if (i + 1 < n) dst[i + 1] = from_f32<D>(mean + b);
 }
 
+__global__ void round_rows_kernel(const float* __restrict__ x, act_t* __restrict__ out, size_t n) {
+  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < n) out[i] = from_f32<act_t>(x[i]);
+}
+
 __global__ void zero_kernel(uint32_t* __restrict__ p, size_t n_words) {
   size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i < n_words) p[i] = 0u;
@@ -780,8 +789,17 @@ int zk_rmsnorm(const void* x, int x_is_f32, const int* rows, const float* w, voi
   return zk_launch_status("zk_rmsnorm");
 }
 
+// out[i] = x[i] rounded to the activation type.
+int zk_round_rows(const float* x, void* out, size_t n, void* stream) {
+  ZK_REQUIRE(x != nullptr && out != nullptr, "zk_round_rows: no rows");
+  if (n == 0) return 0;
+  round_rows_kernel<<<(unsigned)((n + 255) / 256), 256, 0, (hipStream_t)stream>>>(x, (act_t*)out, n);
+  return zk_launch_status("zk_round_rows");
+}
+
 // sub_parts > 0: sub holds that many float planes of [T, H] partial sums instead of [T, H]
-// values of the activation type (see sub_value).
+// values of the activation type (see sub_value).  An output without w_next receives the new stream
+// itself, rounded to the activation type.
 int zk_norm_add_norm(const void* sub, int sub_parts, const float* w_post, float eps_post, int uo_post, float* h,
                      const float* w_next, float eps_next, int uo_next, void* out, int T, int H,
                      void* stream) {

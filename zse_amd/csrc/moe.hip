@@ -11,6 +11,8 @@
 // weights are [E][F][W].  ``zk_gate_rows`` multiplies float rows by the sigmoid
 // of a number a row (a shared layer's gate).  ``zk_moe_route_groups`` chooses by s + a correction per
 // expert, among the experts of the best groups only, and may bring the weights to a sum.
+// Identity experts are numbers from E on that the router may choose: such an expert has no weights and gives
+// its input back, so it adds s x_t.
 //
 // Two ways through the experts.  Few tokens (decoding): one block per (token, choice) multiplies
 // the expert's rows by the token's row, and the weights stream once per choice.  Many tokens
@@ -107,14 +109,15 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
 
 // ---- the router with a correction per expert and groups of neighbouring experts: one wave per token.
 // Choice scores c = s + correction (s = sigmoid of the logits, or their softmax).  With groups, the E
-// experts form ``groups`` runs of E / groups; a group's value is the sum of its two largest c (of one, where it
-// has one), and only experts of the ``keep`` best groups can be chosen.  The ``top`` largest c are
+// experts form ``groups`` runs of E / groups; a group's value is the sum of its ``group_best`` (1 or 2) largest c
+// (of one, where it has one), and only experts of the ``keep`` best groups can be chosen.  The ``top`` largest c are
 // chosen, the lower number among equals, of groups as of experts.  Weights: s, divided by the
 // chosen ones' sum (+ 1e-20) when ``normalise``, times ``scale``.
 __global__ __launch_bounds__(64) void moe_route_groups_kernel(const float* __restrict__ logits, int ld,
                                                               const float* __restrict__ correction, int E, int top,
                                                               int groups, int keep, int softmax, int normalise, float scale,
-                                                              int* __restrict__ ids, float* __restrict__ wts) {
+                                                              int group_best, int* __restrict__ ids,
+                                                              float* __restrict__ wts) {
   __shared__ float sc[MOE_MAX_EXPERTS], ch[MOE_MAX_EXPERTS], gv[MOE_MAX_EXPERTS];
   const int t = blockIdx.x, lane = threadIdx.x;
   const float* z = logits + (size_t)t * ld;
@@ -167,7 +170,7 @@ __global__ __launch_bounds__(64) void moe_route_groups_kernel(const float* __res
           b = c;
         }
       }
-      gv[g] = size > 1 ? a + b : a;
+      gv[g] = (size > 1 && group_best > 1) ? a + b : a;
     }
     __syncthreads();
     for (int k = 0; k < keep; k++) {
@@ -246,10 +249,11 @@ __device__ __forceinline__ float row_dot(const act_t* __restrict__ w, const floa
 __global__ __launch_bounds__(256) void moe_gate_up_kernel(const act_t* __restrict__ x, const int* __restrict__ ids,
                                                           const float* __restrict__ wts, const act_t* __restrict__ w_gu,
                                                           act_t* __restrict__ y, int top, int W, int F, float limit,
-                                                          int rows_per_block, int act, int on_out) {
+                                                          int rows_per_block, int act, int on_out, int experts) {
   extern __shared__ float xs[];                   // [W]
   const int pair = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int e = ids[pair];
+  if (e >= experts) return;                       // an identity expert: nothing to multiply, the whole block alike
   const float s = wts[pair];
   const int t = pair / top;
   const act_t* xr = x + (size_t)t * W;
@@ -270,22 +274,30 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(const act_t* __restric
   }
 }
 
-// out[t, n] = sum_k Wd[e_k][n] . y[(t, k)]
+// out[t, n] = sum_k Wd[e_k][n] . y[(t, k)], an identity expert's term s_k x[t, n]
 __global__ __launch_bounds__(256) void moe_down_kernel(const act_t* __restrict__ y, const int* __restrict__ ids,
                                                        const act_t* __restrict__ w_down, float* __restrict__ out,
                                                        int top, int W, int F, int rows_per_block,
-                                                       const float* __restrict__ wts) {
+                                                       const float* __restrict__ wts, int on_out,
+                                                       const act_t* __restrict__ x, int experts) {
   extern __shared__ float ys[];                   // [top][F]
   const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  for (int i = tid; i < top * F; i += 256) ys[i] = to_f32(y[(size_t)t * top * F + i]);
+  for (int i = tid; i < top * F; i += 256)
+    ys[i] = ids[(size_t)t * top + i / F] < experts ? to_f32(y[(size_t)t * top * F + i]) : 0.f;
   __syncthreads();
   const int n0 = blockIdx.y * rows_per_block;
   for (int n = n0 + wave; n < min(W, n0 + rows_per_block); n += 4) {
     float total = 0.f;
     for (int k = 0; k < top; k++) {
-      const act_t* wr = w_down + ((size_t)ids[(size_t)t * top + k] * W + n) * F;
+      const int e = ids[(size_t)t * top + k];
+      const float s = wts[(size_t)t * top + k];
+      if (e >= experts) {
+        total += s * to_f32(x[(size_t)t * W + n]);
+        continue;
+      }
+      const act_t* wr = w_down + ((size_t)e * W + n) * F;
       const float d = row_dot(wr, ys + k * F, F, lane);
-      total += wts ? wts[(size_t)t * top + k] * d : d;
+      total += on_out ? s * d : d;
     }
     if (lane == 0) out[(size_t)t * W + n] = total;
   }
@@ -324,9 +336,11 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* __restrict__ 
 }
 
 __global__ void moe_gather_kernel(const act_t* __restrict__ x, const int* __restrict__ order,
-                                  const float* __restrict__ wts, act_t* __restrict__ xg, int top, int W) {
+                                  const float* __restrict__ wts, act_t* __restrict__ xg, int top, int W,
+                                  const int* __restrict__ ids, int experts) {
   const int i = blockIdx.x;
   const int pair = order[i];
+  if (ids[pair] >= experts) return;                       // sorted behind every expert's rows, never multiplied
   const float s = wts ? wts[pair] : 1.0f;
   const act_t* xr = x + (size_t)(pair / top) * W;
   for (int c = threadIdx.x; c < W; c += blockDim.x) xg[(size_t)i * W + c] = from_f32<act_t>(s * to_f32(xr[c]));
@@ -419,15 +433,21 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(const __bf16* __restri
   }
 }
 
-// out[t, :] = sum over t's choices, in their order, of the sorted rows' results
+// out[t, :] = sum over t's choices, in their order, of the sorted rows' results (of s x[t, :] for an identity expert)
 __global__ void moe_combine_kernel(const float* __restrict__ rows, const int* __restrict__ place, float* __restrict__ out,
-                                   int top, int W, const float* __restrict__ wts) {
+                                   int top, int W, const float* __restrict__ wts, int on_out,
+                                   const int* __restrict__ ids, const act_t* __restrict__ x, int experts) {
   const int t = blockIdx.x;
   for (int c = threadIdx.x; c < W; c += blockDim.x) {
     float total = 0.f;
     for (int k = 0; k < top; k++) {
+      const float s = wts[(size_t)t * top + k];
+      if (ids[(size_t)t * top + k] >= experts) {
+        total += s * to_f32(x[(size_t)t * W + c]);
+        continue;
+      }
       const float v = rows[(size_t)place[(size_t)t * top + k] * W + c];
-      total += wts ? wts[(size_t)t * top + k] * v : v;
+      total += on_out ? s * v : v;
     }
     out[(size_t)t * W + c] = total;
   }
@@ -467,17 +487,24 @@ int zk_moe_route(const float* logits, void* ids, float* wts, int T, int E, int t
 
 // As zk_moe_route_ext with a correction per expert (float [E], may be null: 0) that counts in the choice
 // alone, ``groups`` groups of neighbours of which ``keep`` stay (groups <= 1: none), and weights that are
-// divided by their sum (normalise) and times ``scale``.
-int zk_moe_route_groups(const float* logits, int ld, const float* correction, void* ids, float* wts, int T, int E, int top,
-                        int groups, int keep, int softmax, int normalise, float scale, void* stream) {
+// divided by their sum (normalise) and times ``scale``.  group_best: a group is judged by the sum of its that
+// many (1 or 2) largest choice scores.
+int zk_moe_route_best(const float* logits, int ld, const float* correction, void* ids, float* wts, int T, int E, int top,
+                      int groups, int keep, int softmax, int normalise, float scale, int group_best, void* stream) {
+  ZK_REQUIRE(group_best == 1 || group_best == 2, "zk_moe_route_groups: a group is judged by its one or two best");
   ZK_REQUIRE(T >= 0 && E > 0 && top > 0 && top <= E && ld >= E, "zk_moe_route_groups: bad sizes");
   ZK_REQUIRE(E <= MOE_MAX_EXPERTS && top <= MOE_MAX_TOP, "zk_moe_route_groups: up to 1024 experts and 16 choices");
   ZK_REQUIRE(groups <= 1 || (E % groups == 0 && keep >= 1 && keep <= groups && keep * (E / groups) >= top),
              "zk_moe_route_groups: equal groups, of which enough stay for the choices");
   if (T == 0) return 0;
   moe_route_groups_kernel<<<T, 64, 0, (hipStream_t)stream>>>(logits, ld, correction, E, top, groups, keep, softmax, normalise,
-                                                            scale, (int*)ids, wts);
+                                                            scale, group_best, (int*)ids, wts);
   return zk_launch_status("zk_moe_route_groups");
+}
+
+int zk_moe_route_groups(const float* logits, int ld, const float* correction, void* ids, float* wts, int T, int E, int top,
+                        int groups, int keep, int softmax, int normalise, float scale, void* stream) {
+  return zk_moe_route_best(logits, ld, correction, ids, wts, T, E, top, groups, keep, softmax, normalise, scale, 2, stream);
 }
 
 // rows: float [T, W], each multiplied by sigmoid(z[t * ld]).
@@ -491,9 +518,12 @@ int zk_gate_rows(float* rows, const float* z, int ld, int T, int W, void* stream
 // x: [T, W]; w_gu: [E][2F][W], an expert's gate rows, then its up rows; w_down: [E][W][F].
 // y: scratch [T * top, F] activations; out: float [T, W].
 // act: 0 the clamped form, 1 silu(gate) up, 2 the square of relu(up) without a gate (w_gu is then
-// [E][F][W]).  on_out: the weight multiplies the expert's output.
-int zk_moe_experts_ext(const void* x, const int* ids, const float* wts, const void* w_gu, const void* w_down, void* y,
-                       float* out, int T, int top, int W, int F, float limit, int act, int on_out, void* stream) {
+// [E][F][W]).  on_out: the weight multiplies the expert's output.  experts: numbers below it have weights,
+// numbers from it on are identity experts.
+int zk_moe_experts_identity(const void* x, const int* ids, const float* wts, const void* w_gu, const void* w_down, void* y,
+                            float* out, int T, int top, int W, int F, float limit, int act, int on_out, int experts,
+                            void* stream) {
+  ZK_REQUIRE(experts > 0, "zk_moe_experts: no experts");
   ZK_REQUIRE(T >= 0 && top > 0 && top <= MOE_MAX_TOP && W > 0 && F > 0, "zk_moe_experts: bad sizes");
   ZK_REQUIRE(T <= 65535 && (size_t)T * top <= 0x7fffffff, "zk_moe_experts: more than 65535 rows");
   ZK_REQUIRE((size_t)W * 4 <= 64 * 1024 && (size_t)top * F * 4 <= 64 * 1024, "zk_moe_experts: rows too wide for local memory");
@@ -507,11 +537,16 @@ int zk_moe_experts_ext(const void* x, const int* ids, const float* wts, const vo
   }
   dim3 grid_up(T * top, (F + rpb - 1) / rpb);
   moe_gate_up_kernel<<<grid_up, 256, (size_t)W * 4, (hipStream_t)stream>>>((const act_t*)x, ids, wts, (const act_t*)w_gu,
-                                                                          (act_t*)y, top, W, F, limit, rpb, act, on_out);
+                                                                          (act_t*)y, top, W, F, limit, rpb, act, on_out, experts);
   dim3 grid(T, (W + rpb - 1) / rpb);
   moe_down_kernel<<<grid, 256, (size_t)top * F * 4, (hipStream_t)stream>>>((const act_t*)y, ids, (const act_t*)w_down, out, top,
-                                                                         W, F, rpb, on_out ? wts : nullptr);
+                                                                         W, F, rpb, wts, on_out, (const act_t*)x, experts);
   return zk_launch_status("zk_moe_experts");
+}
+
+int zk_moe_experts_ext(const void* x, const int* ids, const float* wts, const void* w_gu, const void* w_down, void* y,
+                       float* out, int T, int top, int W, int F, float limit, int act, int on_out, void* stream) {
+  return zk_moe_experts_identity(x, ids, wts, w_gu, w_down, y, out, T, top, W, F, limit, act, on_out, 0x7fffffff, stream);
 }
 
 int zk_moe_experts(const void* x, const int* ids, const float* wts, const void* w_gu, const void* w_down, void* y,
@@ -529,24 +564,26 @@ int zk_clamped_glu(const void* gu, void* y, int T, int F, float limit, void* str
 }
 
 #if ZSE_ACT_BF16
-// The same through the grouped matrix-core product.  work: int32 [E + 1 + 2 * T * top] (first,
-// order, place); xg: [T * top, W] and y: [T * top, F] bfloat16; rows: float [T * top, W].
-int zk_moe_experts_grouped_ext(const void* x, const int* ids, const float* wts, const void* w_gu, const void* w_down,
-                               void* work, void* xg, void* y, float* rows, float* out, int T, int E, int top, int W, int F,
-                               float limit, int act, int on_out, void* stream) {
-  ZK_REQUIRE(T >= 0 && top > 0 && top <= MOE_MAX_TOP && W > 0 && F > 0 && E > 0 && E <= MOE_MAX_EXPERTS,
+// The same through the grouped matrix-core product, with ``identity`` numbers behind the E experts'.  work: int32
+// [E + identity + 1 + 2 * T * top] (first, order, place); xg: [T * top, W] and y: [T * top, F] bfloat16; rows: float
+// [T * top, W].
+int zk_moe_experts_grouped_identity(const void* x, const int* ids, const float* wts, const void* w_gu, const void* w_down,
+                                    void* work, void* xg, void* y, float* rows, float* out, int T, int E, int top, int W,
+                                    int F, float limit, int act, int on_out, int identity, void* stream) {
+  ZK_REQUIRE(T >= 0 && top > 0 && top <= MOE_MAX_TOP && W > 0 && F > 0 && E > 0 && identity >= 0 &&
+                 E + identity <= MOE_MAX_EXPERTS,
              "zk_moe_experts_grouped: bad sizes");
   ZK_REQUIRE(W % 8 == 0 && F % 8 == 0, "zk_moe_experts_grouped: widths in whole groups of eight");
   ZK_REQUIRE(T <= 65535, "zk_moe_experts_grouped: more than 65535 rows");
   if (T == 0) return 0;
   const int pairs = T * top;
   int* first = (int*)work;
-  int* order = first + E + 1;
+  int* order = first + E + identity + 1;
   int* place = order + pairs;
   hipStream_t st = (hipStream_t)stream;
-  moe_sort_kernel<<<1, 1024, 0, st>>>(ids, pairs, E, first, order);
+  moe_sort_kernel<<<1, 1024, 0, st>>>(ids, pairs, E + identity, first, order);
   moe_place_kernel<<<(pairs + 255) / 256, 256, 0, st>>>(order, place, pairs);
-  moe_gather_kernel<<<pairs, 256, 0, st>>>((const act_t*)x, order, on_out ? nullptr : wts, (act_t*)xg, top, W);
+  moe_gather_kernel<<<pairs, 256, 0, st>>>((const act_t*)x, order, on_out ? nullptr : wts, (act_t*)xg, top, W, ids, E);
   const int tiles = (pairs + GG_TM - 1) / GG_TM + E;        // each expert may end in a tile that is not full
   dim3 g0(tiles, (F + GG_TN - 1) / GG_TN);
   if (act == MOE_NO_GATE)
@@ -555,8 +592,15 @@ int zk_moe_experts_grouped_ext(const void* x, const int* ids, const float* wts, 
     moe_grouped_kernel<0><<<g0, 256, 0, st>>>((const __bf16*)xg, (const __bf16*)w_gu, first, E, F, W, (__bf16*)y, nullptr, limit, act);
   dim3 g1(tiles, (W + GG_TN - 1) / GG_TN);
   moe_grouped_kernel<1><<<g1, 256, 0, st>>>((const __bf16*)y, (const __bf16*)w_down, first, E, W, F, nullptr, rows, 0.f, 0);
-  moe_combine_kernel<<<T, 256, 0, st>>>(rows, place, out, top, W, on_out ? wts : nullptr);
+  moe_combine_kernel<<<T, 256, 0, st>>>(rows, place, out, top, W, wts, on_out, ids, (const act_t*)x, E);
   return zk_launch_status("zk_moe_experts_grouped");
+}
+
+int zk_moe_experts_grouped_ext(const void* x, const int* ids, const float* wts, const void* w_gu, const void* w_down,
+                               void* work, void* xg, void* y, float* rows, float* out, int T, int E, int top, int W, int F,
+                               float limit, int act, int on_out, void* stream) {
+  return zk_moe_experts_grouped_identity(x, ids, wts, w_gu, w_down, work, xg, y, rows, out, T, E, top, W, F, limit, act,
+                                         on_out, 0, stream);
 }
 
 int zk_moe_experts_grouped(const void* x, const int* ids, const float* wts, const void* w_gu, const void* w_down,
@@ -571,9 +615,12 @@ int zk_moe_experts_grouped(const void* x, const int* ids, const float* wts, cons
 #if ZSE_ACT_BF16
 ZK_ENTER(zk_moe_experts_grouped)
 ZK_ENTER(zk_moe_experts_grouped_ext)
+ZK_ENTER(zk_moe_experts_grouped_identity)
 #endif
 ZK_ENTER(zk_moe_route_ext)
 ZK_ENTER(zk_moe_route_groups)
+ZK_ENTER(zk_moe_route_best)
+ZK_ENTER(zk_moe_experts_identity)
 ZK_ENTER(zk_moe_experts_ext)
 ZK_ENTER(zk_gate_rows)
 ZK_ENTER(zk_moe_route)

@@ -30,6 +30,7 @@ int zk_rmsnorm(const void* x, int x_is_f32, const int* rows, const float* w, voi
                int n_rows, int H, void* stream);
 int zk_norm_add_norm(const void* sub, int sub_parts, const float* w_post, float eps_post, int uo_post, float* h,
                      const float* w_next, float eps_next, int uo_next, void* out, int T, int H, void* stream);
+int zk_round_rows(const float* x, void* out, size_t n, void* stream);
 int zk_gated_act(const void* gu, void* out, int T, int I, int act, void* stream);
 int zk_softcap(float* z, size_t n, float cap, void* stream);
 int zk_rope_cache_write(void* qkv, const int* positions, const int* slot_map, const float* inv_freq, int rotary_dim,
@@ -62,7 +63,7 @@ int zk_attention_bf16(const void* q, int q_stride, const void* kcache, const voi
 
 namespace {
 
-constexpr int MOST_ARGS = 32;
+constexpr int MOST_ARGS = 40;
 
 // One written-down call: a row of the table, and the entry point's arguments as 64-bit words
 // in the order of its C signature.  The last argument of every entry point is the stream; a
@@ -120,6 +121,7 @@ const int entered_at_load = []() {
   OWN(zk_embed);
   OWN(zk_rmsnorm);
   OWN(zk_norm_add_norm);
+  OWN(zk_round_rows);
   OWN(zk_gated_act);
   OWN(zk_softcap);
   OWN(zk_rope_cache_write);

@@ -1,2 +1,2 @@
 """Importing this package registers every architecture the engine serves."""
-from . import bizepel, bumolix, dafotar, gemma2, pubunex, rotalorn  # noqa: F401
+from . import bizepel, bumolix, buvuzen, dafotar, gemma2, pubunex, rotalorn  # noqa: F401

@@ -48,6 +48,10 @@ class PagedAttention(Part):
         self.unit_sink = bool(getattr(s, "unit_sink", False))
         self.unit_norm = bool(getattr(s, "qk_unit_norm", False))
         self.gate_name = getattr(s, "gate", None)
+        # a learned sink per head, and a gate of one number a head: both in the attention kernels' last step
+        self.sinks_name, self.head_gate_name = getattr(s, "sinks", None), getattr(s, "head_gate", None)
+        if (self.unit_sink and self.sinks_name) or (self.gate_name and self.head_gate_name):
+            raise ValueError("a sink of score 0 or learned sinks, a gate per channel or per head: not both")
         self.wide_weights = bool(getattr(s, "wide_weights", False))
         # a norm over a token's whole query row and whole key row, and values that are the keys as
         # projected: one kernel of their own between the product and the attention
@@ -87,7 +91,7 @@ class PagedAttention(Part):
         self.general = bool(self.conv or self.keep or self.lend_values or self.share_name or self.value_dim != s.head_dim or self.q_norm_name or self.k_norm_name or
                             self.head_scale_name or self.value_base or self.bias_names or
                             self.rot_scale != 1.0 or self.rot_interleaved or self.chunk or self.unit_sink or self.wide_weights or
-                            self.unit_norm or self.gate_name or self.by_rows)
+                            self.unit_norm or self.gate_name or self.sinks_name or self.head_gate_name or self.by_rows)
         if self.by_rows:
             if (self.q_norm_name or self.k_norm_name or self.head_scale_name or self.value_base or self.unit_norm
                     or self.rot_scale != 1.0 or self.rot_interleaved or self.shared_kv):
@@ -102,7 +106,7 @@ class PagedAttention(Part):
             raise ValueError(f"value_dim up to 256, got {self.value_dim}")
         if self.value_base and self.value_dim % 2:
             raise ValueError(f"rotated values need an even value_dim, got {self.value_dim}")
-        self.q_gain = self.k_gain = self.head_scale = self.value_freq = None
+        self.q_gain = self.k_gain = self.head_scale = self.value_freq = self.sinks = None
         self.q_row_gain = self.k_row_gain = None
         self.decode_chunk = 64                     # keys a wave of the split decode attention takes
 
@@ -126,6 +130,10 @@ class PagedAttention(Part):
             out.append(TensorReq(self.head_scale_name, (s.num_heads,), ROLE_GAIN))
         if self.gate_name:
             out.append(TensorReq(self.gate_name, (s.num_heads * self.value_dim, s.hidden_size)))
+        if self.head_gate_name:
+            out.append(TensorReq(self.head_gate_name, (s.num_heads, s.hidden_size)))
+        if self.sinks_name:
+            out.append(TensorReq(self.sinks_name, (s.num_heads,), ROLE_GAIN))
         for role, rows in (("q", s.num_heads * s.head_dim), ("o", s.hidden_size)):
             if role in self.bias_names:
                 out.append(TensorReq(self.bias_names[role], (rows,), ROLE_GAIN))
@@ -149,8 +157,9 @@ class PagedAttention(Part):
         s = self.spec
         stored = ("q", "k") if self.values_are_keys else ("q", "k", "v")
         names = [s.names["q"]] if self.shared_kv else [s.names[r] for r in stored]
-        if self.gate_name:
-            names.append(self.gate_name)       # the gate's rows behind q, k, v: one product
+        if self.gate_name or self.head_gate_name:
+            names.append(self.gate_name or self.head_gate_name)       # the gate's rows behind q, k, v: one product
+        self.sinks = weights.vector(self.sinks_name) if self.sinks_name else None
         strip = getattr(weights, "wants_strip", None)
         self.w_qkv = weights.matrix(names, strip=True) if strip and strip(s.hidden_size) else weights.matrix(names)
         o_cols = s.num_heads * self.value_dim
@@ -240,10 +249,12 @@ class PagedAttention(Part):
         nh, nkv, hd, vd = s.num_heads, s.num_kv_heads, s.head_dim, self.value_dim
         n_store = 0 if self.shared_kv else nkv
         heads_width = (nh + n_store) * hd + (0 if self.values_are_keys else n_store * vd)
-        width = heads_width + (nh * vd if self.gate_name else 0)
+        width = heads_width + (nh * vd if self.gate_name else nh if self.head_gate_name else 0)
+        if self.head_gate_name:
+            width = -(-width // 8) * 8       # rows of queries begin at 16-byte addresses; the columns behind the gate stay empty
         g = ctx.group(cache.group)
         tables = self.position.rotary_tables()
-        rows = qkv = linear(ctx, x, self.w_qkv, ctx.alloc((T, width)))
+        rows = qkv = linear(ctx, x, self.w_qkv, ctx.alloc((T, width)), ldc=width)
         row_width = width            # of the projected rows, which may hold a gate behind the heads
         if self.conv is not None:
             qkv, width = self.conv.forward(ctx, rows, cache.state_offset, ld=row_width), heads_width
@@ -282,19 +293,21 @@ class PagedAttention(Part):
         o = ctx.alloc((T, nh * vd))
         cap = float(s.softcap) if s.softcap else 0.0
         win = int(s.window) if s.window else 0
+        head_gate = rows.ptr + heads_width * ITEMSIZE[ctx.dtype] if self.head_gate_name else None
         if cache.v_transposed and ctx.tuned:
-            k.zk_attention_bf16_sized(qkv.ptr, width, cache.k.ptr, cache.v.ptr, g.block_table, g.max_blocks,
+            k.zk_attention_bf16_gated(qkv.ptr, width, cache.k.ptr, cache.v.ptr, g.block_table, g.max_blocks,
                                       ctx.q_start, ctx.ctx_len, o.ptr, ctx.R, ctx.n_multi, ctx.max_q_len,
                                       ctx.max_ctx, nh, nkv, hd, g.page_size, s.scale, cap, win,
                                       self.decode_chunk, ctx.workspace.ptr, ctx.workspace.nbytes, self.chunk,
-                                      1 if self.unit_sink else 0, 1 if self.wide_weights else 0, 0, vd, self.keep, ctx.stream)
+                                      1 if self.unit_sink else 0, 1 if self.wide_weights else 0, 0, vd, self.keep,
+                                      ptr(self.sinks), head_gate, row_width, ctx.stream)
             if vfreq is not None:
                 k.zk_rotate_heads(o.ptr, ctx.positions, vfreq, T, nh, vd, inter, -1.0, ctx.stream)
         else:
-            k.zk_attention_plain_kept(qkv.ptr, width, cache.k.ptr, cache.v.ptr, g.block_table, g.max_blocks,
+            k.zk_attention_plain_gated(qkv.ptr, width, cache.k.ptr, cache.v.ptr, g.block_table, g.max_blocks,
                                       ctx.req_of_token, ctx.positions, o.ptr, T, nh, nkv, hd, vd, g.page_size, s.scale,
-                                      cap, win, 1 if cache.v_transposed else 0, vfreq, inter, None, 0, self.chunk,
-                                      1 if self.unit_sink else 0, self.keep, ctx.stream)
+                                      cap, win, 1 if cache.v_transposed else 0, vfreq, inter, ptr(self.sinks), 0, self.chunk,
+                                      1 if self.unit_sink else 0, self.keep, head_gate, row_width, ctx.stream)
         if self.gate_name:
             # the heads times sigmoid(W_g x); the gate's columns lie behind the heads' in the product's rows
             k.zk_gate_heads(o.ptr, rows.ptr + heads_width * ITEMSIZE[ctx.dtype], row_width, T, nh * vd, ctx.stream)

@@ -3,17 +3,20 @@
 "sandwich" is Gemma 2's order of four norms,
     h += post_m(mixer(pre_m(h)));  h += post_f(ffn(pre_f(h)))
 the order of the reference's Gemma-family block (orchestrator/model_runner.py:425-439,
-450-537).  "prenorm" leaves the post norms out (its Llama block, :1123-1297).  The
-residual sum stays float throughout (orchestrator/vram_allocator.py:70-72).
+450-537).  "prenorm" leaves the post norms out (its Llama block, :1123-1297).  "postnorm" leaves the pre norms out,
+    h += post_m(mixer(h));  h += post_f(ffn(h))
+so that its sublayers read the stream itself.  The residual sum stays float throughout (orchestrator/vram_allocator.py:70-72).
 """
 from __future__ import annotations
 
 from ..runtime.device import Tensor
+from ..config.plan import NoNormSpec
 from .base import Part, build_part, register_part
-from .norm import LayerNorm, RMSNorm
+from .norm import LayerNorm, NoNorm, RMSNorm
 
 ARRANGEMENTS = {"sandwich": ("pre_mixer", "post_mixer", "pre_ffn", "post_ffn"),
-                "prenorm": ("pre_mixer", "pre_ffn")}
+                "prenorm": ("pre_mixer", "pre_ffn"),
+                "postnorm": ("post_mixer", "post_ffn")}
 
 
 class Block(Part):
@@ -23,23 +26,26 @@ class Block(Part):
         if spec.arrangement not in ARRANGEMENTS:
             raise ValueError(f"arrangement must be one of {sorted(ARRANGEMENTS)}, got {spec.arrangement!r}")
         self.spec = spec
-        roles = ARRANGEMENTS[spec.arrangement]
+        roles = [r for r in ARRANGEMENTS[spec.arrangement] if spec.ffn is not None or not r.endswith("_ffn")]
         missing = [r for r in roles if r not in spec.norms]
         if missing:
             raise ValueError(f"a {spec.arrangement} block needs norms {missing}")
         self.norms = {r: build_part("norm", spec.norms[r]) for r in roles}
+        if spec.arrangement == "postnorm":
+            size = spec.norms["post_mixer"].size
+            self.norms.update({r: build_part("norm", NoNormSpec(size)) for r in ("pre_mixer", "pre_ffn")})
         self.mixer = build_part("mixer", spec.mixer)
-        self.ffn = build_part("ffn", spec.ffn)
+        self.ffn = build_part("ffn", spec.ffn) if spec.ffn is not None else None
 
     def children(self):
-        return list(self.norms.values()) + [self.mixer, self.ffn]
+        return list(self.norms.values()) + [self.mixer] + ([self.ffn] if self.ffn is not None else [])
 
     def _join(self, ctx, sub: Tensor, post, h: Tensor, nxt, out: Tensor = None):
         """h += post(sub) (post None: h += sub); returns nxt(h) if nxt is given, written
-        to ``out`` when the caller brings a buffer."""
+        to ``out`` when the caller brings a buffer (no norm: h itself, in the activation type)."""
         T, H = h.shape
         fused_post = post is None or isinstance(post, RMSNorm)
-        fused_next = nxt is None or isinstance(nxt, RMSNorm)
+        fused_next = nxt is None or isinstance(nxt, (RMSNorm, NoNorm))
         if not fused_post:
             sub, post = post.forward(ctx, sub), None
         if nxt is None or not fused_next:
@@ -47,7 +53,7 @@ class Block(Part):
         elif out is None:
             out = ctx.alloc((T, H))
         ps = post.spec if post is not None else None
-        ns = nxt.spec if (nxt is not None and fused_next) else None
+        ns = nxt.spec if isinstance(nxt, RMSNorm) else None
         parts = sub.shape[0] if sub.layout == "parts" else 0     # partial sums of a product that split K
         ctx.k.zk_norm_add_norm(
             sub.ptr, parts, post.weight.ptr if post is not None else None, ps.eps if ps else 0.0,
@@ -75,14 +81,17 @@ class Block(Part):
         n = self.norms
         x = x_in if x_in is not None else n["pre_mixer"].forward(ctx, h)
         # the joining kernel adds up the partial sums of a part's last product itself
+        if not isinstance(next_norm, (RMSNorm, NoNorm)):
+            next_norm = None         # a norm the closing kernel does not know: the next block applies it
         ctx.sums_welcome = self.mixer if self._joins_sums(n.get("post_mixer")) else None
         a = self.mixer.forward(ctx, x, cache)
+        if self.ffn is None:
+            ctx.sums_welcome = None
+            return self._join(ctx, a, n.get("post_mixer"), h, next_norm, x_out)
         x = self._join(ctx, a, n.get("post_mixer"), h, n["pre_ffn"])
         ctx.sums_welcome = self.ffn if self._joins_sums(n.get("post_ffn")) else None
         m = self.ffn.forward(ctx, x)
         ctx.sums_welcome = None
-        if not isinstance(next_norm, RMSNorm):
-            next_norm = None         # a norm the closing kernel does not know: the next block applies it
         return self._join(ctx, m, n.get("post_ffn"), h, next_norm, x_out)
 
 

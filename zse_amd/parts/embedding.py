@@ -55,9 +55,9 @@ class Embedding(Part):
         self.table = (weights.matrix([self.spec.weight], strip=True) if strip and strip(self.spec.hidden_size)
                       else weights.matrix([self.spec.weight]))
         # the scalar is kept in the table's storage type, as the reference keeps its own
-        # (model_runner.py:155-158); the product is float
+        # (model_runner.py:155-158), unless the spec says otherwise; the product is float
         s = np.float32(self.spec.scale)
-        if dtype == BF16:
+        if dtype == BF16 and not getattr(self.spec, "exact_scale", False):
             from ..weights.safetensors import bf16_bits_to_f32, f32_to_bf16_bits
             s = bf16_bits_to_f32(f32_to_bf16_bits(np.array([s])))[0]
         self.scale = float(s)

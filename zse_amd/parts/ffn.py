@@ -111,7 +111,8 @@ class MLP(Part):
 class RoutedMLP(Part):
     """A mixture of small layers (gated, or without a gate): scores from a float router product (sigmoids, or a softmax
     over all experts), the ``top_k`` largest chosen on the device (the lower index among equals;
-    optionally by score plus a correction, among the experts of the best groups only),
+    optionally by score plus a correction, among the experts of the best groups only; some of the numbers
+    to choose from may stand for identity experts, which have no weights and give their input back),
     the chosen scores as weights on the experts' inputs or on their outputs, the experts' results
     added in the order they were chosen, a shared layer on top (optionally times the sigmoid of a
     number a token, whose row rides below the router's in one product).  Steps of few tokens read each chosen expert's rows once per (token, choice); steps of
@@ -131,18 +132,25 @@ class RoutedMLP(Part):
             raise ValueError(f"experts without a gate are relu2 layers with weights on their results, got {s.activation!r}")
         self.correction_name = getattr(s, "correction", None)
         self.groups = tuple(getattr(s, "groups", None) or (1, 1))
-        if s.num_experts % self.groups[0] or not (1 <= self.groups[1] <= self.groups[0]) or \
-                self.groups[1] * (s.num_experts // self.groups[0]) < s.top_k:
-            raise ValueError(f"equal groups of experts of which enough stay for {s.top_k} choices, got {s.num_experts} "
+        self.group_best = int(getattr(s, "group_best", 2))
+        self.identity = int(getattr(s, "identity", 0) or 0)
+        n = self.choices = s.num_experts + self.identity          # what the router chooses from
+        if self.identity < 0 or s.num_experts < 1:
+            raise ValueError(f"at least one expert and no fewer than 0 identity experts, got {s.num_experts} and {self.identity}")
+        if n % self.groups[0] or not (1 <= self.groups[1] <= self.groups[0]) or \
+                self.groups[1] * (n // self.groups[0]) < s.top_k:
+            raise ValueError(f"equal groups of experts of which enough stay for {s.top_k} choices, got {n} "
                              f"experts in {self.groups[0]} groups, {self.groups[1]} kept")
+        if self.group_best not in (1, 2):
+            raise ValueError(f"a group is judged by its one or two best scores, got {self.group_best}")
         # a choice by anything but the scores alone, or weights that are not the scores: the wider router kernel
         self.wide_route = bool(self.correction_name or self.groups != (1, 1) or getattr(s, "normalise", False)
                                or getattr(s, "weight_scale", 1.0) != 1.0)
         self.correction = None
         if self.gated and s.activation not in (CLAMPED, "silu"):
             raise ValueError(f"routed experts are {CLAMPED} or silu layers, got {s.activation!r}")
-        if not (1 <= s.top_k <= min(s.num_experts, 16)) or s.num_experts > 1024:
-            raise ValueError(f"1 to 16 of up to 1024 experts a token, got {s.top_k} of {s.num_experts}")
+        if not (1 <= s.top_k <= min(n, 16)) or n > 1024:
+            raise ValueError(f"1 to 16 of up to 1024 experts a token, got {s.top_k} of {n}")
         if s.activation == CLAMPED and not (s.limit or 0) > 0:
             raise ValueError(f"{CLAMPED} needs a positive limit, got {s.limit!r}")
         self.scoring = getattr(s, "scoring", "sigmoid")
@@ -162,11 +170,11 @@ class RoutedMLP(Part):
 
     def tensor_reqs(self) -> List[TensorReq]:
         s = self.spec
-        out = [TensorReq(s.router, (s.num_experts, s.hidden_size))]
+        out = [TensorReq(s.router, (self.choices, s.hidden_size))]
         if self.shared_gate:
             out.append(TensorReq(self.shared_gate, (1, s.hidden_size)))
         if self.correction_name:
-            out.append(TensorReq(self.correction_name, (s.num_experts,), ROLE_GAIN))
+            out.append(TensorReq(self.correction_name, (self.choices,), ROLE_GAIN))
         for e in range(s.num_experts):
             if self.gated:
                 out.append(TensorReq(self._name(e, "gate"), (s.intermediate_size, s.hidden_size)))
@@ -185,42 +193,45 @@ class RoutedMLP(Part):
         self.w_down = weights.matrix([self._name(e, "down") for e in range(s.num_experts)])
 
     def flops_per_token(self) -> float:
+        # (with identity experts: as many experts at work as an even choice gives)
         s = self.spec
-        return 2.0 * s.num_experts * s.hidden_size + s.top_k * (6.0 if self.gated else 4.0) * s.intermediate_size * s.hidden_size
+        at_work = s.top_k * s.num_experts / self.choices
+        return 2.0 * self.choices * s.hidden_size + at_work * (6.0 if self.gated else 4.0) * s.intermediate_size * s.hidden_size
 
     def forward(self, ctx, x: Tensor) -> Tensor:
         s, k = self.spec, ctx.k
         T, W, F, E, top = x.shape[0], s.hidden_size, s.intermediate_size, s.num_experts, s.top_k
-        ld = E + (1 if self.shared_gate else 0)
+        n = self.choices
+        ld = n + (1 if self.shared_gate else 0)
         logits = linear(ctx, x, self.w_router, ctx.alloc((T, ld), F32))
         ids, wts = ctx.alloc((T, top), I32), ctx.alloc((T, top), F32)
         softmax = 1 if self.scoring == "softmax" else 0
         if self.wide_route:
-            k.zk_moe_route_groups(logits.ptr, ld, self.correction.ptr if self.correction is not None else None, ids.ptr, wts.ptr,
-                                  T, E, top, self.groups[0], self.groups[1], softmax, 1 if getattr(s, "normalise", False) else 0,
-                                  float(getattr(s, "weight_scale", 1.0)), ctx.stream)
+            k.zk_moe_route_best(logits.ptr, ld, self.correction.ptr if self.correction is not None else None, ids.ptr, wts.ptr,
+                                T, n, top, self.groups[0], self.groups[1], softmax, 1 if getattr(s, "normalise", False) else 0,
+                                float(getattr(s, "weight_scale", 1.0)), self.group_best, ctx.stream)
         else:
-            k.zk_moe_route_ext(logits.ptr, ld, ids.ptr, wts.ptr, T, E, top, softmax, ctx.stream)
+            k.zk_moe_route_ext(logits.ptr, ld, ids.ptr, wts.ptr, T, n, top, softmax, ctx.stream)
         act, on_out, limit = (2 if not self.gated else 1 if s.activation == "silu" else 0), (0 if s.scale_input else 1), float(s.limit or 0.0)
         P = 2 if self.shared is not None else 1
         planes = ctx.alloc((P, T, W), F32)
         y = ctx.alloc((T * top, F))
         enough = T * top >= (self.GROUPED_WIDE_FROM if W * F >= self.WIDE else self.GROUPED_FROM)
         grouped = (ctx.dtype == BF16 and ctx.tuned and enough and W % 8 == 0 and F % 8 == 0
-                   and k.has("zk_moe_experts_grouped_ext"))
+                   and k.has("zk_moe_experts_grouped_identity"))
         if grouped:
-            work = ctx.alloc((E + 1 + 2 * T * top,), I32)
+            work = ctx.alloc((n + 1 + 2 * T * top,), I32)
             xg, rows = ctx.alloc((T * top, W)), ctx.alloc((T * top, W), F32)
-            k.zk_moe_experts_grouped_ext(x.ptr, ids.ptr, wts.ptr, self.w_gu.ptr, self.w_down.ptr, work.ptr, xg.ptr, y.ptr,
-                                         rows.ptr, planes.ptr, T, E, top, W, F, limit, act, on_out, ctx.stream)
+            k.zk_moe_experts_grouped_identity(x.ptr, ids.ptr, wts.ptr, self.w_gu.ptr, self.w_down.ptr, work.ptr, xg.ptr, y.ptr,
+                                              rows.ptr, planes.ptr, T, E, top, W, F, limit, act, on_out, self.identity, ctx.stream)
         else:
-            k.zk_moe_experts_ext(x.ptr, ids.ptr, wts.ptr, self.w_gu.ptr, self.w_down.ptr, y.ptr, planes.ptr, T, top, W, F,
-                                 limit, act, on_out, ctx.stream)
+            k.zk_moe_experts_identity(x.ptr, ids.ptr, wts.ptr, self.w_gu.ptr, self.w_down.ptr, y.ptr, planes.ptr, T, top, W, F,
+                                      limit, act, on_out, E, ctx.stream)
         if self.shared is not None:
             second = planes.rows(1, 2).view(T, W)
             self.shared.forward(ctx, x, out=second)
             if self.shared_gate:
-                k.zk_gate_rows(second.ptr, logits.ptr + E * 4, ld, T, W, ctx.stream)
+                k.zk_gate_rows(second.ptr, logits.ptr + n * 4, ld, T, W, ctx.stream)
         if getattr(ctx, "sums_welcome", None) is self:
             # the block's joining kernel adds the planes up itself
             return Tensor(planes.ptr, (P, T, W), F32, planes.owner, layout="parts")

@@ -1,4 +1,4 @@
-"""Root-mean-square norm, gain (1 + w) or w; layer norm with gain and bias.
+"""Root-mean-square norm, gain (1 + w) or w; layer norm with gain and bias; no norm.
 
 Statistics and the product are float; rsqrt(mean(x^2) + eps) as in the
 reference's kernel (orchestrator/kernels.py:1435-1465); the reference multiplies
@@ -6,6 +6,7 @@ by plain w and names the (1 + w) form of Gemma 2 in a comment (:1476-1478).
 """
 from __future__ import annotations
 
+from dataclasses import replace
 from typing import List, Optional
 
 import numpy as np
@@ -18,14 +19,21 @@ class RMSNorm(Part):
     graph_safe = True      # its launches take what changes from step to step from device memory alone
 
     def __init__(self, spec):
-        self.spec = spec
+        self.spec = self.given = spec
         self.weight: Optional[Tensor] = None
 
     def tensor_reqs(self) -> List[TensorReq]:
         return [TensorReq(self.spec.weight, (self.spec.size,), ROLE_GAIN)]
 
     def load(self, weights, rt, dtype):
-        self.weight = weights.vector(self.spec.weight)
+        s = self.given
+        self.weight = weights.vector(s.weight)
+        scale = float(getattr(s, "gain_scale", 1.0))
+        if scale != 1.0:
+            # the whole gain, as the kernels see it from now on
+            gain = rt.download(self.weight) + np.float32(1.0 if s.unit_offset else 0.0)
+            self.weight = rt.upload((gain * np.float32(scale)).astype(np.float32))
+            self.spec = replace(s, unit_offset=False, gain_scale=1.0)
 
     def forward(self, ctx, x: Tensor, out_rows=None) -> Tensor:
         """Norm of every row of ``x`` (float stream or activations), or of the rows
@@ -87,5 +95,21 @@ class LayerNorm(Part):
         return out
 
 
+class NoNorm(Part):
+    """Stands where a sublayer reads the stream itself: its rows in the activation type."""
+    graph_safe = True      # its launches take what changes from step to step from device memory alone
+
+    def __init__(self, spec):
+        self.spec = spec
+
+    def forward(self, ctx, x: Tensor, out_rows=None) -> Tensor:
+        if x.dtype != F32 or out_rows is not None:
+            raise ValueError(f"all rows of the float stream, got {x.dtype} {x.shape}")
+        out = ctx.alloc(x.shape)
+        ctx.k.zk_round_rows(x.ptr, out.ptr, x.numel, ctx.stream)
+        return out
+
+
 register_part("norm", "rmsnorm", RMSNorm)
+register_part("norm", "none", NoNorm)
 register_part("norm", "layernorm", LayerNorm)

@@ -17,7 +17,7 @@ def tuned_gemm(ctx, K: int) -> bool:
 
 
 def linear(ctx, x: Tensor, w: Tensor, out: Tensor, epilogue=None, cap: float = 0.0, last_of=None,
-           sums_ok: bool = False, lda: int = 0) -> Tensor:
+           sums_ok: bool = False, lda: int = 0, ldc: int = 0) -> Tensor:
     """out[M, N] = x[M, K] @ w[N, K]^T with float accumulation.
 
     ``out`` may be float32 (logits) or the activation type.  In the 32-bit
@@ -28,7 +28,8 @@ def linear(ctx, x: Tensor, w: Tensor, out: Tensor, epilogue=None, cap: float = 0
     its limit: g = min(gate, cap), u = clamp(up, -cap, cap), g sigmoid(1.702 g) (u + 1).
 
     "relu2" stores max(x, 0)^2, "gelu" x (1 + erf(x / sqrt(2))) / 2.  ``lda``: the distance between the rows of ``x`` in elements
-    where they are the first K columns of wider rows (0: K).
+    where they are the first K columns of wider rows (0: K).  ``ldc``: the same for the rows of ``out``, whose
+    columns behind the N-th are left as they are (0: N; ``out`` is then [M, N], else [M, ldc]).
 
     ``last_of``: the part whose result this product is (it passes itself).  When the block
     that called that very part has said that partial sums are welcome (``ctx.sums_welcome`` is
@@ -46,7 +47,10 @@ def linear(ctx, x: Tensor, w: Tensor, out: Tensor, epilogue=None, cap: float = 0
         N //= 2
     if epilogue is not None and not tuned_gemm(ctx, K):
         raise ValueError("linear: epilogues belong to the matrix-core product")
-    if K != K2 or out.shape != (M, N):
+    ldc = int(ldc) or N
+    if ldc < N:
+        raise ValueError(f"linear: rows {ldc} apart hold no {N} columns")
+    if K != K2 or out.shape != (M, ldc):
         raise ValueError(f"linear: x {x.shape}, w {w.shape}, out {out.shape} do not fit")
     if x.dtype != ctx.dtype or w.dtype != ctx.dtype:
         raise ValueError(f"linear: operands must be {ctx.dtype}, got x {x.dtype}, w {w.dtype}")
@@ -66,12 +70,12 @@ def linear(ctx, x: Tensor, w: Tensor, out: Tensor, epilogue=None, cap: float = 0
         ws = getattr(ctx, "gemm_workspace", None)      # lets a product of few columns split K over blocks
         welcome = sums_ok or (last_of is not None and getattr(ctx, "sums_welcome", None) is last_of)
         parts = ctypes.c_int(0) if (welcome and ws is not None) else None
-        k.zk_gemm_bf16(x.ptr, lda, w.ptr, out.ptr, N, out_f32, M, N, K, EPILOGUES[epilogue], float(cap),
+        k.zk_gemm_bf16(x.ptr, lda, w.ptr, out.ptr, ldc, out_f32, M, N, K, EPILOGUES[epilogue], float(cap),
                        1 if strip else 0, ws.ptr if ws is not None else None,
                        ws.nbytes if ws is not None else 0, ctypes.byref(parts) if parts is not None else None,
                        ctx.stream)
         if parts is not None and parts.value > 0:
             return Tensor(ws.ptr, (parts.value, M, N), F32, ws.owner, layout="parts")
     else:
-        k.zk_gemm_plain(x.ptr, lda, w.ptr, out.ptr, N, out_f32, M, N, K, ctx.stream)
+        k.zk_gemm_plain(x.ptr, lda, w.ptr, out.ptr, ldc, out_f32, M, N, K, ctx.stream)
     return out

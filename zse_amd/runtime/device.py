@@ -145,6 +145,7 @@ KERNEL_SIGNATURES = {
     "zk_embed": [_VP, _VP, _VP, _F, _I, _I, _I, _I, _VP],
     "zk_rmsnorm": [_VP, _I, _VP, _VP, _VP, _F, _I, _I, _I, _VP],
     "zk_norm_add_norm": [_VP, _I, _VP, _F, _I, _VP, _VP, _F, _I, _VP, _I, _I, _VP],
+    "zk_round_rows": [_VP, _VP, _SZ, _VP],
     "zk_gated_act": [_VP, _VP, _I, _I, _I, _VP],
     "zk_softcap": [_VP, _SZ, _F, _VP],
     "zk_rope_cache_write": [_VP, _VP, _VP, _VP, _I, _VP, _VP, _I, _I, _I, _I, _I, _I, _VP],
@@ -231,6 +232,10 @@ KERNEL_SIGNATURES = {
     "zk_moe_route_groups": [_VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _F, _VP],
     "zk_attention_plain_kept": [_VP, _I, _VP, _VP, _VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _F, _F,
                                 _I, _I, _VP, _I, _VP, _I, _I, _I, _I, _VP],
+    "zk_moe_route_best": [_VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _F, _I, _VP],
+    "zk_moe_experts_identity": [_VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _F, _I, _I, _I, _VP],
+    "zk_attention_plain_gated": [_VP, _I, _VP, _VP, _VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _F, _F,
+                                 _I, _I, _VP, _I, _VP, _I, _I, _I, _I, _VP, _I, _VP],
     "zk_gdelta_gates": [_VP, _I, _I, _I, _VP, _VP, _VP, _VP, _VP, _I, _I, _VP],
     "zk_gdelta": [_VP, _I, _I, _I, _VP, _I, _VP, _VP, _VP, _VP, _I, _I, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _F, _VP],
 }
@@ -255,6 +260,9 @@ BF16_KERNEL_SIGNATURES = {
     "zk_moe_experts_grouped_ext": [_VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _F, _I, _I, _VP],
     "zk_attention_bf16_sized": [_VP, _I, _VP, _VP, _VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I,
                                 _F, _F, _I, _I, _VP, _SZ, _I, _I, _I, _I, _I, _I, _VP],
+    "zk_attention_bf16_gated": [_VP, _I, _VP, _VP, _VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I,
+                                _F, _F, _I, _I, _VP, _SZ, _I, _I, _I, _I, _I, _I, _VP, _VP, _I, _VP],
+    "zk_moe_experts_grouped_identity": [_VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _F, _I, _I, _I, _VP],
     "zk_gdelta_chunked": [_VP, _I, _I, _I, _VP, _I, _VP, _VP, _VP, _VP, _I, _I, _VP, _VP, _VP, _VP, _VP, _VP, _SZ, _I, _I, _I, _I,
                           _I, _F, _VP],
     "zk_gdelta_token": [_VP, _I, _I, _I, _VP, _I, _VP, _VP, _VP, _VP, _I, _I, _VP, _VP, _VP, _VP, _I, _I, _I, _F, _VP],
