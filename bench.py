@@ -540,6 +540,26 @@ def bizepel_config(width, heads, kv_heads, dim, ff, groups, vocab, window):
             "token_side": {"dim": width // 8}, "logit_scale": 0.5, "layers": layers}
 
 
+def buvuzen_config(width, heads, kv_heads, dim, ff, groups, vocab, window):
+    """Three times ``groups`` layers with weights of their own: the windowed attention with the relative's heads, a sink
+    and a gate a head, and eight routed experts of a quarter of the feed-forward size beside four identity experts, in
+    three groups of which two stay, two a token, and a shared expert of half of the feed-forward size."""
+    layer = {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+                                            "mask": {"size": window}},
+             "mlp": {"kind": "moe", "expert": {"ff": ff // 4},
+                     "router": {"experts": 8, "top": 2, "identity": 4, "scale": 2.5, "groups": {"count": 3, "keep": 2}},
+                     "shared": {"ff": ff // 2}}}
+    return {"architecture": "Buvuzen", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 40.0},
+            "logit_scale": 0.5, "layers": [dict(layer) for _ in range(3 * groups)]}
+
+
+def rotalorn_attention_config(width, heads, kv_heads, dim, ff, groups, vocab, window):
+    """Rotalorn with as many layers, all of them its windowed attention with routed silu experts."""
+    cfg = rotalorn_config(width, heads, kv_heads, dim, ff, groups, vocab, window)
+    one = next(l for l in cfg["layers"] if l["type"] == "attention")
+    return dict(cfg, layers=[dict(one) for _ in range(3 * groups)])
+
+
 # what is timed, beside which relative, against which plain implementation it is checked first, and
 # the deviations of the random tensors that are not drawn like matrices or gains
 DESIGNS = {
@@ -557,6 +577,13 @@ DESIGNS = {
                     std_of={".b": 0.02, ".conv": 0.3, "canon": 0.3, "A_log": 0.5, "dt.b": 0.5, "a.b": 0.5, ".D": 0.5, "norm": 1.0,
                             ".ls": 0.5, "w0": 1.0, "correction": 0.1, "router": 0.03, "vmix": 0.3},
                     beside=("pubunex", "Pubunex", pubunex_config)),
+    "buvuzen": dict(name="Buvuzen", make=buvuzen_config, plain="buvuzen_plain",
+                    std_of={"q.norm": 1.0, "k.norm": 1.0, ".sink": 1.0, "correction": 0.1, "router": 0.03},
+                    # a choice that rounding decides the other way moves the token's stream by its own size, behind the norm of
+                    # the result, and with it the rows that attend to the token: in the bfloat16 half of the check the
+                    # corrections lie so far apart that few choices are that close
+                    std_of_bf16_check={"q.norm": 1.0, "k.norm": 1.0, ".sink": 1.0, "correction": 3.0, "router": 0.02},
+                    beside=("rotalorn", "Rotalorn, attention layers alone,", rotalorn_attention_config)),
     "bumolix": dict(name="Bumolix", make=bumolix_config, plain="bumolix_plain",
                     std_of={".b": 0.02, ".conv": 0.3, "A_log": 0.5, "dt.b": 0.5, "a2.b": 1.0, ".D": 0.5, "norm": 0.5},
                     beside=("dafotar", "Dafotar", dafotar_config)),
@@ -574,11 +601,12 @@ def state_bytes_touched(model):
     return total
 
 
-def check_design_slice(cfg, rt, seed, std, gain_std, std_of, plain="dafotar_plain"):
+def check_design_slice(cfg, rt, seed, std, gain_std, std_of, plain="dafotar_plain", std_of_bf16=None):
     """The first three layers of the model that is timed, at full width, against the plain
     implementation under ``tests/plain`` on the same weights made on the host: a prompt of 150 tokens
     whole (the mLSTM's chunks side by side), another in portions and then token by token beside a
-    third, in 32-bit and in bfloat16.  The head is restricted to the first 4,096 rows of the embedding."""
+    third, in 32-bit and in bfloat16.  The head is restricted to the first 4,096 rows of the embedding.
+    ``std_of_bf16``: other deviations for the bfloat16 half."""
     import importlib
     sys.path.insert(0, os.path.join(ROOT, "tests"))
     P = importlib.import_module("plain." + plain)
@@ -592,7 +620,8 @@ def check_design_slice(cfg, rt, seed, std, gain_std, std_of, plain="dafotar_plai
     host_cfg = dict(small, vocab=Vc)
     arch = resolve_architecture(host_cfg)
     plan = arch.plan(arch.config_from_dict(host_cfg))
-    w32 = random_tensors(Model(plan).tensor_reqs(), seed, std, gain_std, std_of, plan.optional_prefixes)
+    drawn = lambda how: random_tensors(Model(plan).tensor_reqs(), seed, std, gain_std, how, plan.optional_prefixes)
+    w32 = drawn(std_of)
     rng = np.random.default_rng(11)
     streams = {"a": rng.integers(0, Vc, 150).tolist(), "b": rng.integers(0, Vc, 90).tolist(),
                "c": rng.integers(0, Vc, 21).tolist()}
@@ -600,8 +629,9 @@ def check_design_slice(cfg, rt, seed, std, gain_std, std_of, plain="dafotar_plai
     steps += [[("b", 1), ("c", 3 if i == 0 else 1)] for i in range(13)]
     out = {}
     for dtype in ("float32", "bfloat16"):
-        w = w32 if dtype == "float32" else {n: bf16_round(t) for n, t in w32.items()}
-        model = random_model(small, dtype, seed=seed, std=std, gain_std=gain_std, rt=rt, std_of=std_of)
+        how = std_of if dtype == "float32" or std_of_bf16 is None else std_of_bf16
+        w = w32 if dtype == "float32" else {n: bf16_round(t) for n, t in (w32 if how is std_of else drawn(how)).items()}
+        model = random_model(small, dtype, seed=seed, std=std, gain_std=gain_std, rt=rt, std_of=how)
         runner = StepRunner(model, rt, dtype, page_size=16, cache_tokens=512, max_seqs=4, max_batch_tokens=256,
                             max_model_len=256, use_graphs=False)
         fed = {r: 0 for r in streams}
@@ -676,7 +706,7 @@ def run_design(a):
                 continue
             std_of = DESIGNS[which]["std_of"] if which in DESIGNS else {}
             if which == a.design and not a.no_check and not a.only:
-                errs = check_design_slice(cfg, rt, 0, 0.02, 0.1, std_of, design["plain"])
+                errs = check_design_slice(cfg, rt, 0, 0.02, 0.1, std_of, design["plain"], design.get("std_of_bf16_check"))
                 rec["check"] = {"fp32_max_rel_err": float(f"{errs['float32']:.3g}"), "bf16_max_rel_err": float(f"{errs['bfloat16']:.3g}"),
                                 "slice_layers": 3, "cuts": "whole, portions, token by token, mixed"}
                 if errs.get("close_calls"):
@@ -719,7 +749,7 @@ def main():
                     help="instead of the default workload: prefill and decode of this design beside its closest relative "
                          "(Dafotar beside Gemma 2, Pubunex and Bumolix beside Dafotar, Rotalorn and Bizepel beside Pubunex) at equal layer sizes")
     ap.add_argument("--design-sizes", default="w1024,w2048,w4096", help="with --design: which of " + ", ".join(DESIGN_SIZES))
-    ap.add_argument("--only-model", choices=["bizepel", "bumolix", "dafotar", "gemma2", "pubunex", "rotalorn"], default=None, help="with --design, a profiling aid: one of the two")
+    ap.add_argument("--only-model", choices=["bizepel", "bumolix", "buvuzen", "dafotar", "gemma2", "pubunex", "rotalorn"], default=None, help="with --design, a profiling aid: one of the two")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=64)
     ap.add_argument("--warmup", type=int, default=8)

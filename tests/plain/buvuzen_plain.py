@@ -121,7 +121,7 @@ def choose(choice, top, groups):
     return order[:top], gap
 
 
-def mixture(ml, w, pre, x, dt, margins=None):
+def mixture(ml, w, pre, x, dt, close=None):
     """sum over the chosen of weight * expert(x), the last ``identity`` of the router's outputs being
     experts that give x back; plus the shared expert times sigmoid(W_sg x), one number a token."""
     r = ml["router"]
@@ -129,32 +129,33 @@ def mixture(ml, w, pre, x, dt, margins=None):
     s = router_scores(x, w[pre + "router"], dt)
     choice = s + w[pre + "correction"].astype(dt)
     out = np.zeros_like(x, dtype=dt)
-    gaps = []
     for t in range(x.shape[0]):
         ids, gap = choose(choice[t], r["top"], (gr["count"], gr["keep"]) if gr else None)
-        gaps.append(gap)
+        if close is not None:
+            close[t] = min(close[t], gap)
         for e in ids:
             y = x[t] if e >= r["experts"] else gated(x[t:t + 1], w, f"{pre}e{e}.", dt)[0]
             out[t] += s[t, e] * dt(r.get("scale", 1.0)) * y
-    if margins is not None:
-        margins.append(np.array(gaps))
     if ml.get("shared"):
         out += gated(x, w, pre + "shared.", dt) * sigmoid(x @ w[pre + "shared.sg"].astype(dt).T)
     return out
 
 
 # ---------------------------------------------------------------- the model
-def forward(cfg, w, tokens, dt=np.float64, layers_out=None, margins=None):
+def forward(cfg, w, tokens, dt=np.float64, layers_out=None, close=None):
     """Logits [T, vocab] of one sequence.  ``layers_out``: a list that receives the stream after
-    every layer; ``margins``: a list that receives each routed layer's per-token margins."""
+    every layer; ``close``: an array [T] that receives how close each token's nearest choice of
+    experts was, as a gap between choice scores."""
     eps = cfg["norm"]["eps"]
+    if close is not None:
+        close[:] = np.inf
     x = embed(cfg, w, tokens, dt)
     for i in range(len(cfg["layers"])):
         j = weights_layer(cfg, i)
         l, p = cfg["layers"][j], f"l{j}."
         x = x + model_norm(attention_mixer(l["mixer"], w, p + "mix.", x, eps, dt), w[p + "norm1"], eps, dt)
         if l.get("mlp"):
-            x = x + model_norm(mixture(l["mlp"], w, p + "mlp.", x, dt, margins), w[p + "norm2"], eps, dt)
+            x = x + model_norm(mixture(l["mlp"], w, p + "mlp.", x, dt, close), w[p + "norm2"], eps, dt)
         if layers_out is not None:
             layers_out.append(x.copy())
     x = model_norm(x, w["final.norm"], eps, dt)
