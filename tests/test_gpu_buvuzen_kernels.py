@@ -173,7 +173,8 @@ def test_groups_judged_by_their_best(n, top, groups, keep):
 
 
 @pytest.mark.parametrize("T,E,I,top,W,F", [(3, 5, 2, 2, 48, 24), (40, 4, 3, 3, 36, 20), (1, 2, 1, 2, 64, 96), (90, 12, 4, 4, 64, 32),
-                                           (70, 1, 3, 2, 40, 16), (200, 3, 0, 2, 128, 64)])
+                                           (70, 1, 3, 2, 40, 16), (200, 3, 0, 2, 128, 64), (300, 2, 1, 2, 72, 136), (33, 70, 3, 4, 136, 72),
+                                           (150, 3, 1, 3, 1032, 200)])
 @pytest.mark.parametrize("all_identity", [False, True])
 def test_identity_experts_among_the_choices(T, E, I, top, W, F, all_identity):
     """Row by row in 32-bit; row by row and grouped on the matrix cores in bfloat16.  The scratch memory
@@ -194,25 +195,30 @@ def test_identity_experts_among_the_choices(T, E, I, top, W, F, all_identity):
         for e, s in zip(ids[t], wts[t]):
             want[t] += s * (xd[t] if e >= E else (P.silu(xd[t] @ wg[e].T) * (xd[t] @ wu[e].T)) @ wd[e].T)
     gu = np.concatenate([wg, wu], axis=1)
+    # a shared layer's rows on top: none, as they are, or times the sigmoid of the fourth of five numbers a row
+    add, z = rng.normal(size=(T, W)).astype(np.float32), rng.normal(0, 2, (T, 5)).astype(np.float32)
+    how = (T + E + all_identity) % 3
+    want = want + (0.0 if how == 0 else add if how == 1 else add * P.sigmoid(z[:, 3:4].astype(np.float64)))
+    more = lambda rt: (None if how == 0 else up(rt, add).ptr, up(rt, z).ptr + 12 if how == 2 else None, 5)
     scale = np.abs(want).max()
     nan = lambda shape, dtype: up(rt, np.full(shape, np.nan), dtype)
     out = new(rt, (T, W))
     k.zk_moe_experts_identity(up(rt, x).ptr, i32(rt, ids).ptr, up(rt, wts).ptr, up(rt, gu).ptr, up(rt, wd).ptr, nan((T * top, F), "float32").ptr,
-                              out.ptr, T, top, W, F, 0.0, 1, 1, E, rt.stream)
+                              out.ptr, T, top, W, F, 0.0, 1, 1, E, *more(rt), rt.stream)
     assert np.abs(rt.download(out) - want).max() < 1e-5 * scale
     rt, kb = lib("bfloat16")
     h16 = lambda a: up(rt, a, "bfloat16").ptr
     out = new(rt, (T, W))
     kb.zk_moe_experts_identity(h16(x), i32(rt, ids).ptr, up(rt, wts).ptr, h16(gu), h16(wd), nan((T * top, F), "bfloat16").ptr, out.ptr, T, top, W,
-                               F, 0.0, 1, 1, E, rt.stream)
+                               F, 0.0, 1, 1, E, *more(rt), rt.stream)
     assert np.abs(rt.download(out) - want).max() < 0.02 * scale
     if W % 8 or F % 8:
         return
     work = i32(rt, np.zeros(E + I + 1 + 2 * T * top))
     out = new(rt, (T, W))
-    kb.zk_moe_experts_grouped_identity(h16(x), i32(rt, ids).ptr, up(rt, wts).ptr, h16(gu), h16(wd), work.ptr, nan((T * top, W), "bfloat16").ptr,
+    kb.zk_moe_experts_grouped_identity(h16(x), i32(rt, ids).ptr, up(rt, wts).ptr, h16(gu), h16(wd), work.ptr, None,
                                        nan((T * top, F), "bfloat16").ptr, nan((T * top, W), "float32").ptr, out.ptr, T, E, top, W, F, 0.0, 1, 1,
-                                       I, rt.stream)
+                                       I, *more(rt), rt.stream)
     assert np.abs(rt.download(out) - want).max() < 0.02 * scale
 
 

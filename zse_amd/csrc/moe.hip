@@ -8,17 +8,17 @@
 // Variants, as parameters of the ``_ext`` entry points: scores softmax(router logits) over all experts
 // instead of sigmoids; the weight on the expert's output instead of its input (out_t = sum s_e Wd y);
 // y = silu(g) u instead of the clamped form; experts without a gate, y = max(Wu x', 0)^2, whose
-// weights are [E][F][W].  ``zk_gate_rows`` multiplies float rows by the sigmoid
-// of a number a row (a shared layer's gate).  ``zk_moe_route_groups`` chooses by s + a correction per
+// weights are [E][F][W].  A shared layer's rows may be added to the experts' sum, times the sigmoid of
+// a number a row.  ``zk_moe_route_groups`` chooses by s + a correction per
 // expert, among the experts of the best groups only, and may bring the weights to a sum.
 // Identity experts are numbers from E on that the router may choose: such an expert has no weights and gives
 // its input back, so it adds s x_t.
 //
 // Two ways through the experts.  Few tokens (decoding): one block per (token, choice) multiplies
 // the expert's rows by the token's row, and the weights stream once per choice.  Many tokens
-// (bfloat16 only): the (token, choice) pairs are sorted by expert on the device, the scaled rows
-// are gathered in that order, and a grouped matrix-core product runs over tiles of one expert's
-// rows each; nothing comes back to the host, so a step can be written down and repeated.  Either
+// (bfloat16 only): the (token, choice) pairs are sorted by expert on the device, and a grouped
+// matrix-core product runs over tiles of one expert's rows each, which it reads from where they are (or,
+// where the weights multiply the inputs, from scaled rows gathered in that order); nothing comes back to the host, so a step can be written down and repeated.  Either
 // way a row's sums run in an order fixed by the channel numbers, and a token's result does not
 // depend on what else is in the step.
 #include "common.h"
@@ -274,18 +274,30 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(const act_t* __restric
   }
 }
 
-// out[t, n] = sum_k Wd[e_k][n] . y[(t, k)], an identity expert's term s_k x[t, n]
+// What a shared layer adds to a row's sum: ``add`` [T, W] (may be null), times the sigmoid of the row's number in
+// ``gate`` (may be null).
+struct SharedRows {
+  const float* add;
+  const float* gate;
+  int gate_ld;
+  __device__ __forceinline__ float factor(int t) const {
+    return (add && gate) ? 1.0f / (1.0f + expf(-gate[(size_t)t * gate_ld])) : 1.0f;
+  }
+};
+
+// out[t, n] = sum_k Wd[e_k][n] . y[(t, k)], an identity expert's term s_k x[t, n], plus the shared layer's row
 __global__ __launch_bounds__(256) void moe_down_kernel(const act_t* __restrict__ y, const int* __restrict__ ids,
                                                        const act_t* __restrict__ w_down, float* __restrict__ out,
                                                        int top, int W, int F, int rows_per_block,
                                                        const float* __restrict__ wts, int on_out,
-                                                       const act_t* __restrict__ x, int experts) {
+                                                       const act_t* __restrict__ x, int experts, SharedRows shared) {
   extern __shared__ float ys[];                   // [top][F]
   const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   for (int i = tid; i < top * F; i += 256)
     ys[i] = ids[(size_t)t * top + i / F] < experts ? to_f32(y[(size_t)t * top * F + i]) : 0.f;
   __syncthreads();
   const int n0 = blockIdx.y * rows_per_block;
+  const float sg = shared.factor(t);
   for (int n = n0 + wave; n < min(W, n0 + rows_per_block); n += 4) {
     float total = 0.f;
     for (int k = 0; k < top; k++) {
@@ -299,7 +311,7 @@ __global__ __launch_bounds__(256) void moe_down_kernel(const act_t* __restrict__
       const float d = row_dot(wr, ys + k * F, F, lane);
       total += on_out ? s * d : d;
     }
-    if (lane == 0) out[(size_t)t * W + n] = total;
+    if (lane == 0) out[(size_t)t * W + n] = shared.add ? total + sg * shared.add[(size_t)t * W + n] : total;
   }
 }
 
@@ -312,12 +324,13 @@ __global__ void clamped_glu_kernel(const act_t* __restrict__ gu, act_t* __restri
   y[(size_t)t * F + n] = from_f32<act_t>(clamped_swiglu(to_f32(row[n]), to_f32(row[F + n]), limit));
 }
 
-// ---- many tokens: sort the pairs by expert, gather the scaled rows
-// One block.  order[i] = the pair at sorted place i; first[e] = the first place of expert e
-// (first[E] = pairs).  Which place among its expert's a pair gets is left to chance: a row's
+// ---- many tokens: sort the pairs by expert
+// One block.  order[i] = the pair at sorted place i, place[] the reverse; first[e] = the first place of
+// expert e (first[E] = pairs).  Which place among its expert's a pair gets is left to chance: a row's
 // result does not depend on its place.
 __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* __restrict__ ids, int pairs, int E,
-                                                        int* __restrict__ first, int* __restrict__ order) {
+                                                        int* __restrict__ first, int* __restrict__ order,
+                                                       int* __restrict__ place) {
   __shared__ int count[MOE_MAX_EXPERTS + 1];
   __shared__ int cursor[MOE_MAX_EXPERTS];
   const int tid = threadIdx.x;
@@ -332,139 +345,225 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* __restrict__ 
   for (int e = tid; e <= E; e += 1024) first[e] = count[e];
   for (int e = tid; e < E; e += 1024) cursor[e] = count[e];
   __syncthreads();
-  for (int i = tid; i < pairs; i += 1024) order[atomicAdd(&cursor[ids[i]], 1)] = i;
+  for (int i = tid; i < pairs; i += 1024) {
+    const int at = atomicAdd(&cursor[ids[i]], 1);
+    order[at] = i;
+    place[i] = at;
+  }
 }
 
+// the rows times their weights, in sorted order (weights that multiply the inputs)
 __global__ void moe_gather_kernel(const act_t* __restrict__ x, const int* __restrict__ order,
                                   const float* __restrict__ wts, act_t* __restrict__ xg, int top, int W,
                                   const int* __restrict__ ids, int experts) {
   const int i = blockIdx.x;
   const int pair = order[i];
   if (ids[pair] >= experts) return;                       // sorted behind every expert's rows, never multiplied
-  const float s = wts ? wts[pair] : 1.0f;
+  const float s = wts[pair];
   const act_t* xr = x + (size_t)(pair / top) * W;
   for (int c = threadIdx.x; c < W; c += blockDim.x) xg[(size_t)i * W + c] = from_f32<act_t>(s * to_f32(xr[c]));
 }
 
 #if ZSE_ACT_BF16
 // Grouped product on the matrix cores: C[i, n] = sum_k A[i, k] B[e(i)][n, k] over rows sorted by
-// expert.  A block takes 64 rows of one expert and 64 columns; which expert and which rows it
-// finds by walking first[] (tiles never span two experts; a tile past the last one ends at once).
-// Four waves, each a 32 x 32 corner, 32 x 32 x 16 products, operands through local memory.
+// expert.  A block takes TM rows of one expert and 64 columns (or NB times 64); which expert and which
+// rows it finds in first[] (tiles never span two experts; a tile past the last one ends at once).
+// Four waves, each TM / 2 rows by 32 of every 64 columns, 32 x 32 x 16 products.  Operands pass through
+// local memory in steps of TK channels, two buffers; DEPTH steps are on their way in registers while one is
+// multiplied, their loads without conditions (rows and columns past the end read the last one and are not
+// stored, channels past the end are replaced by zeros).
+//
+// order (may be null): the sorted row i is row order[i] / top of A; without it A is sorted itself.
+// mode 0: C = act(gate, up) with B = [E][2F][K], stores y[i, n] (n < F), the 64 columns' gate rows and up
+// rows in the two halves of a B tile; mode 1: plain product with B = [E][N][K], stores float
+// rows; mode 2: the square of relu of that product, stores y.
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float floatx16 __attribute__((ext_vector_type(16)));
 
-#define GG_TM 64
-#define GG_TN 64
-#define GG_TK 32
-#define GG_PAD 8
-
-// mode 0: C = act(gate, up) with B = [E][2F][K], stores y[i, n] (n < F); mode 1: plain product
-// with B = [E][N][K], stores float rows at out[order..] (see the launch); mode 2: the square of
-// relu of that product, stores y.
-template <int MODE>
-__global__ __launch_bounds__(256) void moe_grouped_kernel(const __bf16* __restrict__ A, const __bf16* __restrict__ B,
-                                                          const int* __restrict__ first, int E, int N, int K,
-                                                          __bf16* __restrict__ y, float* __restrict__ out_rows,
+template <int MODE, int TM, int NB, int TK, int DEPTH>
+__global__ __launch_bounds__(256) void moe_grouped_kernel(const __bf16* __restrict__ A, const int* __restrict__ order, int top,
+                                                          const __bf16* __restrict__ B, const int* __restrict__ first, int E,
+                                                          int N, int K, __bf16* __restrict__ y, float* __restrict__ out_rows,
                                                           float limit, int act) {
-  __shared__ __bf16 As[GG_TM][GG_TK + GG_PAD];
-  __shared__ __bf16 Bs[(MODE == 0 ? 2 : 1) * GG_TN][GG_TK + GG_PAD];
+  static_assert(MODE != 0 || NB == 2, "a gate tile and an up tile");
+  constexpr int LD = TK + 8, CPR = TK / 8, TN = NB * 64, MI = TM / 64;
+  constexpr int APT = TM * CPR / 256, BPT = TN * CPR / 256;          // 16-byte pieces a thread moves
+  constexpr int COLS = MODE == 0 ? 64 : TN;                          // columns of the result a block makes
+  extern __shared__ __attribute__((aligned(16))) unsigned char grouped_raw[];
+  __bf16* As = (__bf16*)grouped_raw;             // [2][TM][LD]
+  __bf16* Bs = As + 2 * TM * LD;                 // [2][TN][LD]
   __shared__ int tile_e, tile_row, tile_end;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  if (tid == 0) {
-    // the blockIdx.x-th tile of rows, counting each expert's rows in whole tiles
-    int left = blockIdx.x, e = 0, row = -1, end = 0;
-    for (; e < E; e++) {
-      const int lo = first[e], hi = first[e + 1];
-      const int tiles = (hi - lo + GG_TM - 1) / GG_TM;
-      if (left < tiles) {
-        row = lo + left * GG_TM;
-        end = hi;
-        break;
+  if (wave == 0) {
+    // the blockIdx.x-th tile of rows, counting each expert's rows in whole tiles, 64 experts a turn
+    int left = blockIdx.x;
+    bool found = false;
+    for (int e0 = 0; e0 < E && !found; e0 += 64) {
+      const int e = e0 + lane;
+      const int lo = first[min(e, E)], hi = first[min(e + 1, E)];
+      const int tiles = (hi - lo + TM - 1) / TM;
+      int sum = tiles;
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const int other = __shfl_up(sum, o, 64);
+        if (lane >= o) sum += other;
       }
-      left -= tiles;
+      const bool mine = left < sum && left >= sum - tiles;
+      if (mine) {
+        tile_e = e;
+        tile_row = lo + (left - (sum - tiles)) * TM;
+        tile_end = hi;
+      }
+      found = __any(mine);
+      left -= __shfl(sum, 63, 64);
     }
-    tile_e = e;
-    tile_row = row;
-    tile_end = end;
+    if (!found && lane == 0) tile_row = -1;
   }
   __syncthreads();
   if (tile_row < 0) return;
-  const int e = tile_e, row0 = tile_row, rows = min(GG_TM, tile_end - tile_row);
-  const int n0 = blockIdx.y * GG_TN;
-  const int wm = (wave & 1) * 32, wn = (wave >> 1) * 32;
-  floatx16 acc0 = {0}, acc1 = {0};
+  const int e = tile_e, row0 = tile_row, rows = min(TM, tile_end - tile_row);
+  const int n0 = blockIdx.y * COLS;
+  const int wm = (wave & 1) * (TM / 2), wn = (wave >> 1) * 32;
   const __bf16* Be = B + (size_t)e * (MODE == 0 ? 2 : 1) * N * K;
-  const int lr = tid >> 2, lc = (tid & 3) * 8;         // 64 rows x 4 pieces of 8
-  for (int k0 = 0; k0 < K; k0 += GG_TK) {
-    bf16x8 a = {0}, b = {0}, b2 = {0};
-    const bool kin = k0 + lc < K;                        // K is a multiple of 8
-    if (lr < rows && kin) a = *(const bf16x8*)(A + (size_t)(row0 + lr) * K + k0 + lc);
-    if (n0 + lr < N && kin) {
-      b = *(const bf16x8*)(Be + (size_t)(n0 + lr) * K + k0 + lc);
-      if (MODE == 0) b2 = *(const bf16x8*)(Be + (size_t)(N + n0 + lr) * K + k0 + lc);
-    }
-    __syncthreads();
-    *(bf16x8*)&As[lr][lc] = a;
-    *(bf16x8*)&Bs[lr][lc] = b;
-    if (MODE == 0) *(bf16x8*)&Bs[GG_TN + lr][lc] = b2;
-    __syncthreads();
+  // the thread's pieces: their rows' beginnings, their place in a step of TK channels and in local memory
+  const __bf16* arow[APT];
+  const __bf16* brow[BPT];
 #pragma unroll
-    for (int kk = 0; kk < GG_TK; kk += 16) {
-      const bf16x8 av = *(const bf16x8*)&As[wm + (lane & 31)][kk + (lane >> 5) * 8];
-      const bf16x8 bv = *(const bf16x8*)&Bs[wn + (lane & 31)][kk + (lane >> 5) * 8];
-      acc0 = __builtin_amdgcn_mfma_f32_32x32x16_bf16(av, bv, acc0, 0, 0, 0);
+  for (int j = 0; j < APT; j++) {
+    const int i = row0 + min((tid + 256 * j) / CPR, rows - 1);
+    arow[j] = A + (size_t)(order ? order[i] / top : i) * K;
+  }
+#pragma unroll
+  for (int j = 0; j < BPT; j++) {
+    const int r = (tid + 256 * j) / CPR;
+    brow[j] = Be + (size_t)(MODE == 0 ? (r >> 6) * N + min(n0 + (r & 63), N - 1) : min(n0 + r, N - 1)) * K;
+  }
+  const int lc = (tid % CPR) * 8;                // 256 is a multiple of CPR: the same for all of a thread's pieces
+  bf16x8 ra[DEPTH][APT], rb[DEPTH][BPT];
+  auto load = [&](int k0, bf16x8 (&a)[APT], bf16x8 (&b)[BPT]) {
+    const int k = min(k0 + lc, K - 8);           // K is a multiple of 8
+#pragma unroll
+    for (int j = 0; j < APT; j++) a[j] = *(const bf16x8*)(arow[j] + k);
+#pragma unroll
+    for (int j = 0; j < BPT; j++) b[j] = *(const bf16x8*)(brow[j] + k);
+  };
+  floatx16 acc[MI][NB];
+#pragma unroll
+  for (int mi = 0; mi < MI; mi++)
+#pragma unroll
+    for (int nb = 0; nb < NB; nb++) acc[mi][nb] = floatx16{0};
+#pragma unroll
+  for (int d = 0; d < DEPTH; d++) load(d * TK, ra[d], rb[d]);
+  int buf = 0;
+  for (int k0 = 0; k0 < K; k0 += DEPTH * TK) {
+#pragma unroll
+    for (int d = 0; d < DEPTH; d++) {
+      const int kd = k0 + d * TK;
+      const bool in = kd + lc < K;
+      __bf16* as = As + buf * TM * LD;
+      __bf16* bs = Bs + buf * TN * LD;
+#pragma unroll
+      for (int j = 0; j < APT; j++) *(bf16x8*)(as + ((tid + 256 * j) / CPR) * LD + lc) = in ? ra[d][j] : bf16x8{0};
+#pragma unroll
+      for (int j = 0; j < BPT; j++) *(bf16x8*)(bs + ((tid + 256 * j) / CPR) * LD + lc) = in ? rb[d][j] : bf16x8{0};
+      load(kd + DEPTH * TK, ra[d], rb[d]);
+      __syncthreads();
+      // (a wave whose rows are all past the tile's end has nothing to multiply)
+      if (wm < rows) {
+#pragma unroll
+        for (int kk = 0; kk < TK; kk += 16) {
+          bf16x8 av[MI];
+#pragma unroll
+          for (int mi = 0; mi < MI; mi++)
+            av[mi] = *(const bf16x8*)(as + (wm + mi * 32 + (lane & 31)) * LD + kk + (lane >> 5) * 8);
+#pragma unroll
+          for (int nb = 0; nb < NB; nb++) {
+            const bf16x8 bv = *(const bf16x8*)(bs + (nb * 64 + wn + (lane & 31)) * LD + kk + (lane >> 5) * 8);
+#pragma unroll
+            for (int mi = 0; mi < MI; mi++) acc[mi][nb] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(av[mi], bv, acc[mi][nb], 0, 0, 0);
+          }
+        }
+      }
+      buf ^= 1;
+    }
+  }
+  // element i of an accumulator: row (i / 4) * 8 + (lane / 32) * 4 + i % 4, column lane % 32
+#pragma unroll
+  for (int mi = 0; mi < MI; mi++)
+#pragma unroll
+    for (int i = 0; i < 16; i++) {
+      const int r = wm + mi * 32 + (i / 4) * 8 + (lane >> 5) * 4 + (i % 4);
+      if (r >= rows) continue;
       if (MODE == 0) {
-        const bf16x8 bu = *(const bf16x8*)&Bs[GG_TN + wn + (lane & 31)][kk + (lane >> 5) * 8];
-        acc1 = __builtin_amdgcn_mfma_f32_32x32x16_bf16(av, bu, acc1, 0, 0, 0);
-      }
-    }
-  }
-  // element i of the accumulator: row (i / 4) * 8 + (lane / 32) * 4 + i % 4, column lane % 32
-  const int col = n0 + wn + (lane & 31);
+        const int col = n0 + wn + (lane & 31);
+        if (col < N) y[(size_t)(row0 + r) * N + col] = (__bf16)expert_act(acc[mi][0][i], acc[mi][NB - 1][i], limit, act);
+      } else {
 #pragma unroll
-  for (int i = 0; i < 16; i++) {
-    const int r = wm + (i / 4) * 8 + (lane >> 5) * 4 + (i % 4);
-    if (r < rows && col < N) {
-      if (MODE == 0) y[(size_t)(row0 + r) * N + col] = (__bf16)expert_act(acc0[i], acc1[i], limit, act);
-      else if (MODE == 2) y[(size_t)(row0 + r) * N + col] = (__bf16)square_of_relu(acc0[i]);
-      else out_rows[(size_t)(row0 + r) * N + col] = acc0[i];
-    }
-  }
-}
-
-// out[t, :] = sum over t's choices, in their order, of the sorted rows' results (of s x[t, :] for an identity expert)
-__global__ void moe_combine_kernel(const float* __restrict__ rows, const int* __restrict__ place, float* __restrict__ out,
-                                   int top, int W, const float* __restrict__ wts, int on_out,
-                                   const int* __restrict__ ids, const act_t* __restrict__ x, int experts) {
-  const int t = blockIdx.x;
-  for (int c = threadIdx.x; c < W; c += blockDim.x) {
-    float total = 0.f;
-    for (int k = 0; k < top; k++) {
-      const float s = wts[(size_t)t * top + k];
-      if (ids[(size_t)t * top + k] >= experts) {
-        total += s * to_f32(x[(size_t)t * W + c]);
-        continue;
+        for (int nb = 0; nb < NB; nb++) {
+          const int col = n0 + nb * 64 + wn + (lane & 31);
+          if (col >= N) continue;
+          if (MODE == 2) y[(size_t)(row0 + r) * N + col] = (__bf16)square_of_relu(acc[mi][nb][i]);
+          else out_rows[(size_t)(row0 + r) * N + col] = acc[mi][nb][i];
+        }
       }
-      const float v = rows[(size_t)place[(size_t)t * top + k] * W + c];
-      total += on_out ? s * v : v;
     }
-    out[(size_t)t * W + c] = total;
-  }
 }
 
-__global__ void moe_place_kernel(const int* __restrict__ order, int* __restrict__ place, int pairs) {
-  const int i = blockIdx.x * blockDim.x + threadIdx.x;
-  if (i < pairs) place[order[i]] = i;
+template <int MODE, int TM, int NB, int TK, int DEPTH>
+static int launch_grouped(const void* A, const int* order, int top, const void* B, const int* first, int pairs, int E, int N, int K,
+                          void* y, float* out_rows, float limit, int act, hipStream_t st) {
+  constexpr size_t lds = (size_t)2 * (TM + NB * 64) * (TK + 8) * sizeof(__bf16);
+  static bool raised = false;
+  if (!raised) {
+    if (lds > 64 * 1024 && hipFuncSetAttribute((const void*)moe_grouped_kernel<MODE, TM, NB, TK, DEPTH>,
+                                               hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
+      return zk_fail("zk_moe_experts_grouped: the local memory was refused");
+    raised = true;
+  }
+  constexpr int cols = MODE == 0 ? 64 : NB * 64;
+  const dim3 grid((pairs + TM - 1) / TM + E, (N + cols - 1) / cols);       // each expert may end in a tile that is not full
+  moe_grouped_kernel<MODE, TM, NB, TK, DEPTH><<<grid, 256, lds, st>>>((const __bf16*)A, order, top, (const __bf16*)B, first, E, N, K,
+                                                                      (__bf16*)y, out_rows, limit, act);
+  return zk_launch_status("zk_moe_experts_grouped");
+}
+
+// out[t, :] = sum over t's choices, in their order, of the sorted rows' results (of s x[t, :] for an identity expert),
+// plus the shared layer's row.  A thread takes four columns (W is a multiple of 8).
+__global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restrict__ rows, const int* __restrict__ place,
+                                                          float* __restrict__ out, int top, int W, const float* __restrict__ wts,
+                                                          int on_out, const int* __restrict__ ids, const __bf16* __restrict__ x,
+                                                          int experts, SharedRows shared) {
+  typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
+  const int t = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * 4;
+  if (c >= W) return;
+  float4 sum = make_float4(0.f, 0.f, 0.f, 0.f), add = sum;
+  if (shared.add) add = *(const float4*)(shared.add + (size_t)t * W + c);
+  for (int k = 0; k < top; k++) {
+    const size_t pair = (size_t)t * top + k;
+    const bool identity = ids[pair] >= experts;
+    const float s = (identity || on_out) ? wts[pair] : 1.f;
+    float4 v;
+    if (identity) {
+      const bf16x4 xv = *(const bf16x4*)(x + (size_t)t * W + c);
+      v = make_float4((float)xv[0], (float)xv[1], (float)xv[2], (float)xv[3]);
+    } else {
+      v = *(const float4*)(rows + (size_t)place[pair] * W + c);
+    }
+    sum.x += s * v.x;
+    sum.y += s * v.y;
+    sum.z += s * v.z;
+    sum.w += s * v.w;
+  }
+  if (shared.add) {
+    const float g = shared.factor(t);
+    sum.x += g * add.x;
+    sum.y += g * add.y;
+    sum.z += g * add.z;
+    sum.w += g * add.w;
+  }
+  *(float4*)(out + (size_t)t * W + c) = sum;
 }
 #endif
-
-// rows[t, :] *= sigmoid(z[t * ld])
-__global__ void gate_rows_kernel(float* __restrict__ rows, const float* __restrict__ z, int ld, int W) {
-  const int t = blockIdx.x;
-  const float g = 1.0f / (1.0f + expf(-z[(size_t)t * ld]));
-  for (int c = threadIdx.x; c < W; c += blockDim.x) rows[(size_t)t * W + c] *= g;
-}
 
 extern "C" {
 
@@ -507,22 +606,15 @@ int zk_moe_route_groups(const float* logits, int ld, const float* correction, vo
   return zk_moe_route_best(logits, ld, correction, ids, wts, T, E, top, groups, keep, softmax, normalise, scale, 2, stream);
 }
 
-// rows: float [T, W], each multiplied by sigmoid(z[t * ld]).
-int zk_gate_rows(float* rows, const float* z, int ld, int T, int W, void* stream) {
-  ZK_REQUIRE(T >= 0 && W > 0 && ld > 0 && rows != nullptr && z != nullptr, "zk_gate_rows: bad arguments");
-  if (T == 0) return 0;
-  gate_rows_kernel<<<T, 256, 0, (hipStream_t)stream>>>(rows, z, ld, W);
-  return zk_launch_status("zk_gate_rows");
-}
-
 // x: [T, W]; w_gu: [E][2F][W], an expert's gate rows, then its up rows; w_down: [E][W][F].
 // y: scratch [T * top, F] activations; out: float [T, W].
 // act: 0 the clamped form, 1 silu(gate) up, 2 the square of relu(up) without a gate (w_gu is then
 // [E][F][W]).  on_out: the weight multiplies the expert's output.  experts: numbers below it have weights,
-// numbers from it on are identity experts.
+// numbers from it on are identity experts.  add (may be null): float [T, W], added to every row's sum, times
+// sigmoid(gate[t * gate_ld]) where a gate is given.
 int zk_moe_experts_identity(const void* x, const int* ids, const float* wts, const void* w_gu, const void* w_down, void* y,
                             float* out, int T, int top, int W, int F, float limit, int act, int on_out, int experts,
-                            void* stream) {
+                            const float* add, const float* gate, int gate_ld, void* stream) {
   ZK_REQUIRE(experts > 0, "zk_moe_experts: no experts");
   ZK_REQUIRE(T >= 0 && top > 0 && top <= MOE_MAX_TOP && W > 0 && F > 0, "zk_moe_experts: bad sizes");
   ZK_REQUIRE(T <= 65535 && (size_t)T * top <= 0x7fffffff, "zk_moe_experts: more than 65535 rows");
@@ -540,13 +632,15 @@ int zk_moe_experts_identity(const void* x, const int* ids, const float* wts, con
                                                                           (act_t*)y, top, W, F, limit, rpb, act, on_out, experts);
   dim3 grid(T, (W + rpb - 1) / rpb);
   moe_down_kernel<<<grid, 256, (size_t)top * F * 4, (hipStream_t)stream>>>((const act_t*)y, ids, (const act_t*)w_down, out, top,
-                                                                         W, F, rpb, wts, on_out, (const act_t*)x, experts);
+                                                                         W, F, rpb, wts, on_out, (const act_t*)x, experts,
+                                                                         SharedRows{add, gate, gate_ld});
   return zk_launch_status("zk_moe_experts");
 }
 
 int zk_moe_experts_ext(const void* x, const int* ids, const float* wts, const void* w_gu, const void* w_down, void* y,
                        float* out, int T, int top, int W, int F, float limit, int act, int on_out, void* stream) {
-  return zk_moe_experts_identity(x, ids, wts, w_gu, w_down, y, out, T, top, W, F, limit, act, on_out, 0x7fffffff, stream);
+  return zk_moe_experts_identity(x, ids, wts, w_gu, w_down, y, out, T, top, W, F, limit, act, on_out, 0x7fffffff, nullptr,
+                                 nullptr, 0, stream);
 }
 
 int zk_moe_experts(const void* x, const int* ids, const float* wts, const void* w_gu, const void* w_down, void* y,
@@ -565,15 +659,18 @@ int zk_clamped_glu(const void* gu, void* y, int T, int F, float limit, void* str
 
 #if ZSE_ACT_BF16
 // The same through the grouped matrix-core product, with ``identity`` numbers behind the E experts'.  work: int32
-// [E + identity + 1 + 2 * T * top] (first, order, place); xg: [T * top, W] and y: [T * top, F] bfloat16; rows: float
-// [T * top, W].
+// [E + identity + 1 + 2 * T * top] (first, order, place); xg: [T * top, W] (used only where the weights multiply the
+// inputs, may be null otherwise) and y: [T * top, F] bfloat16; rows: float [T * top, W].
 int zk_moe_experts_grouped_identity(const void* x, const int* ids, const float* wts, const void* w_gu, const void* w_down,
                                     void* work, void* xg, void* y, float* rows, float* out, int T, int E, int top, int W,
-                                    int F, float limit, int act, int on_out, int identity, void* stream) {
+                                    int F, float limit, int act, int on_out, int identity, const float* add,
+                                    const float* gate, int gate_ld, void* stream) {
   ZK_REQUIRE(T >= 0 && top > 0 && top <= MOE_MAX_TOP && W > 0 && F > 0 && E > 0 && identity >= 0 &&
                  E + identity <= MOE_MAX_EXPERTS,
              "zk_moe_experts_grouped: bad sizes");
   ZK_REQUIRE(W % 8 == 0 && F % 8 == 0, "zk_moe_experts_grouped: widths in whole groups of eight");
+  ZK_REQUIRE(((uintptr_t)x | (uintptr_t)y | (uintptr_t)xg | (uintptr_t)w_gu | (uintptr_t)w_down | (uintptr_t)rows | (uintptr_t)out |
+              (uintptr_t)add) % 16 == 0, "zk_moe_experts_grouped: operands must be 16-byte aligned");
   ZK_REQUIRE(T <= 65535, "zk_moe_experts_grouped: more than 65535 rows");
   if (T == 0) return 0;
   const int pairs = T * top;
@@ -581,18 +678,28 @@ int zk_moe_experts_grouped_identity(const void* x, const int* ids, const float* 
   int* order = first + E + identity + 1;
   int* place = order + pairs;
   hipStream_t st = (hipStream_t)stream;
-  moe_sort_kernel<<<1, 1024, 0, st>>>(ids, pairs, E + identity, first, order);
-  moe_place_kernel<<<(pairs + 255) / 256, 256, 0, st>>>(order, place, pairs);
-  moe_gather_kernel<<<pairs, 256, 0, st>>>((const act_t*)x, order, on_out ? nullptr : wts, (act_t*)xg, top, W, ids, E);
-  const int tiles = (pairs + GG_TM - 1) / GG_TM + E;        // each expert may end in a tile that is not full
-  dim3 g0(tiles, (F + GG_TN - 1) / GG_TN);
-  if (act == MOE_NO_GATE)
-    moe_grouped_kernel<2><<<g0, 256, 0, st>>>((const __bf16*)xg, (const __bf16*)w_gu, first, E, F, W, (__bf16*)y, nullptr, limit, act);
-  else
-    moe_grouped_kernel<0><<<g0, 256, 0, st>>>((const __bf16*)xg, (const __bf16*)w_gu, first, E, F, W, (__bf16*)y, nullptr, limit, act);
-  dim3 g1(tiles, (W + GG_TN - 1) / GG_TN);
-  moe_grouped_kernel<1><<<g1, 256, 0, st>>>((const __bf16*)y, (const __bf16*)w_down, first, E, W, F, nullptr, rows, 0.f, 0);
-  moe_combine_kernel<<<T, 256, 0, st>>>(rows, place, out, top, W, wts, on_out, ids, (const act_t*)x, E);
+  moe_sort_kernel<<<1, 1024, 0, st>>>(ids, pairs, E + identity, first, order, place);
+  const void* in = x;
+  const int* map = order;
+  if (!on_out) {
+    ZK_REQUIRE(xg != nullptr, "zk_moe_experts_grouped: no room for the scaled rows");
+    moe_gather_kernel<<<pairs, 256, 0, st>>>((const act_t*)x, order, wts, (act_t*)xg, top, W, ids, E);
+    in = xg;
+    map = nullptr;
+  }
+  // few rows an expert: tiles of 64 rows, long steps, so that much of the weights is on its way at a time; many: 128 rows
+  const bool few = pairs <= 32 * E;
+  int rc;
+#define ZK_GROUPED(MODE, ...) (few ? launch_grouped<MODE, 64, MODE == 0 ? 2 : 1, 128, 2>(__VA_ARGS__) \
+                                   : launch_grouped<MODE, 128, 2, 64, 1>(__VA_ARGS__))
+  if (act == MOE_NO_GATE) rc = ZK_GROUPED(2, in, map, top, w_gu, first, pairs, E, F, W, y, nullptr, limit, act, st);
+  else rc = ZK_GROUPED(0, in, map, top, w_gu, first, pairs, E, F, W, y, nullptr, limit, act, st);
+  if (rc) return rc;
+  rc = ZK_GROUPED(1, y, nullptr, top, w_down, first, pairs, E, W, F, nullptr, rows, 0.f, 0, st);
+#undef ZK_GROUPED
+  if (rc) return rc;
+  moe_combine_kernel<<<dim3(T, (W / 4 + 255) / 256), 256, 0, st>>>(rows, place, out, top, W, wts, on_out, ids, (const __bf16*)x, E,
+                                                                 SharedRows{add, gate, gate_ld});
   return zk_launch_status("zk_moe_experts_grouped");
 }
 
@@ -600,7 +707,7 @@ int zk_moe_experts_grouped_ext(const void* x, const int* ids, const float* wts, 
                                void* work, void* xg, void* y, float* rows, float* out, int T, int E, int top, int W, int F,
                                float limit, int act, int on_out, void* stream) {
   return zk_moe_experts_grouped_identity(x, ids, wts, w_gu, w_down, work, xg, y, rows, out, T, E, top, W, F, limit, act,
-                                         on_out, 0, stream);
+                                         on_out, 0, nullptr, nullptr, 0, stream);
 }
 
 int zk_moe_experts_grouped(const void* x, const int* ids, const float* wts, const void* w_gu, const void* w_down,
@@ -622,7 +729,6 @@ ZK_ENTER(zk_moe_route_groups)
 ZK_ENTER(zk_moe_route_best)
 ZK_ENTER(zk_moe_experts_identity)
 ZK_ENTER(zk_moe_experts_ext)
-ZK_ENTER(zk_gate_rows)
 ZK_ENTER(zk_moe_route)
 ZK_ENTER(zk_moe_experts)
 ZK_ENTER(zk_clamped_glu)

@@ -213,30 +213,31 @@ class RoutedMLP(Part):
         else:
             k.zk_moe_route_ext(logits.ptr, ld, ids.ptr, wts.ptr, T, n, top, softmax, ctx.stream)
         act, on_out, limit = (2 if not self.gated else 1 if s.activation == "silu" else 0), (0 if s.scale_input else 1), float(s.limit or 0.0)
-        P = 2 if self.shared is not None else 1
-        planes = ctx.alloc((P, T, W), F32)
+        # the shared layer's rows first: what adds up the chosen experts' results takes them in, with their gate
+        add = gate = None
+        if self.shared is not None:
+            add = self.shared.forward(ctx, x, out=ctx.alloc((T, W), F32)).ptr
+            gate = logits.ptr + n * 4 if self.shared_gate else None
+        plane = ctx.alloc((1, T, W), F32)
         y = ctx.alloc((T * top, F))
         enough = T * top >= (self.GROUPED_WIDE_FROM if W * F >= self.WIDE else self.GROUPED_FROM)
-        grouped = (ctx.dtype == BF16 and ctx.tuned and enough and W % 8 == 0 and F % 8 == 0
+        grouped = (ctx.dtype == BF16 and ctx.tuned and enough and W % 8 == 0 and F % 8 == 0 and x.ptr % 16 == 0
                    and k.has("zk_moe_experts_grouped_identity"))
         if grouped:
             work = ctx.alloc((n + 1 + 2 * T * top,), I32)
-            xg, rows = ctx.alloc((T * top, W)), ctx.alloc((T * top, W), F32)
-            k.zk_moe_experts_grouped_identity(x.ptr, ids.ptr, wts.ptr, self.w_gu.ptr, self.w_down.ptr, work.ptr, xg.ptr, y.ptr,
-                                              rows.ptr, planes.ptr, T, E, top, W, F, limit, act, on_out, self.identity, ctx.stream)
+            xg = ctx.alloc((T * top, W)).ptr if s.scale_input else None
+            rows = ctx.alloc((T * top, W), F32)
+            k.zk_moe_experts_grouped_identity(x.ptr, ids.ptr, wts.ptr, self.w_gu.ptr, self.w_down.ptr, work.ptr, xg, y.ptr,
+                                              rows.ptr, plane.ptr, T, E, top, W, F, limit, act, on_out, self.identity, add, gate, ld,
+                                              ctx.stream)
         else:
-            k.zk_moe_experts_identity(x.ptr, ids.ptr, wts.ptr, self.w_gu.ptr, self.w_down.ptr, y.ptr, planes.ptr, T, top, W, F,
-                                      limit, act, on_out, E, ctx.stream)
-        if self.shared is not None:
-            second = planes.rows(1, 2).view(T, W)
-            self.shared.forward(ctx, x, out=second)
-            if self.shared_gate:
-                k.zk_gate_rows(second.ptr, logits.ptr + n * 4, ld, T, W, ctx.stream)
+            k.zk_moe_experts_identity(x.ptr, ids.ptr, wts.ptr, self.w_gu.ptr, self.w_down.ptr, y.ptr, plane.ptr, T, top, W, F,
+                                      limit, act, on_out, E, add, gate, ld, ctx.stream)
         if getattr(ctx, "sums_welcome", None) is self:
-            # the block's joining kernel adds the planes up itself
-            return Tensor(planes.ptr, (P, T, W), F32, planes.owner, layout="parts")
+            # the block's joining kernel takes the float rows as they are
+            return Tensor(plane.ptr, (1, T, W), F32, plane.owner, layout="parts")
         out = ctx.alloc((T, W))
-        k.zk_planes_sum(planes.ptr, P, out.ptr, T, W, ctx.stream)
+        k.zk_planes_sum(plane.ptr, 1, out.ptr, T, W, ctx.stream)
         return out
 
 

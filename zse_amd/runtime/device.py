@@ -214,7 +214,6 @@ KERNEL_SIGNATURES = {
     "zk_sum_layer_norm": [_VP, _VP, _I, _VP, _I, _VP, _VP, _VP, _F, _VP, _I, _I, _VP],
     "zk_moe_route_ext": [_VP, _I, _VP, _VP, _I, _I, _I, _I, _VP],
     "zk_moe_experts_ext": [_VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _F, _I, _I, _VP],
-    "zk_gate_rows": [_VP, _VP, _I, _I, _I, _VP],
     "zk_cache_store": [_VP, _I, _I, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _VP],
     "zk_cache_store_temperature": [_VP, _I, _I, _I, _I, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _F, _I, _VP],
     "zk_query_temperature": [_VP, _I, _I, _VP, _I, _F, _I, _VP],
@@ -233,7 +232,7 @@ KERNEL_SIGNATURES = {
     "zk_attention_plain_kept": [_VP, _I, _VP, _VP, _VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _F, _F,
                                 _I, _I, _VP, _I, _VP, _I, _I, _I, _I, _VP],
     "zk_moe_route_best": [_VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _F, _I, _VP],
-    "zk_moe_experts_identity": [_VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _F, _I, _I, _I, _VP],
+    "zk_moe_experts_identity": [_VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _F, _I, _I, _I, _VP, _VP, _I, _VP],
     "zk_attention_plain_gated": [_VP, _I, _VP, _VP, _VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _F, _F,
                                  _I, _I, _VP, _I, _VP, _I, _I, _I, _I, _VP, _I, _VP],
     "zk_gdelta_gates": [_VP, _I, _I, _I, _VP, _VP, _VP, _VP, _VP, _I, _I, _VP],
@@ -262,7 +261,8 @@ BF16_KERNEL_SIGNATURES = {
                                 _F, _F, _I, _I, _VP, _SZ, _I, _I, _I, _I, _I, _I, _VP],
     "zk_attention_bf16_gated": [_VP, _I, _VP, _VP, _VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I,
                                 _F, _F, _I, _I, _VP, _SZ, _I, _I, _I, _I, _I, _I, _VP, _VP, _I, _VP],
-    "zk_moe_experts_grouped_identity": [_VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _F, _I, _I, _I, _VP],
+    "zk_moe_experts_grouped_identity": [_VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _F, _I, _I, _I, _VP,
+                                        _VP, _I, _VP],
     "zk_gdelta_chunked": [_VP, _I, _I, _I, _VP, _I, _VP, _VP, _VP, _VP, _I, _I, _VP, _VP, _VP, _VP, _VP, _VP, _SZ, _I, _I, _I, _I,
                           _I, _F, _VP],
     "zk_gdelta_token": [_VP, _I, _I, _I, _VP, _I, _VP, _VP, _VP, _VP, _I, _I, _VP, _VP, _VP, _VP, _I, _I, _I, _F, _VP],
