@@ -395,8 +395,8 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(const __bf16* __restri
   __shared__ int tile_e, tile_row, tile_end;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   if (wave == 0) {
-    // the blockIdx.x-th tile of rows, counting each expert's rows in whole tiles, 64 experts a turn
-    int left = blockIdx.x;
+    // the blockIdx.y-th tile of rows, counting each expert's rows in whole tiles, 64 experts a turn
+    int left = blockIdx.y;
     bool found = false;
     for (int e0 = 0; e0 < E && !found; e0 += 64) {
       const int e = e0 + lane;
@@ -422,7 +422,7 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(const __bf16* __restri
   __syncthreads();
   if (tile_row < 0) return;
   const int e = tile_e, row0 = tile_row, rows = min(TM, tile_end - tile_row);
-  const int n0 = blockIdx.y * COLS;
+  const int n0 = blockIdx.x * COLS;
   const int wm = (wave & 1) * (TM / 2), wn = (wave >> 1) * 32;
   const __bf16* Be = B + (size_t)e * (MODE == 0 ? 2 : 1) * N * K;
   // the thread's pieces: their rows' beginnings, their place in a step of TK channels and in local memory
@@ -521,7 +521,7 @@ static int launch_grouped(const void* A, const int* order, int top, const void* 
     raised = true;
   }
   constexpr int cols = MODE == 0 ? 64 : NB * 64;
-  const dim3 grid((pairs + TM - 1) / TM + E, (N + cols - 1) / cols);       // each expert may end in a tile that is not full
+  const dim3 grid((N + cols - 1) / cols, (pairs + TM - 1) / TM + E);       // each expert may end in a tile that is not full
   moe_grouped_kernel<MODE, TM, NB, TK, DEPTH><<<grid, 256, lds, st>>>((const __bf16*)A, order, top, (const __bf16*)B, first, E, N, K,
                                                                       (__bf16*)y, out_rows, limit, act);
   return zk_launch_status("zk_moe_experts_grouped");
@@ -691,7 +691,7 @@ int zk_moe_experts_grouped_identity(const void* x, const int* ids, const float* 
   const bool few = pairs <= 32 * E;
   int rc;
 #define ZK_GROUPED(MODE, ...) (few ? launch_grouped<MODE, 64, MODE == 0 ? 2 : 1, 128, 2>(__VA_ARGS__) \
-                                   : launch_grouped<MODE, 128, 2, 64, 1>(__VA_ARGS__))
+                                   : launch_grouped<MODE, 128, 2, 64, 2>(__VA_ARGS__))
   if (act == MOE_NO_GATE) rc = ZK_GROUPED(2, in, map, top, w_gu, first, pairs, E, F, W, y, nullptr, limit, act, st);
   else rc = ZK_GROUPED(0, in, map, top, w_gu, first, pairs, E, F, W, y, nullptr, limit, act, st);
   if (rc) return rc;
