@@ -299,8 +299,7 @@ def test_sinks_and_gates_that_differ_from_head_to_head(tmp_path, sizes):
 # ---------------------------------------------------------------- experts
 @pytest.mark.parametrize("W,ff", [(64, 32), (36, 20)])
 def test_identity_experts_groups_and_the_shared_experts_gate(tmp_path, W, ff):
-    """Steps of many tokens take the grouped products in bfloat16 where the width allows it, steps of few
-    the row-by-row kernels.  Left out, each of the mechanisms moves most rows by much."""
+    """In bfloat16 through the grouped products where the width allows it, else row by row.  Left out, each of the mechanisms moves most rows by much."""
     cfg = config([layer(heads=1, kv_heads=1, dim=16, window=4, mlp=moe(7, 3, ff, 24, identity=2, scale=2.0, groups=(3, 2)))], vocab=90, width=W, scale=1.5)
     w = random_weights(cfg, 12)
     w["l0.mlp.router"] = round16(w["l0.mlp.router"] * 2.0)

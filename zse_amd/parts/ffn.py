@@ -115,15 +115,11 @@ class RoutedMLP(Part):
     to choose from may stand for identity experts, which have no weights and give their input back),
     the chosen scores as weights on the experts' inputs or on their outputs, the experts' results
     added in the order they were chosen, a shared layer on top (optionally times the sigmoid of a
-    number a token, whose row rides below the router's in one product).  Steps of few tokens read each chosen expert's rows once per (token, choice); steps of
-    many tokens sort the pairs by expert on the device and run a grouped matrix-core product.
+    number a token, whose row rides below the router's in one product).  In bfloat16 the (token, choice) pairs are sorted by
+    expert on the device and a grouped matrix-core product runs over each expert's rows, whatever their number; in
+    32-bit, and where a width is no multiple of eight, each chosen expert's rows are read once per pair.
     Nothing comes back to the host, so steps are captured and written down like any other."""
     graph_safe = True
-    GROUPED_FROM = 64          # (token, choice) pairs from which the grouped product is used (bfloat16)
-    # experts of 2M weights a matrix and more: from 16 pairs on (two tokens an expert re-read its rows
-    # row by row; measured at 8 requests, 2 of 8 experts: 1.26 -> 1.20 ms a step at 2048 x 2048,
-    # 1.51 -> 1.14 ms at 4096 x 3584, but 0.72 -> 0.76 ms at 1024 x 1024)
-    GROUPED_WIDE_FROM, WIDE = 16, 2 << 20
 
     def __init__(self, spec):
         s = self.spec = spec
@@ -220,8 +216,9 @@ class RoutedMLP(Part):
             gate = logits.ptr + n * 4 if self.shared_gate else None
         plane = ctx.alloc((1, T, W), F32)
         y = ctx.alloc((T * top, F))
-        enough = T * top >= (self.GROUPED_WIDE_FROM if W * F >= self.WIDE else self.GROUPED_FROM)
-        grouped = (ctx.dtype == BF16 and ctx.tuned and enough and W % 8 == 0 and F % 8 == 0 and x.ptr % 16 == 0
+        # (measured with six layers of 8 experts, 2 a token: 0.87 -> 0.66 ms a decode step of one request at
+        # 2048 x 2048, 0.51 -> 0.46 at 1024 x 1024, and more with more requests)
+        grouped = (ctx.dtype == BF16 and ctx.tuned and W % 8 == 0 and F % 8 == 0 and x.ptr % 16 == 0
                    and k.has("zk_moe_experts_grouped_identity"))
         if grouped:
             work = ctx.alloc((n + 1 + 2 * T * top,), I32)
