@@ -621,7 +621,9 @@ class Runtime:
 
     def zero_(self, t: Tensor):
         nbytes = (t.nbytes + 3) // 4 * 4
-        self.kernels(F32).zk_zero(t.ptr, nbytes, self.stream)
+        # any library that is loaded already: a run of one storage type needs (and builds) that one alone
+        k = next(iter(self._kernels.values()), None) or self.kernels(F32)
+        k.zk_zero(t.ptr, nbytes, self.stream)
 
     def pinned(self, nbytes: int) -> PinnedBuffer:
         return PinnedBuffer(self, nbytes)
